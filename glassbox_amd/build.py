@@ -52,6 +52,8 @@ LIBRARIES: Dict[str, tuple] = {
     "moe": ("hip", ["hip/moe.hip"], ["hip/common.h"]),
     "headmix": ("hip", ["hip/headmix.hip"], ["hip/common.h"]),
     "tanhmix": ("hip", ["hip/tanhmix.hip"], ["hip/common.h"]),
+    "groupmix": ("hip", ["hip/groupmix.hip"], ["hip/common.h"]),
+    "latent": ("hip", ["hip/latent.hip"], ["hip/common.h"]),
 }
 
 _lock = threading.Lock()

@@ -1880,10 +1880,12 @@ extern "C" int gb_gemm_bf16_glu(const void* a, int lda, const void* w, int ldw, 
 // Products of groups of rows, each group with a W of its own (the tiled kernel's GROUPED form): `map` holds three
 // numbers for each of `tiles` row tiles of `tile_rows` (64 or 128) rows, as a kernel on the device laid them out; a
 // group's W starts w_stride elements behind the one before.  Epilogue 0 stores (bfloat16 or float32), 2 forms
-// silu(gate) * up from the N / 2 gate rows of a group and the up rows up_off rows behind them.
+// silu(gate) * up, or the clamped unit (limit, alpha, plus: see Glu), from the N / 2 gate rows of a group and the up rows
+// up_off rows behind them.
 extern "C" int gb_gemm_bf16_grouped(const void* a, int lda, const int32_t* rows, const void* w, int ldw, long long w_stride,
                                     int up_off, void* c, int ldc, int c_dtype, const int32_t* map, int tiles, int tile_rows,
-                                    int N, int K, int epilogue, hipStream_t stream) {
+                                    int N, int K, int epilogue, float limit, float alpha, float plus, hipStream_t stream) {
+  GB_REQUIRE(limit > 0.f, "gemm_bf16_grouped: the unit's limit must be positive");
   GB_REQUIRE(tiles >= 0 && N > 0 && K > 0 && (tile_rows == 64 || tile_rows == 128), "gemm_bf16_grouped: bad sizes tiles=%d of %d rows, N=%d K=%d",
              tiles, tile_rows, N, K);
   GB_REQUIRE(K % 8 == 0 && ldw % 8 == 0 && lda % 8 == 0 && w_stride % 8 == 0 && lda >= K && ldw >= K,
@@ -1903,7 +1905,7 @@ extern "C" int gb_gemm_bf16_grouped(const void* a, int lda, const int32_t* rows,
   const bool kfull = K % TBK == 0;
 #define GB_G(WM, EPI, CT, FULL)                                                                                              \
   if (tile_rows == 64 * WM && epilogue == EPI && kfull == FULL && (EPI == EPI_SILU_MUL || (c_dtype == kF32) == std::is_same_v<CT, float>)) \
-    hipLaunchKernelGGL((gemm_tiled_kernel<WM, 2, 1, EPI, FULL, CT, true>), grid, block, 0, stream, A, lda, W, ldw, (CT*)c, ldc, 0, N, K, 0, grp, Glu{});
+    hipLaunchKernelGGL((gemm_tiled_kernel<WM, 2, 1, EPI, FULL, CT, true>), grid, block, 0, stream, A, lda, W, ldw, (CT*)c, ldc, 0, N, K, 0, grp, Glu{limit, alpha, plus});
 #define GB_GG(WM, FULL) GB_G(WM, EPI_SILU_MUL, bf16, FULL) GB_G(WM, EPI_STORE, float, FULL) GB_G(WM, EPI_STORE, bf16, FULL)
   GB_GG(1, true) GB_GG(1, false) GB_GG(2, true) GB_GG(2, false)
 #undef GB_GG

@@ -1,0 +1,670 @@
+// Attention whose cache holds one latent row c of R channels a token instead of every head's key and value.  A head's key
+// is W_uk c and its value W_uv c, so
+//   score = q . (W_uk c) = (W_uk^T q) . c          and          sum_j p_j W_uv c_j = W_uv (sum_j p_j c_j) :
+// a token that is decoded alone takes its queries into the latents' space, attends to the latents themselves (each is read
+// once for all heads), and takes the sums through W_uv.  The tokens of a prompt portion, of which there are many for each
+// key, get the keys and values of their request's whole context expanded into scratch pages instead, and go through the
+// ordinary attention kernels.
+//
+//   latent_store    the RMS norm of a latent row and its way into the pages: [page][R / 8][slot][8] as a key head of R columns
+//   latent_absorb   q' [n, H * R] = W_uk^T q, head by head
+//   latent_decode   partial softmax sums of q' over a chunk of the context's latents, one workgroup a (chunk, 16 or 32 heads,
+//                   token); latent_decode_plain the same for any sizes and types, a workgroup a (chunk, token, head)
+//   latent_finish   the chunks' partial results added in their order, with the head's sink; W_uv; the sigmoid gate
+//   latent_tables   the pages that the portions of a step expand into: one scratch page for each page of their contexts
+//   latent_gather   the latents of those contexts as rows, zeros behind a context's end
+//   latent_expand   rows [key heads | value heads] into the scratch pages (keys in pieces, values transposed)
+//
+// Scores and softmax are 32-bit and in units of log2: a weight is 2^(score * log2(e) - max).
+#include "common.h"
+
+using namespace gb;
+
+GB_DEFINE_LAST_ERROR
+
+namespace {
+
+constexpr float kLog2e = 1.4426950408889634f;
+constexpr int kMaxRank = 2048;      // latents that the plain kernel and the last pass keep in LDS
+constexpr int kMaxSplits = 256;     // chunks of a context that the last pass adds
+
+__device__ __forceinline__ bf16x8 load8(const bf16* p) { return *reinterpret_cast<const bf16x8*>(p); }
+__device__ __forceinline__ bf16x8 load8_once(const bf16* p) { return __builtin_nontemporal_load(reinterpret_cast<const bf16x8*>(p)); }
+__device__ __forceinline__ bf16x8 zero8() {
+  bf16x8 z;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) z[i] = (bf16)0.f;
+  return z;
+}
+inline bool words16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }
+inline bool grid_fits(long long count, int per_block) { return (count + per_block - 1) / per_block < (1ll << 31); }
+
+// ------------------------------------------------------------------------------------------------ latent_store
+// A wave a row.
+template <typename T>
+__global__ __launch_bounds__(256) void latent_store_kernel(const T* __restrict__ in, int ld, const float* __restrict__ gamma, float eps,
+                                                           const int32_t* __restrict__ slots, T* __restrict__ pages, int page_size,
+                                                           int n, int R, int words) {
+  const int t = blockIdx.x * 4 + threadIdx.x / kWave, lane = threadIdx.x % kWave;
+  if (t >= n) return;
+  const T* row = in + (size_t)t * ld;
+  const int slot = slots[t];
+  T* page = pages + (size_t)(slot / page_size) * page_size * R;
+  const int at = slot % page_size;
+  float ss = 0.f;
+  if constexpr (std::is_same<T, bf16>::value) {
+    if (words) {   // rows of whole 16-byte words: a word is a piece
+      for (int p = lane; p < R / 8; p += kWave) {
+        const bf16x8 v = load8(row + 8 * p);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) ss = fmaf((float)v[e], (float)v[e], ss);
+      }
+      ss = wave_sum(ss);
+      const float r = 1.0f / sqrtf(ss / (float)R + eps);
+      for (int p = lane; p < R / 8; p += kWave) {
+        bf16x8 v = load8(row + 8 * p);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] = (bf16)((float)v[e] * r * gamma[8 * p + e]);
+        *reinterpret_cast<bf16x8*>(page + ((size_t)p * page_size + at) * 8) = v;
+      }
+      return;
+    }
+  }
+  for (int c = lane; c < R; c += kWave) ss = fmaf(to_f(row[c]), to_f(row[c]), ss);
+  ss = wave_sum(ss);
+  const float r = 1.0f / sqrtf(ss / (float)R + eps);
+  const int piece = key_piece(R);
+  for (int c = lane; c < R; c += kWave) page[key_offset(at, c, page_size, piece)] = from_f<T>(to_f(row[c]) * r * gamma[c]);
+}
+
+// ------------------------------------------------------------------------------------------------ latent_absorb
+// A wave a (64 latent channels, head, 16 tokens): D[channel][token], A = rows of W_uk^T ([H][R][hc], 16 bytes a lane), B =
+// the tokens' queries.
+__global__ __launch_bounds__(64) void latent_absorb_kernel(const bf16* __restrict__ q, int ldq, const bf16* __restrict__ uk_t, int hc,
+                                                           bf16* __restrict__ out, int n, int H, int R) {
+  const int h = blockIdx.y, r0 = blockIdx.x * 64, t0 = blockIdx.z * 16;
+  const int lane = threadIdx.x, j = lane & 15, c = lane >> 4;
+  const int tok = t0 + j;
+  f32x4 acc[4];
+#pragma unroll
+  for (int b = 0; b < 4; ++b) acc[b] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int k = 0; k < hc; k += 32) {
+    const int k0 = k + 8 * c;
+    const bf16x8 qf = (tok < n && k0 < hc) ? load8(q + (size_t)tok * ldq + (size_t)h * hc + k0) : zero8();
+#pragma unroll
+    for (int b = 0; b < 4; ++b) {
+      const int r = r0 + 16 * b + j;
+      const bf16x8 wf = (r < R && k0 < hc) ? load8(uk_t + ((size_t)h * R + r) * hc + k0) : zero8();
+      acc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, qf, acc[b], 0, 0, 0);
+    }
+  }
+  if (tok >= n) return;
+#pragma unroll
+  for (int b = 0; b < 4; ++b) {
+    const int r = r0 + 16 * b + 4 * c;
+    if (r >= R) continue;   // (R is a multiple of 8)
+    bf16x4 o;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) o[e] = (bf16)acc[b][e];
+    *reinterpret_cast<bf16x4*>(out + ((size_t)tok * H + h) * R + r) = o;
+  }
+}
+
+// A thread a (token, head, channel): uk [H * hc, R], the first dim rows of a head.
+template <typename T>
+__global__ void latent_absorb_plain_kernel(const T* __restrict__ q, int ldq, const T* __restrict__ uk, int hc, int dim, T* __restrict__ out,
+                                           long long count, int H, int R) {
+  const long long idx = (long long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (idx >= count) return;
+  const int r = (int)(idx % R), h = (int)(idx / R % H);
+  const long long t = idx / R / H;
+  const T* qr = q + (size_t)t * ldq + (size_t)h * hc;
+  const T* w = uk + (size_t)h * hc * R + r;
+  float acc = 0.f;
+  for (int d = 0; d < dim; ++d) acc = fmaf(to_f(qr[d]), to_f(w[(size_t)d * R]), acc);
+  out[idx] = from_f<T>(acc);
+}
+
+// ------------------------------------------------------------------------------------------------ latent_decode
+// Four waves; a step takes 64 latents of the context.  Each wave reads 16 of them from their page straight into MFMA operands
+// (lane (j, c): key j, channels 32 ks + 8 c .. + 7, as the pages' pieces lie), forms the scores of its keys for all columns
+// (a column is a head), and leaves scores and latents in LDS.  Then every wave takes part of the channels of the sums: per 32
+// keys it reads 8 keys x 8 channels a lane and turns them in registers (a pair of words gives two channels' pairs of keys),
+// which makes eight operands of 16 channels, one of each run of eight; the columns' running maximum is formed by each wave for
+// itself, from the same scores in the same order.  Two buffers: one barrier a step.
+//   S^T[key, col]     A = 16 keys x 32 channels,       B = 32 channels x 16 columns (the queries, in registers)
+//   O^T[chan, col]    A = 16 channels x 32 keys,       B = 32 keys x 16 columns (the weights, as the lanes form them)
+// KS: k-steps of 32 channels that hold R; CT: tiles of 16 columns.
+template <int KS, int CT>
+__global__ __launch_bounds__(256, 1) void latent_decode_kernel(const bf16* __restrict__ q, const bf16* __restrict__ pages,
+                                                               const int32_t* __restrict__ tables, int table_stride,
+                                                               const int32_t* __restrict__ positions, int H, int R, int P, float scale2,
+                                                               int chunk, int splits, float* __restrict__ ws_acc,
+                                                               float* __restrict__ ws_ml) {
+  constexpr int ROW = KS * 32 + 8;          // a latent in LDS, with 16 bytes between rows so that 16 rows' words spread over the banks
+  constexpr int SROW = 68;                  // a column's 64 scores
+  constexpr int NB = KS / 4;                // blocks of 128 channels
+  constexpr int UNITS = NB * CT, UPW = (UNITS + 3) / 4;   // (block, column tile) pairs, and how many a wave takes
+  static_assert(UPW == 1 || NB == 4, "a wave's pairs share their block");
+  __shared__ __align__(16) bf16 cbuf[2][64 * ROW];
+  __shared__ __align__(16) float sbuf[2][CT * 16 * SROW];
+  const int row = blockIdx.z, hg = blockIdx.y, split = blockIdx.x;
+  const int pos = positions[row];
+  const int c0 = split * chunk;
+  if (c0 > pos) return;                     // the chunk holds no key of the request (the whole workgroup)
+  const int last = min(c0 + chunk - 1, pos);
+  const int lane = threadIdx.x & 63, j = lane & 15, c = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int32_t* table = tables + (size_t)row * table_stride;
+
+  bf16x8 kf[KS];
+  auto load_tile = [&](int kb) {
+    const int key0 = kb + wave * 16;        // 16 keys in a row lie in one page
+    const bool valid = key0 + j <= last;
+    const int page = key0 <= last ? table[key0 / P] : 0;
+    const bf16* b = pages + (size_t)page * P * R + (size_t)(key0 % P + j) * 8;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      const int piece = ks * 4 + c;
+      kf[ks] = (valid && piece * 8 < R) ? load8_once(b + (size_t)piece * P * 8) : zero8();
+    }
+  };
+  load_tile(c0);
+
+  bf16x8 qf[CT][KS];
+#pragma unroll
+  for (int ct = 0; ct < CT; ++ct) {
+    const int head = (hg * CT + ct) * 16 + j;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      const int ch = ks * 32 + 8 * c;
+      qf[ct][ks] = (head < H && ch < R) ? load8(q + ((size_t)row * H + head) * R + ch) : zero8();
+    }
+  }
+  f32x4 acc[UPW][8];
+  float m[UPW], l[UPW];
+#pragma unroll
+  for (int u = 0; u < UPW; ++u) {
+    m[u] = -INFINITY;
+    l[u] = 0.f;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) acc[u][i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  }
+  const int block = wave % NB;              // this wave's channels: pieces 16 block .. 16 block + 15
+
+  int buf = 0;
+  for (int kb = c0; kb <= last; kb += 64, buf ^= 1) {
+    bf16* cb = cbuf[buf];
+    float* sb = sbuf[buf];
+#pragma unroll
+    for (int ct = 0; ct < CT; ++ct) {
+      f32x4 s = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks) s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[ks], qf[ct][ks], s, 0, 0, 0);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) s[r] = kb + wave * 16 + 4 * c + r <= last ? s[r] * scale2 : -INFINITY;
+      *reinterpret_cast<f32x4*>(&sb[(ct * 16 + j) * SROW + wave * 16 + 4 * c]) = s;
+    }
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) *reinterpret_cast<bf16x8*>(&cb[(wave * 16 + j) * ROW + (ks * 4 + c) * 8]) = kf[ks];
+    if (kb + 64 <= last) load_tile(kb + 64);
+    // what this wave wrote is in LDS, and every wave is past its reads of this buffer (two steps ago); the loads on their way
+    // go on
+    asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+    if (wave < UNITS) {
+      bf16x8 pf[UPW][2];
+#pragma unroll
+      for (int u = 0; u < UPW; ++u) {
+        const int ct = (wave + 4 * u) / NB;
+        float sv[2][8];
+        float mx = -INFINITY;
+#pragma unroll
+        for (int g = 0; g < 2; ++g) {
+          const float* sp = &sb[(ct * 16 + j) * SROW + 32 * g + 8 * c];
+          const f32x4 a = *reinterpret_cast<const f32x4*>(sp), b = *reinterpret_cast<const f32x4*>(sp + 4);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            sv[g][e] = a[e];
+            sv[g][4 + e] = b[e];
+            mx = fmaxf(mx, fmaxf(a[e], b[e]));
+          }
+        }
+        mx = fmaxf(mx, __shfl_xor(mx, 16, kWave));
+        mx = fmaxf(mx, __shfl_xor(mx, 32, kWave));
+        const float m_new = fmaxf(m[u], mx);   // (a step holds at least one key: finite)
+        const float alpha = __builtin_amdgcn_exp2f(m[u] - m_new);
+        float sum = 0.f;
+#pragma unroll
+        for (int g = 0; g < 2; ++g)
+#pragma unroll
+          for (int e = 0; e < 8; ++e) {
+            const float w = __builtin_amdgcn_exp2f(sv[g][e] - m_new);
+            sum += w;
+            pf[u][g][e] = (bf16)w;
+          }
+        l[u] = l[u] * alpha + sum;
+        m[u] = m_new;
+        if (__any(alpha != 1.f)) {
+#pragma unroll
+          for (int i = 0; i < 8; ++i)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) acc[u][i][r] *= alpha;
+        }
+      }
+#pragma unroll
+      for (int g = 0; g < 2; ++g) {
+        uint32_t in[8][4];   // key 32 g + 8 c + e, channels 8 piece .. + 7
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          const uint4 v = *reinterpret_cast<const uint4*>(&cb[(32 * g + 8 * c + e) * ROW + (block * 16 + j) * 8]);
+          in[e][0] = v.x, in[e][1] = v.y, in[e][2] = v.z, in[e][3] = v.w;
+        }
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          union {
+            uint32_t w[4];
+            bf16x8 v;
+          } af;   // channel 8 piece + i, keys 8 c .. 8 c + 7
+#pragma unroll
+          for (int k = 0; k < 4; ++k)
+            af.w[k] = __builtin_amdgcn_perm(in[2 * k + 1][i / 2], in[2 * k][i / 2], (i & 1) ? 0x07060302u : 0x05040100u);
+#pragma unroll
+          for (int u = 0; u < UPW; ++u) acc[u][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(af.v, pf[u][g], acc[u][i], 0, 0, 0);
+        }
+      }
+    }
+  }
+  if (wave >= UNITS) return;
+#pragma unroll
+  for (int u = 0; u < UPW; ++u) {
+    const int ct = (wave + 4 * u) / NB, head = (hg * CT + ct) * 16 + j;
+    float total = l[u] + __shfl_xor(l[u], 16, kWave);
+    total += __shfl_xor(total, 32, kWave);
+    if (head >= H) continue;
+    const size_t cell = ((size_t)row * H + head) * splits + split;
+    if (block == 0 && c == 0) {
+      ws_ml[cell * 2] = m[u];
+      ws_ml[cell * 2 + 1] = total;
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int ch = (block * 16 + 4 * c + r) * 8;
+      if (ch >= R) continue;
+      f32x4 a, b;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) a[e] = acc[u][e][r], b[e] = acc[u][4 + e][r];
+      *reinterpret_cast<f32x4*>(ws_acc + cell * R + ch) = a;
+      *reinterpret_cast<f32x4*>(ws_acc + cell * R + ch + 4) = b;
+    }
+  }
+}
+
+// Any sizes and types: 256 threads, a thread a key for the scores and a thread a channel (and every 256th after it) for the sums.
+template <typename T>
+__global__ __launch_bounds__(256) void latent_decode_plain_kernel(const T* __restrict__ q, const T* __restrict__ pages,
+                                                                  const int32_t* __restrict__ tables, int table_stride,
+                                                                  const int32_t* __restrict__ positions,
+                                                                  const int32_t* __restrict__ tok_seq, int H, int R, int P,
+                                                                  float scale2, int chunk, int splits, float* __restrict__ ws_acc,
+                                                                  float* __restrict__ ws_ml) {
+  extern __shared__ float smem[];
+  float* qs = smem;            // [R]
+  float* es = smem + R;        // [256]
+  float* scratch = es + 256;   // [17]
+  const int t = blockIdx.y / H, h = blockIdx.y % H, split = blockIdx.x, tid = threadIdx.x;
+  const int pos = positions[t], c0 = split * chunk;
+  if (c0 > pos) return;
+  const int last = min(c0 + chunk - 1, pos);
+  const int32_t* table = tables + (size_t)tok_seq[t] * table_stride;
+  const int piece = key_piece(R);
+  for (int r = tid; r < R; r += 256) qs[r] = to_f(q[((size_t)t * H + h) * R + r]);
+  __syncthreads();
+  float m = -INFINITY, l = 0.f, acc[kMaxRank / 256];
+#pragma unroll
+  for (int i = 0; i < kMaxRank / 256; ++i) acc[i] = 0.f;
+  for (int k0 = c0; k0 <= last; k0 += 256) {
+    const int key = k0 + tid;
+    float s = -INFINITY;
+    if (key <= last) {
+      const T* page = pages + (size_t)table[key / P] * P * R;
+      float dot = 0.f;
+      for (int r0 = 0; r0 < R; r0 += piece) {
+        const T* kr = page + key_offset(key % P, r0, P, piece);
+        for (int e = 0; e < piece; ++e) dot = fmaf(qs[r0 + e], to_f(kr[e]), dot);
+      }
+      s = dot * scale2;
+    }
+    const float m_new = fmaxf(m, block_max(s, scratch));
+    const float e = key <= last ? exp2f(s - m_new) : 0.f;
+    es[tid] = e;
+    const float alpha = exp2f(m - m_new);
+    l = fmaf(l, alpha, block_sum(e, scratch));   // (also orders the writes of es before the reads below)
+    m = m_new;
+#pragma unroll
+    for (int i = 0; i < kMaxRank / 256; ++i) acc[i] *= alpha;
+    const int top = min(k0 + 255, last);
+    for (int k = k0; k <= top; ++k) {
+      const T* page = pages + (size_t)table[k / P] * P * R;
+      const float w = es[k - k0];
+#pragma unroll
+      for (int i = 0; i < kMaxRank / 256; ++i) {
+        const int r = tid + 256 * i;
+        if (r < R) acc[i] = fmaf(w, to_f(page[key_offset(k % P, r, P, piece)]), acc[i]);
+      }
+    }
+    __syncthreads();   // es is written again
+  }
+  const size_t cell = ((size_t)t * H + h) * splits + split;
+  if (tid == 0) {
+    ws_ml[cell * 2] = m;
+    ws_ml[cell * 2 + 1] = l;
+  }
+#pragma unroll
+  for (int i = 0; i < kMaxRank / 256; ++i)
+    if (tid + 256 * i < R) ws_acc[cell * R + tid + 256 * i] = acc[i];
+}
+
+// ------------------------------------------------------------------------------------------------ latent_finish
+// A workgroup a (token, head): uv [H * hc, R] (the first vdim rows of a head), gate [n, ldg] (or nullptr: none).
+template <typename T>
+__global__ __launch_bounds__(256) void latent_finish_kernel(const float* __restrict__ ws_acc, const float* __restrict__ ws_ml,
+                                                            const int32_t* __restrict__ positions, int chunk, int splits,
+                                                            const float* __restrict__ sinks, const T* __restrict__ uv, int hc,
+                                                            const T* __restrict__ gate, int ldg, T* __restrict__ out, int ldo, int H,
+                                                            int R, int vdim, int words) {
+  __shared__ float weight[kMaxSplits];
+  __shared__ __align__(16) float o[kMaxRank];
+  __shared__ float scratch[17];
+  const int t = blockIdx.x / H, h = blockIdx.x % H, tid = threadIdx.x;
+  const int count = min(positions[t] / chunk + 1, splits);   // chunks that hold keys
+  const size_t cell0 = ((size_t)t * H + h) * splits;
+  const float mine = tid < count ? ws_ml[(cell0 + tid) * 2] : -INFINITY, mine_l = tid < count ? ws_ml[(cell0 + tid) * 2 + 1] : 0.f;
+  const float top = block_max(mine, scratch);
+  const float f = tid < count ? exp2f(mine - top) : 0.f;
+  weight[tid] = f;
+  float total = block_sum(f * mine_l, scratch);   // (also orders the writes of weight before the reads below)
+  if (sinks) total += exp2f(fmaf(sinks[h], kLog2e, -top));
+  const float inv = 1.0f / total;
+  for (int r = tid; r < R; r += 256) {
+    float s = 0.f;
+#pragma unroll 8
+    for (int k = 0; k < count; ++k) s = fmaf(ws_acc[(cell0 + k) * R + r], weight[k], s);
+    o[r] = s * inv;
+  }
+  __syncthreads();
+  const int g16 = tid / 16, l16 = tid % 16;   // sixteen lanes a channel of the value
+  for (int d = g16; d < vdim; d += 16) {
+    const T* w = uv + ((size_t)h * hc + d) * R;
+    float s = 0.f;
+    bool done = false;
+    if constexpr (std::is_same<T, bf16>::value) {
+      if (words) {
+        for (int p = l16; p < R / 8; p += 16) {
+          const bf16x8 v = load8(w + 8 * p);
+          const f32x4 a = *reinterpret_cast<const f32x4*>(&o[8 * p]), b = *reinterpret_cast<const f32x4*>(&o[8 * p + 4]);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) s = fmaf((float)v[e], a[e], s);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) s = fmaf((float)v[4 + e], b[e], s);
+        }
+        done = true;
+      }
+    }
+    if (!done)
+      for (int r = l16; r < R; r += 16) s = fmaf(to_f(w[r]), o[r], s);
+#pragma unroll
+    for (int off = 8; off >= 1; off >>= 1) s += __shfl_xor(s, off, 16);
+    if (l16 == 0) {
+      if (gate) s = s / (1.0f + expf(-to_f(gate[(size_t)t * ldg + (size_t)h * vdim + d])));
+      out[(size_t)t * ldo + (size_t)h * vdim + d] = from_f<T>(s);
+    }
+  }
+}
+
+// ------------------------------------------------------------------------------------------------ scratch pages of portions
+// Requests first .. first + count - 1 of the step; a request's context is pos0 + q_len tokens.  table [*, stride] (rows by
+// request) receives the scratch pages in order, source [total][2] the (request, page of its context) behind each.
+__global__ __launch_bounds__(256) void latent_tables_kernel(const int32_t* __restrict__ q_len, const int32_t* __restrict__ pos0, int first,
+                                                            int count, int P, int32_t* __restrict__ table, int stride,
+                                                            int32_t* __restrict__ source, int total) {
+  int base = 0;
+  for (int s = first; s < first + count; ++s) {
+    const int pages = (pos0[s] + q_len[s] + P - 1) / P;
+    for (int i = threadIdx.x; i < pages && i < stride && base + i < total; i += 256) {
+      table[(size_t)s * stride + i] = base + i;
+      source[2 * (base + i)] = s;
+      source[2 * (base + i) + 1] = i;
+    }
+    base += pages;
+  }
+}
+
+// A workgroup a scratch page: its tokens' latents as rows [P][R], zeros behind the context's end.
+template <typename T>
+__global__ __launch_bounds__(256) void latent_gather_kernel(const T* __restrict__ pages, const int32_t* __restrict__ tables,
+                                                            int table_stride, const int32_t* __restrict__ source,
+                                                            const int32_t* __restrict__ q_len, const int32_t* __restrict__ pos0, int P,
+                                                            int R, T* __restrict__ out) {
+  const int s = source[2 * blockIdx.x], i = source[2 * blockIdx.x + 1];
+  const int valid = min(P, pos0[s] + q_len[s] - i * P);
+  const T* page = pages + (size_t)tables[(size_t)s * table_stride + i] * P * R;
+  T* rows = out + (size_t)blockIdx.x * P * R;
+  if constexpr (std::is_same<T, bf16>::value) {
+    if (R % 8 == 0) {
+      const int pieces = R / 8;
+      for (int u = threadIdx.x; u < P * pieces; u += 256) {
+        const int slot = u / pieces, p = u % pieces;
+        *reinterpret_cast<bf16x8*>(rows + (size_t)slot * R + 8 * p) = slot < valid ? load8(page + ((size_t)p * P + slot) * 8) : zero8();
+      }
+      return;
+    }
+  }
+  const int piece = key_piece(R);
+  for (int u = threadIdx.x; u < P * R; u += 256) {
+    const int slot = u / R, r = u % R;
+    rows[u] = slot < valid ? page[key_offset(slot, r, P, piece)] : from_f<T>(0.f);
+  }
+}
+
+// Rows [n][H key heads | H value heads] of hc columns; row r goes to slot r % P of scratch page r / P.  A workgroup (16 rows,
+// head): keys word by word into their pieces, values turned in LDS.
+__global__ __launch_bounds__(256) void latent_expand_words_kernel(const bf16* __restrict__ kv, int ld, bf16* __restrict__ k_pages,
+                                                                  bf16* __restrict__ v_pages, int H, int hc, int P) {
+  extern __shared__ uint32_t tile[];   // [16][hc / 2 + 1]
+  const int r0 = blockIdx.x * 16, h = blockIdx.y, page = r0 / P, slot0 = r0 % P;
+  const int words = hc / 8, pitch = hc / 2 + 1;
+  bf16* kb = k_pages + ((size_t)page * H + h) * hc * P;
+  bf16* vb = v_pages + ((size_t)page * H + h) * hc * P;
+  for (int u = threadIdx.x; u < 16 * words; u += 256) {
+    const int slot = u / words, p = u % words;
+    const uint4 v = *reinterpret_cast<const uint4*>(kv + (size_t)(r0 + slot) * ld + (size_t)(H + h) * hc + 8 * p);
+    uint32_t* d = tile + slot * pitch + 4 * p;
+    d[0] = v.x, d[1] = v.y, d[2] = v.z, d[3] = v.w;
+  }
+  for (int u = threadIdx.x; u < 16 * words; u += 256) {
+    const int p = u / 16, slot = u % 16;
+    *reinterpret_cast<bf16x8*>(kb + ((size_t)p * P + slot0 + slot) * 8) = load8(kv + (size_t)(r0 + slot) * ld + (size_t)h * hc + 8 * p);
+  }
+  __syncthreads();
+  for (int u = threadIdx.x; u < hc * 2; u += 256) {   // (channel, half of the 16 slots)
+    const int d = u / 2, s0 = (u % 2) * 8;
+    uint4 w;
+    uint32_t* wp = &w.x;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const uint32_t lo = tile[(s0 + 2 * k) * pitch + d / 2], hi = tile[(s0 + 2 * k + 1) * pitch + d / 2];
+      wp[k] = (d & 1) ? __builtin_amdgcn_perm(hi, lo, 0x07060302u) : __builtin_amdgcn_perm(hi, lo, 0x05040100u);
+    }
+    *reinterpret_cast<uint4*>(vb + (size_t)d * P + slot0 + s0) = w;
+  }
+}
+
+template <typename T>
+__global__ void latent_expand_kernel(const T* __restrict__ kv, int ld, T* __restrict__ k_pages, T* __restrict__ v_pages, int H, int hc,
+                                     int P, long long count) {
+  const long long idx = (long long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (idx >= count) return;
+  const int d = (int)(idx % hc), h = (int)(idx / hc % H);
+  const long long r = idx / hc / H;
+  const size_t base = ((size_t)(r / P) * H + h) * hc * P;
+  const int slot = (int)(r % P);
+  k_pages[base + key_offset(slot, d, P, key_piece(hc))] = kv[(size_t)r * ld + (size_t)h * hc + d];
+  v_pages[base + (size_t)d * P + slot] = kv[(size_t)r * ld + (size_t)(H + h) * hc + d];
+}
+
+}  // namespace
+
+#define GB_BY_DTYPE(dtype, what, CALL)              \
+  if (dtype == kF32) {                              \
+    typedef float TT;                               \
+    CALL;                                           \
+  } else if (dtype == kBF16) {                      \
+    typedef bf16 TT;                                \
+    CALL;                                           \
+  } else {                                          \
+    return fail(what ": unknown dtype %d", dtype);  \
+  }
+
+// in [n, ld] of `dtype`, the latent in the first R columns; pages [pages][R / piece][P][piece].
+extern "C" int gb_latent_store(const void* in, int dtype, int ld, const float* gamma, float eps, const int32_t* slots, void* pages,
+                               int page_size, int n, int R, hipStream_t stream) {
+  GB_REQUIRE(n >= 0 && R > 0 && ld >= R && page_size > 0 && in && gamma && slots && pages, "latent_store: bad sizes n=%d R=%d ld=%d", n, R, ld);
+  if (n == 0) return 0;
+  const int words = dtype == kBF16 && R % 8 == 0 && ld % 8 == 0 && words16(in) && words16(pages);
+  GB_BY_DTYPE(dtype, "latent_store",
+              hipLaunchKernelGGL(latent_store_kernel<TT>, dim3((unsigned)((n + 3) / 4)), dim3(256), 0, stream, (const TT*)in, ld, gamma,
+                                 eps, slots, (TT*)pages, page_size, n, R, words))
+  return launched("latent_store");
+}
+
+// q [n, ldq]: H heads of hc columns; uk [H * hc, R]; uk_t [H, R, hc] or nullptr (then, and in 32-bit, the plain kernel); out
+// [n, H * R].
+extern "C" int gb_latent_absorb(const void* q, int dtype, int ldq, const void* uk, const void* uk_t, int hc, int dim, void* out, int n,
+                                int H, int R, hipStream_t stream) {
+  GB_REQUIRE(n >= 0 && H > 0 && R > 0 && dim > 0 && hc >= dim && ldq >= H * hc && q && uk && out, "latent_absorb: bad sizes n=%d heads=%d R=%d dim=%d of %d", n, H, R, dim, hc);
+  if (n == 0) return 0;
+  if (dtype == kBF16 && uk_t && R % 8 == 0 && hc % 8 == 0 && ldq % 8 == 0 && words16(q) && words16(uk_t) && words16(out) && H <= 65535 && n <= 65535 * 16) {
+    const dim3 grid((unsigned)((R + 63) / 64), (unsigned)H, (unsigned)((n + 15) / 16));
+    hipLaunchKernelGGL(latent_absorb_kernel, grid, dim3(64), 0, stream, (const bf16*)q, ldq, (const bf16*)uk_t, hc, (bf16*)out, n, H, R);
+    return launched("latent_absorb");
+  }
+  const long long count = (long long)n * H * R;
+  GB_REQUIRE(grid_fits(count, 256), "latent_absorb: too many elements");
+  GB_BY_DTYPE(dtype, "latent_absorb",
+              hipLaunchKernelGGL(latent_absorb_plain_kernel<TT>, dim3((unsigned)((count + 255) / 256)), dim3(256), 0, stream, (const TT*)q,
+                                 ldq, (const TT*)uk, hc, dim, (TT*)out, count, H, R))
+  return launched("latent_absorb");
+}
+
+// Whether the matrix-core kernel takes latents of R channels in pages of P tokens.
+extern "C" int gb_latent_decode_takes(int R, int P) { return R >= 8 && R % 8 == 0 && R <= 512 && P >= 16 && P % 16 == 0; }
+
+// q [n, H * R] (row t is request t's single token for the matrix-core kernel; any rows with tok_seq for the plain one), pages as
+// gb_latent_store writes them, ws_acc [n, H, splits, R] and ws_ml [n, H, splits, 2] float32 with splits = ceil(longest context /
+// chunk); only the chunks that hold keys of a row are written.
+extern "C" int gb_latent_decode(const void* q, int dtype, const void* pages, const int32_t* tables, int table_stride,
+                                const int32_t* positions, const int32_t* tok_seq, int n, int H, int R, int P, float scale, int chunk,
+                                int splits, float* ws_acc, float* ws_ml, int plain, hipStream_t stream) {
+  GB_REQUIRE(n >= 0 && H > 0 && R > 0 && R <= kMaxRank && P > 0 && table_stride > 0, "latent_decode: bad sizes n=%d heads=%d R=%d (at most %d)", n, H, R, kMaxRank);
+  GB_REQUIRE(chunk > 0 && splits >= 1 && splits <= kMaxSplits, "latent_decode: %d chunks of a context (at most %d)", splits, kMaxSplits);
+  GB_REQUIRE(q && pages && tables && positions && ws_acc && ws_ml, "latent_decode: operands are missing");
+  if (n == 0) return 0;
+  const float scale2 = scale * kLog2e;
+  if (!plain) {
+    GB_REQUIRE(dtype == kBF16 && gb_latent_decode_takes(R, P), "latent_decode: R=%d in pages of %d goes through the plain kernel", R, P);
+    GB_REQUIRE(chunk % 64 == 0 && n <= 65535 && words16(q) && words16(pages) && words16(ws_acc), "latent_decode: chunks of whole 64 keys, aligned operands");
+    const int ct = H > 16 ? 2 : 1;
+    const dim3 grid((unsigned)splits, (unsigned)((H + 16 * ct - 1) / (16 * ct)), (unsigned)n);
+#define GB_LATENT(KS, CT)                                                                                                       \
+  if (ct == CT)                                                                                                                 \
+    hipLaunchKernelGGL((latent_decode_kernel<KS, CT>), grid, dim3(256), 0, stream, (const bf16*)q, (const bf16*)pages, tables, \
+                       table_stride, positions, H, R, P, scale2, chunk, splits, ws_acc, ws_ml);
+    if (R <= 128) {
+      GB_LATENT(4, 1) GB_LATENT(4, 2)
+    } else if (R <= 256) {
+      GB_LATENT(8, 1) GB_LATENT(8, 2)
+    } else {
+      GB_LATENT(16, 1) GB_LATENT(16, 2)
+    }
+#undef GB_LATENT
+    return launched("latent_decode");
+  }
+  GB_REQUIRE(tok_seq, "latent_decode: the plain kernel needs the rows' requests");
+  const int rows_max = 65535 / H;   // (grid.y)
+  GB_REQUIRE(rows_max >= 1, "latent_decode: %d heads", H);
+  for (int first = 0; first < n; first += rows_max) {
+    const int rows = n - first < rows_max ? n - first : rows_max;
+    const dim3 grid((unsigned)splits, (unsigned)(rows * H));
+    const size_t lds = (size_t)(R + 256 + 17) * sizeof(float);
+    GB_BY_DTYPE(dtype, "latent_decode",
+                hipLaunchKernelGGL(latent_decode_plain_kernel<TT>, grid, dim3(256), lds, stream, (const TT*)q + (size_t)first * H * R,
+                                   (const TT*)pages, tables, table_stride, positions + first, tok_seq + first, H, R, P, scale2, chunk,
+                                   splits, ws_acc + (size_t)first * H * splits * R, ws_ml + (size_t)first * H * splits * 2))
+  }
+  return launched("latent_decode (plain)");
+}
+
+// The partial results of gb_latent_decode to out [n, ldo] of `dtype`: H heads of vdim columns, gated.
+extern "C" int gb_latent_finish(const float* ws_acc, const float* ws_ml, const int32_t* positions, int chunk, int splits,
+                                const float* sinks, const void* uv, int hc, const void* gate, int ldg, void* out, int ldo, int dtype,
+                                int n, int H, int R, int vdim, hipStream_t stream) {
+  GB_REQUIRE(n >= 0 && H > 0 && R > 0 && R <= kMaxRank && vdim > 0 && hc >= vdim && ldo >= H * vdim && (!gate || ldg >= H * vdim),
+             "latent_finish: bad sizes n=%d heads=%d R=%d vdim=%d", n, H, R, vdim);
+  GB_REQUIRE(chunk > 0 && splits >= 1 && splits <= kMaxSplits && ws_acc && ws_ml && positions && uv && out, "latent_finish: %d chunks, or operands are missing", splits);
+  if (n == 0) return 0;
+  GB_REQUIRE((long long)n * H < (1ll << 31), "latent_finish: too many (token, head) pairs");
+  const int words = dtype == kBF16 && R % 8 == 0 && words16(uv);
+  GB_BY_DTYPE(dtype, "latent_finish",
+              hipLaunchKernelGGL(latent_finish_kernel<TT>, dim3((unsigned)(n * H)), dim3(256), 0, stream, ws_acc, ws_ml, positions, chunk,
+                                 splits, sinks, (const TT*)uv, hc, (const TT*)gate, ldg, (TT*)out, ldo, H, R, vdim, words))
+  return launched("latent_finish");
+}
+
+extern "C" int gb_latent_tables(const int32_t* q_len, const int32_t* pos0, int first, int count, int P, int32_t* table, int stride,
+                                int32_t* source, int total, hipStream_t stream) {
+  GB_REQUIRE(first >= 0 && count >= 0 && P > 0 && stride > 0 && total >= 0 && q_len && pos0 && table && source, "latent_tables: bad sizes");
+  if (count == 0) return 0;
+  hipLaunchKernelGGL(latent_tables_kernel, dim3(1), dim3(256), 0, stream, q_len, pos0, first, count, P, table, stride, source, total);
+  return launched("latent_tables");
+}
+
+// out [total * P, R]
+extern "C" int gb_latent_gather(const void* pages, int dtype, const int32_t* tables, int table_stride, const int32_t* source,
+                                const int32_t* q_len, const int32_t* pos0, int P, int R, int total, void* out, hipStream_t stream) {
+  GB_REQUIRE(P > 0 && R > 0 && total >= 0 && pages && tables && source && q_len && pos0 && out, "latent_gather: bad sizes");
+  GB_REQUIRE(R % 8 != 0 || (words16(pages) && words16(out)), "latent_gather: operands must be 16-byte aligned");
+  if (total == 0) return 0;
+  GB_BY_DTYPE(dtype, "latent_gather",
+              hipLaunchKernelGGL(latent_gather_kernel<TT>, dim3((unsigned)total), dim3(256), 0, stream, (const TT*)pages, tables,
+                                 table_stride, source, q_len, pos0, P, R, (TT*)out))
+  return launched("latent_gather");
+}
+
+// kv [total * P, ld]: H key heads, then H value heads, of hc columns; k_pages [total, H, hc / piece, P, piece], v_pages [total, H,
+// hc, P].
+extern "C" int gb_latent_expand(const void* kv, int dtype, int ld, void* k_pages, void* v_pages, int H, int hc, int P, int total,
+                                hipStream_t stream) {
+  GB_REQUIRE(H > 0 && hc > 0 && P > 0 && total >= 0 && ld >= 2 * H * hc && kv && k_pages && v_pages, "latent_expand: bad sizes heads=%d of %d", H, hc);
+  if (total == 0) return 0;
+  if (dtype == kBF16 && hc % 8 == 0 && P % 16 == 0 && ld % 8 == 0 && words16(kv) && words16(k_pages) && words16(v_pages) && H <= 65535) {
+    const dim3 grid((unsigned)(total * (P / 16)), (unsigned)H);
+    hipLaunchKernelGGL(latent_expand_words_kernel, grid, dim3(256), (size_t)16 * (hc / 2 + 1) * 4, stream, (const bf16*)kv, ld,
+                       (bf16*)k_pages, (bf16*)v_pages, H, hc, P);
+    return launched("latent_expand");
+  }
+  const long long count = (long long)total * P * H * hc;
+  GB_REQUIRE(grid_fits(count, 256), "latent_expand: too many elements");
+  GB_BY_DTYPE(dtype, "latent_expand",
+              hipLaunchKernelGGL(latent_expand_kernel<TT>, dim3((unsigned)((count + 255) / 256)), dim3(256), 0, stream, (const TT*)kv, ld,
+                                 (TT*)k_pages, (TT*)v_pages, H, hc, P, count))
+  return launched("latent_expand");
+}
+
+// the launches of a layer can be recorded and made again for the layers like it (common.h)
+GB_TAPED(gb_latent_store)
+GB_TAPED(gb_latent_absorb)
+GB_TAPED(gb_latent_decode)
+GB_TAPED(gb_latent_finish)
+GB_TAPED(gb_latent_tables)
+GB_TAPED(gb_latent_gather)
+GB_TAPED(gb_latent_expand)

@@ -12,7 +12,7 @@
 // `route` leaves the result in two forms: the chosen experts and their weights a token ([n, top]), and a row of E
 // weights a token with zeros for the experts not chosen (with `shared`, one more column: sigmoid of z's column E, the
 // gate of an expert that every token uses).  `gated_units` turns the stacked gate and up projections of all experts
-// into act = silu(gate) * up * weight, so that one product with the experts' down matrices side by side adds up
+// into act = silu(gate) * up * weight (or a clamped unit, see UnitOf), so that one product with the experts' down matrices side by side adds up
 // sum_e a_e y_e over the token's experts (an expert not chosen contributes exact zeros).
 //
 // With many tokens a step, the experts run on the rows that chose them alone.  `sort` puts the (token, choice) entries
@@ -33,7 +33,8 @@ namespace {
 constexpr int kPerLane = 8;   // experts a lane: up to 512 experts
 constexpr int kMaxTop = 16;
 
-// shared: 0 none, 1 a gate sigmoid(z[E]), 2 weight 1.  softmax: scores over all experts (else sigmoid of each).
+// shared: 0 none, 1 a gate sigmoid(z[E]), 2 weight 1.  softmax: 1 scores over all experts, 2 the choice by z + correction
+// and scores e^(z + correction) (with renorm: the softmax over the chosen), else sigmoid of each.
 // renorm: weights divided by the sum of the chosen scores.  groups > 0: see above.
 __global__ __launch_bounds__(4 * kWave) void route_kernel(const float* __restrict__ z, int ldz, int E,
                                                         const float* __restrict__ correction, int top, float scale,
@@ -48,7 +49,12 @@ __global__ __launch_bounds__(4 * kWave) void route_kernel(const float* __restric
   const float* row = z + (size_t)t * ldz;
   float s[kPerLane], c[kPerLane];
   float top_z = -INFINITY, denom = 0.f;
-  if (softmax) {
+  if (softmax == 2) {
+#pragma unroll
+    for (int j = 0; j < kPerLane; ++j)
+      if (lane + j * kWave < E) top_z = fmaxf(top_z, row[lane + j * kWave] + (correction ? correction[lane + j * kWave] : 0.f));
+    top_z = wave_max(top_z);
+  } else if (softmax) {
 #pragma unroll
     for (int j = 0; j < kPerLane; ++j)
       if (lane + j * kWave < E) top_z = fmaxf(top_z, row[lane + j * kWave]);
@@ -63,7 +69,10 @@ __global__ __launch_bounds__(4 * kWave) void route_kernel(const float* __restric
     const int e = lane + j * kWave;
     s[j] = 0.f;
     c[j] = -INFINITY;
-    if (e < E) {
+    if (e < E && softmax == 2) {
+      c[j] = row[e] + (correction ? correction[e] : 0.f);
+      s[j] = expf(c[j] - top_z);
+    } else if (e < E) {
       s[j] = softmax ? expf(row[e] - top_z) / denom : 1.0f / (1.0f + expf(-row[e]));
       c[j] = s[j] + (correction ? correction[e] : 0.f);
     }
@@ -156,12 +165,22 @@ __global__ __launch_bounds__(4 * kWave) void route_kernel(const float* __restric
     }
 }
 
-// act[t, j] = silu(g) * u * combine[t, expert of column j]: columns e * ff .. (e + 1) * ff - 1 are expert e's, the
+// The unit: g' = min(g, limit), u' = clamp(u, -limit, limit), g' sigmoid(alpha g') (u' + plus); as it stands here silu(g) u.
+struct UnitOf {
+  float limit = INFINITY, alpha = 1.0f, plus = 0.0f;
+  __device__ __forceinline__ float operator()(float g, float u) const {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return g / (1.0f + expf(-(alpha * g))) * (u + plus);
+  }
+};
+
+// act[t, j] = unit(g, u) * combine[t, expert of column j]: columns e * ff .. (e + 1) * ff - 1 are expert e's, the
 // columns from E * ff on the shared expert's (weight in column E of combine).  Rows of `gu`: the experts' gate columns,
 // the experts' up columns, then the shared expert's gate columns and its up columns.
 template <typename I, typename O>
 __global__ void gated_units_kernel(const I* __restrict__ gu, int ld, const float* __restrict__ combine, int cols, O* __restrict__ act,
-                                   long long count, int inter, int E, int ff) {
+                                   long long count, int inter, int E, int ff, UnitOf unit) {
   const long long idx = (long long)blockIdx.x * blockDim.x + threadIdx.x;
   if (idx >= count) return;
   const long long t = idx / inter;
@@ -173,10 +192,31 @@ __global__ void gated_units_kernel(const I* __restrict__ gu, int ld, const float
   if (w != 0.f) {
     const I* row = gu + (size_t)t * ld;
     const int at = j < routed ? j : 2 * routed + (j - routed), up = j < routed ? routed : inter - routed;
-    const float g = to_f(row[at]), u = to_f(row[at + up]);
-    y = g / (1.0f + expf(-g)) * u * w;
+    y = unit(to_f(row[at]), to_f(row[at + up])) * w;
   }
   act[idx] = from_f<O>(y);
+}
+
+// The same from 32-bit sums, four columns a thread (experts of whole groups of four columns, aligned rows).
+__global__ void gated_units_words_kernel(const float* __restrict__ gu, int ld, const float* __restrict__ combine, int cols,
+                                         bf16* __restrict__ act, long long count, int inter, int E, int ff, UnitOf unit) {
+  const long long idx = (long long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (idx >= count) return;
+  const int words = inter / 4, j = (int)(idx % words) * 4, routed = E * ff;
+  const long long t = idx / words;
+  const float w = combine[(size_t)t * cols + (j < routed ? j / ff : E)];
+  bf16x4 o;
+  if (w != 0.f) {
+    const float* row = gu + (size_t)t * ld;
+    const int at = j < routed ? j : 2 * routed + (j - routed), up = j < routed ? routed : inter - routed;
+    const f32x4 g = *reinterpret_cast<const f32x4*>(row + at), u = *reinterpret_cast<const f32x4*>(row + at + up);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) o[e] = (bf16)(unit(g[e], u[e]) * w);
+  } else {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) o[e] = (bf16)0.f;
+  }
+  *reinterpret_cast<bf16x4*>(act + (size_t)t * inter + j) = o;
 }
 
 // act[t, j] = relu(z[t, j])^2 * combine[t, expert of column j] for units without a gate half: columns
@@ -390,20 +430,28 @@ extern "C" int gb_moe_relu2_units(const void* z, int in_dtype, int ld, const flo
   return launched("moe_relu2_units");
 }
 
+// The unit's numbers: limit (INFINITY: none), alpha, plus (see UnitOf; INFINITY, 1, 0 is silu(gate) * up).
 extern "C" int gb_moe_gated_units(const void* gu, int in_dtype, int ld, const float* combine, int cols, void* act, int out_dtype,
-                                  int n, int inter, int E, int ff, hipStream_t stream) {
+                                  int n, int inter, int E, int ff, float limit, float alpha, float plus, hipStream_t stream) {
   GB_REQUIRE(n >= 0 && inter > 0 && ld >= 2 * inter && E >= 0 && ff > 0 && E * ff <= inter && cols >= E + (E * ff < inter ? 1 : 0),
              "moe_gated_units: bad sizes n=%d inter=%d experts=%d of %d cols=%d", n, inter, E, ff, cols);
+  GB_REQUIRE(limit > 0.f, "moe_gated_units: the limit must be positive");
   if (n == 0) return 0;
   const long long count = (long long)n * inter;
   GB_REQUIRE((count + 255) / 256 < (1ll << 31), "moe_gated_units: too many elements");
+  const UnitOf unit{limit, alpha, plus};
+  if (in_dtype == kF32 && out_dtype == kBF16 && inter % 4 == 0 && ff % 4 == 0 && ld % 4 == 0 && (uintptr_t)gu % 16 == 0 && (uintptr_t)act % 8 == 0) {
+    hipLaunchKernelGGL(gated_units_words_kernel, dim3((unsigned)((count / 4 + 255) / 256)), dim3(256), 0, stream, (const float*)gu, ld,
+                       combine, cols, (bf16*)act, count / 4, inter, E, ff, unit);
+    return launched("moe_gated_units");
+  }
   const dim3 grid((unsigned)((count + 255) / 256));
   if (in_dtype == kF32 && out_dtype == kF32)
-    hipLaunchKernelGGL((gated_units_kernel<float, float>), grid, dim3(256), 0, stream, (const float*)gu, ld, combine, cols, (float*)act, count, inter, E, ff);
+    hipLaunchKernelGGL((gated_units_kernel<float, float>), grid, dim3(256), 0, stream, (const float*)gu, ld, combine, cols, (float*)act, count, inter, E, ff, unit);
   else if (in_dtype == kF32 && out_dtype == kBF16)
-    hipLaunchKernelGGL((gated_units_kernel<float, bf16>), grid, dim3(256), 0, stream, (const float*)gu, ld, combine, cols, (bf16*)act, count, inter, E, ff);
+    hipLaunchKernelGGL((gated_units_kernel<float, bf16>), grid, dim3(256), 0, stream, (const float*)gu, ld, combine, cols, (bf16*)act, count, inter, E, ff, unit);
   else if (in_dtype == kBF16 && out_dtype == kBF16)
-    hipLaunchKernelGGL((gated_units_kernel<bf16, bf16>), grid, dim3(256), 0, stream, (const bf16*)gu, ld, combine, cols, (bf16*)act, count, inter, E, ff);
+    hipLaunchKernelGGL((gated_units_kernel<bf16, bf16>), grid, dim3(256), 0, stream, (const bf16*)gu, ld, combine, cols, (bf16*)act, count, inter, E, ff, unit);
   else
     return fail("moe_gated_units: no kernel for operand type %d and result type %d", in_dtype, out_dtype);
   return launched("moe_gated_units");

@@ -140,8 +140,9 @@ class Engine:
                 # write there (engine.decode_graphs)
                 shape = ops.key_pages_shape(num_pages + 1, spec.num_kv_heads, self.page_size, spec.head_dim)
                 lc.k_pages = torch.zeros(shape, dtype=self.dtype, device=self.device)
-                lc.v_pages = torch.zeros((num_pages + 1, spec.num_kv_heads, spec.head_dim, self.page_size),
-                                         dtype=self.dtype, device=self.device)   # transposed: see ops._check_pages
+                if spec.values:
+                    lc.v_pages = torch.zeros((num_pages + 1, spec.num_kv_heads, spec.head_dim, self.page_size),
+                                             dtype=self.dtype, device=self.device)   # transposed: see ops._check_pages
             if state is not None:
                 lc.state = torch.full((self.max_seqs + 1,) + tuple(state.shape), state.initial, dtype=state.dtype,
                                       device=self.device)
@@ -252,7 +253,8 @@ class Engine:
                         ops.copy_rows(lc.state, src, dst)
                 elif lc.k_pages is not None and lc.group == g:
                     ops.copy_rows(lc.k_pages, src, dst)   # copy-on-write in every layer (kv.rs:189-196)
-                    ops.copy_rows(lc.v_pages, src, dst)
+                    if lc.v_pages is not None:
+                        ops.copy_rows(lc.v_pages, src, dst)
 
     def step(self, entries: Sequence[Entry]) -> torch.Tensor:
         """Runs exactly the given tokens, as one batch, from the cache that earlier steps left.

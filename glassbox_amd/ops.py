@@ -103,15 +103,45 @@ _SIGS = {
         # att, lda, hd, gate, ldg, one gate a head, dtype, out, ldo, n, H, dv, stream
         "gb_gate_rows": [_vp, _i, _i, _vp, _i, _i, _i, _vp, _i, _i, _i, _i, _vp],
     },
-    "moe": {        # z, ldz, n, experts, correction, top, scale, shared, combine, ids, weights, stream
+    "groupmix": {
+        # table, dtype, ids, positions, turns, x, n, d, vocab, scale, copies, stream
+        "gb_embed_sinusoid": [_vp, _i, _vp, _vp, _vp, _vp, _i, _i, _i, _f, _i, _vp],
+        # x, y, slices, slice stride, hist, its stride, coef, count, out, rows, gamma, groups, eps, scales, h, its dtype,
+        # conv w, taps, state, slot stride, tok_seq, pos0, state slots, n, d, stream
+        "gb_residual_rows": [_vp, _vp, _i, C.c_longlong, _vp, C.c_longlong, _vp, _i, _vp, _vp, _vp, _i, _f, _vp, _vp, _i,
+                             _vp, _i, _vp, C.c_longlong, _vp, _vp, _vp, _i, _i, _vp],
+        # x, scales, groups, gamma, w, taps, state, slot stride, tok_seq, q_start, pos0, state slots, out, its dtype, n, d, stream
+        "gb_norm_conv": [_vp, _vp, _i, _vp, _vp, _i, _vp, C.c_longlong, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _vp],
+        # x, scales, groups, gamma, state, slot stride, q_start, q_len, state slots, requests, d, taps, stream
+        "gb_norm_conv_state": [_vp, _vp, _i, _vp, _vp, C.c_longlong, _vp, _vp, _vp, _i, _i, _i, _vp],
+    },
+    "latent": {
+        # in, dtype, ld, gamma, eps, slots, pages, page size, n, R, stream
+        "gb_latent_store": [_vp, _i, _i, _vp, _f, _vp, _vp, _i, _i, _i, _vp],
+        # q, dtype, ldq, uk, uk_t, head columns, dim, out, n, heads, R, stream
+        "gb_latent_absorb": [_vp, _i, _i, _vp, _vp, _i, _i, _vp, _i, _i, _i, _vp],
+        "gb_latent_decode_takes": [_i, _i],
+        # q, dtype, pages, tables, stride, positions, tok_seq, n, heads, R, page size, scale, chunk, splits, acc, ml, plain, stream
+        "gb_latent_decode": [_vp, _i, _vp, _vp, _i, _vp, _vp, _i, _i, _i, _i, _f, _i, _i, _vp, _vp, _i, _vp],
+        # acc, ml, positions, chunk, splits, sinks, uv, head columns, gate, its stride, out, its stride, dtype, n, heads, R, vdim, stream
+        "gb_latent_finish": [_vp, _vp, _vp, _i, _i, _vp, _vp, _i, _vp, _i, _vp, _i, _i, _i, _i, _i, _i, _vp],
+        # q_len, pos0, first, count, page size, table, stride, source, total, stream
+        "gb_latent_tables": [_vp, _vp, _i, _i, _i, _vp, _i, _vp, _i, _vp],
+        # pages, dtype, tables, stride, source, q_len, pos0, page size, R, total, out, stream
+        "gb_latent_gather": [_vp, _i, _vp, _i, _vp, _vp, _vp, _i, _i, _i, _vp, _vp],
+        # kv, dtype, ld, k pages, v pages, heads, head columns, page size, total, stream
+        "gb_latent_expand": [_vp, _i, _i, _vp, _vp, _i, _i, _i, _i, _vp],
+    },
+    "moe": {
+        # z, ldz, n, experts, correction, top, scale, shared, combine, ids, weights, stream
         "gb_moe_route": [_vp, _i, _i, _i, _vp, _i, _f, _i, _vp, _vp, _vp, _vp],
         # z, ldz, n, experts, correction, top, scale, shared (0, 1 gate, 2 whole), softmax, renorm, groups, kept groups,
         # combine, ids, weights, stream
         "gb_moe_route_by": [_vp, _i, _i, _i, _vp, _i, _f, _i, _i, _i, _i, _i, _vp, _vp, _vp, _vp],
         # z, its dtype, ld, combine, its columns, act, its dtype, lda, n, inter, experts, ff, stream
         "gb_moe_relu2_units": [_vp, _i, _i, _vp, _i, _vp, _i, _i, _i, _i, _i, _i, _vp],
-        # gate_up, its dtype, ld, combine, its columns, act, its dtype, n, inter, experts, ff, stream
-        "gb_moe_gated_units": [_vp, _i, _i, _vp, _i, _vp, _i, _i, _i, _i, _i, _vp],
+        # gate_up, its dtype, ld, combine, its columns, act, its dtype, n, inter, experts, ff, limit, alpha, plus, stream
+        "gb_moe_gated_units": [_vp, _i, _i, _vp, _i, _vp, _i, _i, _i, _i, _i, _f, _f, _f, _vp],
         # ids, n, top, experts, rows a tile, tiles, counts, rows, pos, map, stream
         "gb_moe_sort": [_vp, _i, _i, _i, _i, _i, _vp, _vp, _vp, _vp, _vp],
         # y, ldy, pos, weights, top, y_shared, its stride, gates, their stride, out, ldo, accumulate, n, d, rows of y, stream
@@ -150,8 +180,9 @@ _SIGS = {
         # emit_gamma, emit_gamma_dtype, emit_h, emit_ldh, emit_ss, parts, n_parts, split_ws, split_ws_floats, stream
         "gb_gemm_bf16": [_vp, _i, _vp, _i, _vp, _i, _i, _i, _i, _i, _i, _vp, _i, _f, _vp, _i, _vp, _i, _vp, _vp, _i, _vp,
                          C.c_longlong, _vp],
-        # a, lda, rows, w, ldw, distance between groups, up_off, c, ldc, c_dtype, map, tiles, rows a tile, N, K, epilogue, stream
-        "gb_gemm_bf16_grouped": [_vp, _i, _vp, _vp, _i, C.c_longlong, _i, _vp, _i, _i, _vp, _i, _i, _i, _i, _i, _vp],
+        # a, lda, rows, w, ldw, distance between groups, up_off, c, ldc, c_dtype, map, tiles, rows a tile, N, K, epilogue,
+        # limit, alpha, plus, stream
+        "gb_gemm_bf16_grouped": [_vp, _i, _vp, _vp, _i, C.c_longlong, _i, _vp, _i, _i, _vp, _i, _i, _i, _i, _i, _f, _f, _f, _vp],
         # a, lda, w, ldw, c, ldc, M, N, K, limit, alpha, plus, stream
         "gb_gemm_bf16_glu": [_vp, _i, _vp, _i, _vp, _i, _i, _i, _i, _f, _f, _f, _vp],
         "gb_gemm_bf16_split_floats": [_i, _i, _i],
@@ -319,9 +350,10 @@ class LaunchTape:
 
 
 class TapeOperands:
-    """The tensors of a layer, in a fixed order, as the address ranges the native runner maps between layers."""
+    """The tensors of a layer, in a fixed order, as the address ranges the native runner maps between layers.  ``places``:
+    so many more ranges for tensors that change from step to step (``place``); these must not overlap the others."""
 
-    def __init__(self, tensors: Sequence[torch.Tensor]):
+    def __init__(self, tensors: Sequence[torch.Tensor], places: int = 0):
         n = len(tensors)
         ptrs, sizes = [], []
         for t in tensors:
@@ -329,14 +361,20 @@ class TapeOperands:
             ptrs.append(t.data_ptr())
             sizes.append(span * t.element_size())
         self.sizes = tuple(sizes)
-        self.ptrs = (C.c_uint64 * max(1, n))(*ptrs)
-        self.bytes = (C.c_uint64 * max(1, n))(*sizes)
-        self.count = n
+        self.ptrs = (C.c_uint64 * max(1, n + places))(*ptrs)
+        self.bytes = (C.c_uint64 * max(1, n + places))(*sizes)
+        self.fixed, self.count = n, n + places
         self.keep = list(tensors)
         # pairs of ranges that overlap or coincide (a tensor that the layer holds in two places): a pointer into such a
         # place has two ranges to be moved by
         order = sorted((i for i in range(n) if sizes[i]), key=lambda i: ptrs[i])
         self.overlaps = [(a, b) for k, a in enumerate(order) for b in order[k + 1:] if ptrs[b] < ptrs[a] + sizes[a]]
+
+    def place(self, i: int, t: torch.Tensor) -> None:
+        if not t.is_contiguous():
+            raise KernelError("a tensor placed among a layer's must be contiguous")
+        self.ptrs[self.fixed + i] = t.data_ptr()
+        self.bytes[self.fixed + i] = t.numel() * t.element_size()
 
     def maps_onto(self, target: "TapeOperands") -> bool:
         """Whether every pointer into these tensors has one place in ``target``'s: ranges that overlap here must be
@@ -363,7 +401,7 @@ def stop_tape() -> None:
 
 def run_tape(tape: LaunchTape, recorded: TapeOperands, target: TapeOperands) -> None:
     """Makes the recorded launches again with the tensors of ``recorded`` replaced, one for one, by those of ``target``."""
-    if not tape.usable or recorded.sizes != target.sizes or not recorded.maps_onto(target):
+    if not tape.usable or recorded.sizes != target.sizes or recorded.count != target.count or not recorded.maps_onto(target):
         raise KernelError("run_tape: the layer's tensors do not match those of the recorded layer")
     rc = _host_lib().gbh_tape_run(tape.pointer(), len(tape), C.addressof(recorded.ptrs), C.addressof(recorded.bytes),
                                   C.addressof(target.ptrs), recorded.count)
@@ -1133,15 +1171,16 @@ def norm_add(x: torch.Tensor, y: torch.Tensor, g: torch.Tensor, eps: float, roun
 # ------------------------------------------------------------------- routed experts
 MOE_MAX_EXPERTS = 512   # moe.hip: a lane of the routing wave holds eight experts
 MOE_MAX_TOP = 16
+SILU_UNIT = (float("inf"), 1.0, 0.0)   # (limit, alpha, plus) of a gated unit that is silu(gate) * up
 
 
 def moe_route(z: torch.Tensor, n_experts: int, correction: Optional[torch.Tensor], top: int, scale: float, shared,
-              combine: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, softmax: bool = False, renorm: bool = True,
+              combine: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, softmax=False, renorm: bool = True,
               groups: int = 0, keep_groups: int = 0) -> None:
     """From router logits ``z`` (float32 [n, experts (+ 1)]): scores sigmoid(z), or with ``softmax`` the softmax over all
     experts; the ``top`` experts with the largest score + correction (of equal ones the lower index), with ``groups`` only
-    out of the ``keep_groups`` runs of experts / groups neighbours whose best score + correction is largest; their weights
-    score * scale, with ``renorm`` divided by (the sum of the chosen scores + 1e-20).
+    out of the ``keep_groups`` runs of experts / groups neighbours whose best score + correction is largest
+    (``softmax="chosen"``: scores e^(z + correction), and the choice by z + correction itself); their weights score * scale, with ``renorm`` divided by (the sum of the chosen scores + 1e-20).
     ``ids`` int32 and ``weights`` float32 [n, top] receive the choice, ``combine`` float32 [n, experts (+ 1)] a row of
     weights with zeros for the others; with ``shared`` one more column for an expert that every token uses: sigmoid of
     z's last column (True, "gate"), or 1 ("whole")."""
@@ -1158,7 +1197,8 @@ def moe_route(z: torch.Tensor, n_experts: int, correction: Optional[torch.Tensor
     lib = _lib("moe")
     if softmax or not renorm or groups or shared == "whole":
         _launch(lib, lib.gb_moe_route_by, _p(z), z.stride(0), n, n_experts, _p(correction), int(top), float(scale),
-                2 if shared == "whole" else 1 if shared else 0, 1 if softmax else 0, 1 if renorm else 0, int(groups),
+                2 if shared == "whole" else 1 if shared else 0, 2 if softmax == "chosen" else 1 if softmax else 0,
+                1 if renorm else 0, int(groups),
                 int(keep_groups), _p(combine), _p(ids), _p(weights), _stream())
         return
     _launch(lib, lib.gb_moe_route, _p(z), z.stride(0), n, n_experts, _p(correction), int(top), float(scale),
@@ -1180,8 +1220,10 @@ def moe_relu2_units(z: torch.Tensor, combine: Optional[torch.Tensor], out: torch
             _p(out), dtype_code(out), out.stride(0), n, inter, n_experts, ff, _stream())
 
 
-def moe_gated_units(gate_up: torch.Tensor, combine: torch.Tensor, out: torch.Tensor, n_experts: int, ff: int) -> None:
-    """out[t, j] = silu(gate) * up * combine[t, expert of column j]: ``gate_up`` [n, 2 * I] holds the experts' gate columns, the
+def moe_gated_units(gate_up: torch.Tensor, combine: torch.Tensor, out: torch.Tensor, n_experts: int, ff: int,
+                    unit: tuple = SILU_UNIT) -> None:
+    """out[t, j] = unit(gate, up) * combine[t, expert of column j], ``unit = (limit, alpha, plus)`` with g' = min(g, limit), u' =
+    clamp(u, -limit, limit), g' sigmoid(alpha g') (u' + plus), by default silu(gate) * up: ``gate_up`` [n, 2 * I] holds the experts' gate columns, the
     experts' up columns, then the shared expert's gate columns and its up columns; columns e * ff .. of ``out`` are expert
     e's, those from experts * ff on the shared expert's (weight in the last column of ``combine``)."""
     _dev(gate_up, combine, out)
@@ -1192,10 +1234,9 @@ def moe_gated_units(gate_up: torch.Tensor, combine: torch.Tensor, out: torch.Ten
         raise KernelError("moe_gated_units: combine must be contiguous float32 [n, experts (+ 1)]")
     lib = _lib("moe")
     _launch(lib, lib.gb_moe_gated_units, _p(gate_up), dtype_code(gate_up), gate_up.stride(0), _p(combine), combine.shape[1],
-            _p(out), dtype_code(out), n, inter, n_experts, ff, _stream())
+            _p(out), dtype_code(out), n, inter, n_experts, ff, *map(float, unit), _stream())
 
 
-# ------------------------------------------------------------------- small residual operations
 def moe_sort_tiles(entries: int, n_experts: int, tile_rows: int) -> int:
     """Row tiles that ``moe_sort`` may need: every expert's last tile may be short."""
     return entries // tile_rows + n_experts
@@ -1246,11 +1287,13 @@ def gemm_grouped_takes(a: torch.Tensor, w: torch.Tensor, group_stride: int) -> b
 
 
 def gemm_grouped(a: torch.Tensor, rows: Optional[torch.Tensor], w: torch.Tensor, group_stride: int, n_out: int,
-                 tile_map: torch.Tensor, tile_rows: int, out: torch.Tensor, silu_mul: bool = False, up_offset: int = 0) -> None:
+                 tile_map: torch.Tensor, tile_rows: int, out: torch.Tensor, silu_mul: bool = False, up_offset: int = 0,
+                 unit: tuple = SILU_UNIT) -> None:
     """Products of groups of rows with a matrix of their own each.  Sorted row r of the product reads row ``rows[r]`` of
     ``a`` (row r without ``rows``); ``tile_map`` (as ``moe_sort`` writes it) names each row tile's group and rows; group g
     uses the ``n_out`` rows of ``w`` that begin ``g * group_stride`` elements into it.  ``silu_mul``: the group's rows
-    are n_out / 2 gate rows, with the up row of each ``up_offset`` rows behind it, and out = silu(gate) * up."""
+    are n_out / 2 gate rows, with the up row of each ``up_offset`` rows behind it, and out = silu(gate) * up, or another
+    ``unit = (limit, alpha, plus)`` as ``moe_gated_units`` takes it."""
     _dev(a, rows, w, tile_map, out)
     K = a.shape[1]
     cols = n_out // 2 if silu_mul else n_out
@@ -1264,9 +1307,11 @@ def gemm_grouped(a: torch.Tensor, rows: Optional[torch.Tensor], w: torch.Tensor,
         _i32(rows, "rows")
     lib = _lib("gemm_bf16")
     _launch(lib, lib.gb_gemm_bf16_grouped, _p(a), a.stride(0), _p(rows), _p(w), w.stride(0), int(group_stride), int(up_offset),
-            _p(out), out.stride(0), dtype_code(out), _p(tile_map), tiles, tile_rows, n_out, K, 2 if silu_mul else 0, _stream())
+            _p(out), out.stride(0), dtype_code(out), _p(tile_map), tiles, tile_rows, n_out, K, 2 if silu_mul else 0,
+            *map(float, unit), _stream())
 
 
+# ------------------------------------------------------------------- small residual operations
 def embed_pairs(table: torch.Tensor, pairs: torch.Tensor, ctx, out: torch.Tensor, buckets: int, mul_prev: int, mul_cur: int,
                 prev: torch.Tensor) -> None:
     """out[i] = table[id_i] + pairs[(id_(i-1) * mul_prev + id_i * mul_cur) mod buckets], row ``buckets`` of ``pairs`` for
@@ -1685,15 +1730,20 @@ def _prefill_parts(max_q: int, max_ctx: int, n_heads: int, n_seqs: int, hd: int)
 
 
 def attention_prefill(q: torch.Tensor, out: torch.Tensor, ctx, cache, n_heads: int, scale: float, window: int,
-                      keep_first: int = 0, chunk: int = 0, softcap: float = 0.0, sinks: Optional[torch.Tensor] = None) -> None:
-    """The requests of the step that bring more than one token (they follow the single-token ones)."""
+                      keep_first: int = 0, chunk: int = 0, softcap: float = 0.0, sinks: Optional[torch.Tensor] = None,
+                      tables: Optional[torch.Tensor] = None) -> None:
+    """The requests of the step that bring more than one token (they follow the single-token ones).  ``tables``: block
+    tables other than the cache's own (int32 [requests, pages]), for keys and values in pages of the step's making."""
     n_dec, S = ctx.host["n_decode"], ctx.num_seqs
     k_pages, v_pages = cache.k_pages, cache.v_pages
     _dev(q, out, k_pages, v_pages)
     _, nkv, page, hd = _check_pages(k_pages, v_pages, torch.bfloat16, "attention_prefill")
     if q.dtype != torch.bfloat16 or out.dtype not in (torch.bfloat16, torch.float32) or q.shape[1] != n_heads * hd:
         raise KernelError("attention_prefill: q must be bfloat16 [n, heads * head size], out bfloat16 or float32")
-    tables = ctx.tables[cache.group]
+    if tables is None:
+        tables = ctx.tables[cache.group]
+    elif tables.dtype != torch.int32 or tables.dim() != 2 or tables.stride(1) != 1 or tables.shape[0] < S:
+        raise KernelError("attention_prefill: block tables must be int32 [requests, pages]")
     lib = _lib("attention_bf16")
     max_q, max_ctx = int(ctx.host["max_q_len"]), int(ctx.host["max_context"])
     # the portions' rows follow the single-token requests' rows; few and short portions over long contexts share
@@ -1877,3 +1927,250 @@ def gate_rows(att: torch.Tensor, head_cols: int, gate: torch.Tensor, out: torch.
     lib = _lib("tanhmix")
     _launch(lib, lib.gb_gate_rows, _p(att), _rows(att, "att"), int(head_cols), _p(gate), _rows(gate, "gate"), 1 if per_head else 0,
             dtype_code(att), _p(out), _rows(out, "out"), n, n_heads, vdim, _stream())
+
+
+# ------------------------------------------------- grouped norms, convolutions of normed rows, sums over depth (groupmix.hip)
+GROUP_NORM_MAX_GROUPS = 64
+RESIDUAL_ROWS_MAX = 12288   # the widest row groupmix.hip keeps in LDS
+NORM_CONV_MAX_TAPS = 8
+
+
+def embed_sinusoid(table: torch.Tensor, ids: torch.Tensor, positions: torch.Tensor, turns: torch.Tensor, out: torch.Tensor,
+                   scale: float = 1.0) -> None:
+    """out[i] = table[ids[i]] * scale + [sin a_0, cos a_0, sin a_1, cos a_1, ...], a_k = 2 pi * positions[i] * turns[k]; out
+    float32 [n, d] or [copies, n, d], ``turns`` float64 [ceil(d / 2)]."""
+    _dev(table, ids, positions, turns, out)
+    copies = out.shape[0] if out.dim() == 3 else 1
+    n, d = out.shape[-2:]
+    _i32(ids, "ids", n)
+    _i32(positions, "positions", n)
+    if out.dtype != torch.float32 or not out.is_contiguous() or not table.is_contiguous() or table.shape[1] != d:
+        raise KernelError("embed_sinusoid: out must be contiguous float32 [n, d] or [copies, n, d] and table [vocab, d]")
+    if turns.dtype != torch.float64 or not turns.is_contiguous() or turns.numel() != (d + 1) // 2:
+        raise KernelError("embed_sinusoid: turns must be contiguous float64 [ceil(d / 2)]")
+    lib = _lib("groupmix")
+    _launch(lib, lib.gb_embed_sinusoid, _p(table), dtype_code(table), _p(ids), _p(positions), _p(turns), _p(out), n, d,
+            table.shape[0], float(scale), int(copies), _stream())
+
+
+def _conv_slots(w: Optional[torch.Tensor], state: Optional[torch.Tensor], d: int, what: str):
+    """(taps, distance of two slots) of convolution weights [taps, d] and of their state [slots, taps - 1, d], whose slots
+    may lie further apart than they are long (several convolutions in one slot)."""
+    if w is None:
+        return 0, 0
+    taps = w.shape[0]
+    _f32_rows(w, (taps, d), f"{what}: w")
+    if not 1 <= taps <= NORM_CONV_MAX_TAPS:
+        raise KernelError(f"{what}: {taps} taps are above {NORM_CONV_MAX_TAPS}")
+    if taps == 1:
+        return 1, 0
+    if (state is None or state.dtype != torch.float32 or tuple(state.shape[1:]) != (taps - 1, d) or state.stride(2) != 1
+            or (taps > 2 and state.stride(1) != d)):
+        raise KernelError(f"{what}: state must be float32 [slots, taps - 1, d] with dense slots")
+    return taps, state.stride(0)
+
+
+def residual_rows(x: torch.Tensor, y: Optional[torch.Tensor] = None, slices: int = 1, average: Optional[tuple] = None,
+                  gamma: Optional[torch.Tensor] = None, groups: int = 0, eps: float = 0.0, scales: Optional[torch.Tensor] = None,
+                  h: Optional[torch.Tensor] = None, conv: Optional[tuple] = None, ctx=None,
+                  rows: Optional[torch.Tensor] = None) -> None:
+    """One pass over the rows of the residual ``x`` (float32 [n, d]): x += y (float32 [n, d], or with ``slices`` > 1 the sum
+    of [slices, n, d], as a product that divides k leaves it); with ``average = (hist, coef, out)`` (hist float32 [count, n,
+    d], coef [count + 1], out [n, d]) out = sum_j coef[j] hist[j] + coef[count] x; then, with ``groups``, the RMS norm of x (or
+    of out) in equal runs of channels: a factor a (row, group) to ``scales`` (float32 [n, groups]) and / or the rows, times
+    ``gamma``, to ``h`` ([n, d], any activations' type).  ``conv = (w, state)`` (every request of the step ``ctx`` brings one
+    row): h receives rows + conv(rows) and the requests' slots move on.  ``rows``: the rows of x to norm, in their order."""
+    _dev(x, y, gamma, scales, h, rows)
+    d = x.shape[1]
+    _f32_rows(x, (x.shape[0], d), "x")
+    n = x.shape[0] if rows is None else rows.numel()
+    _i32(rows, "rows")
+    if y is not None:
+        if slices > 1:
+            if y.dtype != torch.float32 or not y.is_contiguous() or y.numel() < slices * n * d:
+                raise KernelError("residual_rows: slices of y must be contiguous float32 [slices, n, d]")
+        else:
+            _f32_rows(y, (n, d), "y")
+    hist = coef = out = None
+    count = 0
+    if average is not None:
+        hist, coef, out = average
+        _dev(hist, coef, out)
+        count = hist.shape[0]
+        if hist.dtype != torch.float32 or tuple(hist.shape[1:]) != (n, d) or not hist.is_contiguous() or count < 1:
+            raise KernelError("residual_rows: hist must be contiguous float32 [count, n, d]")
+        _f32_rows(coef, (count + 1,), "coef")
+        _f32_rows(out, (n, d), "out")
+    if groups:
+        if d % groups or groups > GROUP_NORM_MAX_GROUPS:
+            raise KernelError(f"residual_rows: {groups} groups of {d} columns (at most {GROUP_NORM_MAX_GROUPS})")
+        if scales is not None:
+            _f32_rows(scales, (n, groups), "scales")
+        if h is not None:
+            _f32_rows(gamma, (d,), "gamma")
+            if tuple(h.shape) != (n, d) or not h.is_contiguous():
+                raise KernelError("residual_rows: h must be contiguous [n, d]")
+    w, state = conv if conv is not None else (None, None)
+    taps, slot = _conv_slots(w, state, d, "residual_rows")
+    if conv is not None:
+        _dev(w, state)
+        if h is None or ctx is None or int(ctx.host["max_q_len"]) != 1:
+            raise KernelError("residual_rows: the convolution goes with a step of single rows and a result")
+    tables = conv is not None
+    lib = _lib("groupmix")
+    _launch(lib, lib.gb_residual_rows, _p(x), _p(y), int(slices), n * d, _p(hist), n * d, _p(coef), count, _p(out), _p(rows),
+            _p(gamma), int(groups), float(eps), _p(scales), _p(h), dtype_code(h) if h is not None else F32, _p(w), taps,
+            _p(state) if taps > 1 else None, slot, _p(ctx.tok_seq) if tables else None, _p(ctx.pos0) if tables else None,
+            _p(ctx.state_slots) if tables else None, n, d, _stream())
+
+
+def norm_conv(x: torch.Tensor, scales: torch.Tensor, gamma: torch.Tensor, w: Optional[torch.Tensor], state: Optional[torch.Tensor],
+              ctx, out: torch.Tensor) -> None:
+    """out = g + conv(g) in the type of ``out``, g = x * scales * gamma (x float32 [n, d], ``scales`` float32 [n, groups] as
+    ``residual_rows`` leaves them), conv(g)[t] = sum_j w[j] g[t - taps + 1 + j] over the request's own tokens, zeros before its
+    first (``w`` float32 [taps, d], or None).  The request's last taps - 1 rows of g live in ``state`` (float32 [slots, taps - 1,
+    d]) and are moved on by this call, so it must come before x changes."""
+    _dev(x, scales, gamma, w, state, out)
+    n, d = x.shape
+    _f32_rows(x, (n, d), "x")
+    groups = scales.shape[1]
+    _f32_rows(scales, (n, groups), "scales")
+    _f32_rows(gamma, (d,), "gamma")
+    if tuple(out.shape) != (n, d) or not out.is_contiguous() or d % groups:
+        raise KernelError("norm_conv: out must be contiguous [n, d], the groups equal runs of its columns")
+    taps, slot = _conv_slots(w, state, d, "norm_conv")
+    lib = _lib("groupmix")
+    _launch(lib, lib.gb_norm_conv, _p(x), _p(scales), groups, _p(gamma), _p(w), taps, _p(state) if taps > 1 else None, slot,
+            _p(ctx.tok_seq), _p(ctx.q_start), _p(ctx.pos0), _p(ctx.state_slots), _p(out), dtype_code(out), n, d, _stream())
+    if taps > 1:
+        _launch(lib, lib.gb_norm_conv_state, _p(x), _p(scales), groups, _p(gamma), _p(state), slot, _p(ctx.q_start),
+                _p(ctx.q_len), _p(ctx.state_slots), ctx.num_seqs, d, taps, _stream())
+
+
+# ------------------------------------------------------------------ attention over cached latents (latent.hip)
+LATENT_MAX_RANK = 2048
+
+
+def _latent_pages(pages: torch.Tensor, dtype, what: str):
+    """Pages of one latent row a token ([pages, 1, R / piece, page size, piece]): (page size, R)."""
+    if pages is None or pages.dim() != 5 or pages.shape[1] != 1 or not pages.is_contiguous() or pages.dtype != dtype:
+        raise KernelError(f"{what}: pages must be contiguous [pages, 1, R / piece, page size, piece] of the activations' type")
+    _, _, n, P, piece = pages.shape
+    if piece != key_piece(n * piece):
+        raise KernelError(f"{what}: latents of {n * piece} channels are kept in pieces of {key_piece(n * piece)}, not {piece}")
+    return P, n * piece
+
+
+def latent_store(rows: torch.Tensor, gamma: torch.Tensor, eps: float, slots: torch.Tensor, pages: torch.Tensor) -> None:
+    """The RMS norm of the latents in the first R columns of ``rows``, with weight ``gamma`` (float32 [R]), into the cache rows
+    ``slots`` of ``pages``."""
+    _dev(rows, gamma, slots, pages)
+    P, R = _latent_pages(pages, rows.dtype, "latent_store")
+    n = rows.shape[0]
+    _f32_rows(gamma, (R,), "gamma")
+    _i32(slots, "slots", n)
+    lib = _lib("latent")
+    _launch(lib, lib.gb_latent_store, _p(rows), dtype_code(rows), _act_rows(rows, rows.dtype, R, "rows"), _p(gamma), float(eps),
+            _p(slots), _p(pages), P, n, R, _stream())
+
+
+def latent_absorb(q: torch.Tensor, uk: torch.Tensor, uk_t: Optional[torch.Tensor], head_cols: int, dim: int, out: torch.Tensor,
+                  n_heads: int) -> None:
+    """out[:, h] = W_uk,h^T q_h: ``q`` [n, >= heads * head_cols], ``uk`` [>= heads * head_cols, R] (the first ``dim`` rows of a head
+    count), ``uk_t`` [heads, R, head_cols] the same turned, for the matrix cores (None: the plain kernel); out [n, heads * R]."""
+    _dev(q, uk, uk_t, out)
+    n, R = q.shape[0], uk.shape[1]
+    if not uk.is_contiguous() or uk.shape[0] < n_heads * head_cols or uk.dtype != q.dtype or out.dtype != q.dtype \
+            or tuple(out.shape) != (n, n_heads * R) or not out.is_contiguous():
+        raise KernelError("latent_absorb: uk must be [>= heads * head columns, R], out contiguous [n, heads * R], all of one type")
+    if uk_t is not None and (tuple(uk_t.shape) != (n_heads, R, head_cols) or not uk_t.is_contiguous() or uk_t.dtype != q.dtype):
+        raise KernelError("latent_absorb: uk_t must be contiguous [heads, R, head columns]")
+    lib = _lib("latent")
+    _launch(lib, lib.gb_latent_absorb, _p(q), dtype_code(q), _act_rows(q, q.dtype, n_heads * head_cols, "q"), _p(uk), _p(uk_t),
+            head_cols, dim, _p(out), n, n_heads, R, _stream())
+
+
+@functools.lru_cache(maxsize=4096)
+def latent_tuned_takes(dtype, R: int, page_size: int) -> bool:
+    """Whether the matrix-core kernel attends to latents of R channels in pages of ``page_size`` tokens."""
+    return dtype == torch.bfloat16 and bool(_lib("latent").gb_latent_decode_takes(R, page_size))
+
+
+@functools.lru_cache(maxsize=4096)
+def latent_chunk(rows: int, n_heads: int, max_context: int, tuned: bool) -> int:
+    """Latents a workgroup attends to: about one workgroup for every compute unit (a workgroup of the matrix-core kernel takes
+    all of one), at least 128 keys each, since every chunk leaves a row of sums a head for the last pass."""
+    if tuned:
+        groups = rows * -(-n_heads // (32 if n_heads > 16 else 16))
+        want, step, least = max(1, 256 // groups), 64, 128
+    else:
+        want, step, least = max(1, 1024 // (rows * n_heads)), 256, 256
+    chunk = -(-max_context // min(want, 256))
+    return max(least, -(-chunk // step) * step)
+
+
+def latent_decode(q: torch.Tensor, pages: torch.Tensor, tables: torch.Tensor, positions: torch.Tensor, tok_seq: torch.Tensor,
+                  n_heads: int, scale: float, max_context: int, sinks: Optional[torch.Tensor], uv: torch.Tensor, head_cols: int,
+                  vdim: int, gate: Optional[torch.Tensor], out: torch.Tensor, buffer, plain: bool = False) -> None:
+    """Attention of rows with absorbed queries ``q`` ([n, heads * R]) over their requests' cached latents: out [n, heads * vdim] =
+    sigmoid(gate) * W_uv (softmax(scale * q . c, with a sink a head) c).  ``uv`` [>= heads * head_cols, R], the first ``vdim`` rows
+    of a head.  The matrix-core kernel takes row t for request t's single token; ``plain``: any rows, by ``tok_seq``.
+    ``buffer(name, shape, dtype)`` gives the workspace of the chunks' sums."""
+    _dev(q, pages, tables, positions, tok_seq, uv, gate, out)
+    P, R = _latent_pages(pages, q.dtype, "latent_decode")
+    n = q.shape[0]
+    if tuple(q.shape) != (n, n_heads * R) or not q.is_contiguous():
+        raise KernelError("latent_decode: q must be contiguous [n, heads * R]")
+    if not uv.is_contiguous() or uv.shape[1] != R or uv.shape[0] < n_heads * head_cols or uv.dtype != q.dtype:
+        raise KernelError("latent_decode: uv must be contiguous [>= heads * head columns, R]")
+    if tables.dtype != torch.int32 or tables.dim() != 2 or tables.stride(1) != 1:
+        raise KernelError("latent_decode: block tables must be int32 [requests, pages]")
+    _i32(positions, "positions", n)
+    _i32(tok_seq, "tok_seq", n)
+    chunk = latent_chunk(n, n_heads, max_context, not plain)
+    splits = -(-max_context // chunk)
+    acc = buffer("latent_acc", (n * n_heads * splits * R,), torch.float32)
+    ml = buffer("latent_ml", (n * n_heads * splits * 2,), torch.float32)
+    lib = _lib("latent")
+    _launch(lib, lib.gb_latent_decode, _p(q), dtype_code(q), _p(pages), _p(tables), tables.stride(0), _p(positions), _p(tok_seq), n,
+            n_heads, R, P, float(scale), chunk, splits, _p(acc), _p(ml), 1 if plain else 0, _stream())
+    _launch(lib, lib.gb_latent_finish, _p(acc), _p(ml), _p(positions), chunk, splits, _p(_sinks(sinks, n_heads)), _p(uv), head_cols,
+            _p(gate), _act_rows(gate, q.dtype, n_heads * vdim, "gate") if gate is not None else 0, _p(out),
+            _act_rows(out, q.dtype, n_heads * vdim, "out"), dtype_code(out), n, n_heads, R, vdim, _stream())
+
+
+def latent_tables(ctx, first: int, page_size: int, table: torch.Tensor, source: torch.Tensor) -> None:
+    """Scratch pages for the contexts of requests first .. of the step, one for each page of each: ``table`` int32 [requests,
+    pages] their numbers by request, ``source`` int32 [total, 2] the (request, page of its context) behind each."""
+    _dev(table, source)
+    if table.dtype != torch.int32 or table.shape[0] < ctx.num_seqs or not table.is_contiguous() or source.dtype != torch.int32 \
+            or not source.is_contiguous():
+        raise KernelError("latent_tables: table must be contiguous int32 [requests, pages], source int32 [total, 2]")
+    lib = _lib("latent")
+    _launch(lib, lib.gb_latent_tables, _p(ctx.q_len), _p(ctx.pos0), int(first), ctx.num_seqs - int(first), int(page_size), _p(table),
+            table.stride(0), _p(source), source.shape[0], _stream())
+
+
+def latent_gather(pages: torch.Tensor, tables: torch.Tensor, source: torch.Tensor, ctx, out: torch.Tensor) -> None:
+    """Rows of the latents behind the scratch pages ``source`` (``latent_tables``): out [total * page size, R], zeros behind a
+    context's end."""
+    _dev(pages, tables, source, out)
+    P, R = _latent_pages(pages, out.dtype, "latent_gather")
+    total = source.shape[0]
+    if tuple(out.shape) != (total * P, R) or not out.is_contiguous() or tables.dtype != torch.int32 or tables.stride(1) != 1:
+        raise KernelError("latent_gather: out must be contiguous [total * page size, R], tables int32 [requests, pages]")
+    lib = _lib("latent")
+    _launch(lib, lib.gb_latent_gather, _p(pages), dtype_code(pages), _p(tables), tables.stride(0), _p(source), _p(ctx.q_len),
+            _p(ctx.pos0), P, R, total, _p(out), _stream())
+
+
+def latent_expand(kv: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor) -> None:
+    """Rows [total * page size, 2 * heads * head size] ([key heads | value heads]) into pages, row r to slot r mod page size of
+    page r / page size."""
+    _dev(kv, k_pages, v_pages)
+    total, H, P, hc = _check_pages(k_pages, v_pages, kv.dtype, "latent_expand")
+    if kv.shape[0] != total * P:
+        raise KernelError("latent_expand: a row for every slot of the pages")
+    lib = _lib("latent")
+    _launch(lib, lib.gb_latent_expand, _p(kv), dtype_code(kv), _act_rows(kv, kv.dtype, 2 * H * hc, "kv"), _p(k_pages), _p(v_pages), H,
+            hc, P, total, _stream())

@@ -663,3 +663,130 @@ class GatedAttention(Mixer):
             return product_in_slices(ctx, gated, self.wo, residual)
         product(ctx, gated, self.wo, residual, accumulate=True)
         return None
+
+
+class LatentCacheAttention(Mixer):
+    """Attention through a narrow latent that is all a position leaves in the cache: c = norm(W_dkv h) (RMS norm with a weight,
+    ``kv_rank`` channels), a head's key W_uk c (``dim`` channels) and value W_uv c (``vdim``), queries W_q h; positions enter
+    nowhere.  Scores q . k * ``scale`` over all earlier keys; with ``sink`` exp(sink_h), one number a head, joins the softmax's
+    denominator and has no value; the heads are multiplied by sigmoid(W_g h); output projection.
+
+    Tensors: ``q``, ``dkv``, ``dkv.norm``, ``uk``, ``uv``, ``sink``, ``g``, ``o``.  The pages hold one row of ``kv_rank`` channels a
+    position (no value pages).  A token that comes alone attends to the latents themselves: its queries go through W_uk^T, the
+    weighted sums of latents through W_uv (``ops.latent_decode``), so that a latent is read once for all heads.  Prompt portions
+    have many tokens to every key: the latents of their requests' contexts are taken through W_uk and W_uv into scratch pages of
+    keys and values, and the paged attention kernels do the rest.
+
+    The stacked matrices give every head ``cache_head_cols(dim, vdim)`` columns, zeros behind its own: queries, keys and values
+    come out of their products as the attention kernels read them."""
+    replayable = True
+    taped = True
+    accepts_store = True
+
+    def __init__(self, width: int, n_heads: int, dim: int, vdim: int, kv_rank: int, scale: float, eps: float, sink: bool = False):
+        self.width, self.n_heads, self.dim, self.vdim, self.kv_rank = width, int(n_heads), int(dim), int(vdim), int(kv_rank)
+        self.scale, self.eps, self.sink = float(scale), float(eps), bool(sink)
+        self.head_cols = cache_head_cols(dim, vdim)
+        self.cache_spec = CacheSpec(1, self.kv_rank, FULL, 0, values=False)
+        self.w_in = self.w_ukv = self.w_uk_t = self.wo = self.norm_kv = self.sinks = None
+
+    def tensor_specs(self) -> Dict[str, TensorSpec]:
+        H, D, V = self.n_heads, self.dim, self.vdim
+        specs = {"q": TensorSpec((H * D, self.width)), "dkv": TensorSpec((self.kv_rank, self.width)),
+                 "dkv.norm": TensorSpec((self.kv_rank,), kind="f32", init="ones"),
+                 "uk": TensorSpec((H * D, self.kv_rank)), "uv": TensorSpec((H * V, self.kv_rank))}
+        if self.sink:
+            specs["sink"] = TensorSpec((H,), kind="f32")
+        specs["g"] = TensorSpec((H * V, self.width))
+        specs["o"] = TensorSpec((self.width, H * V))
+        return specs
+
+    def _padded_heads(self, w: torch.Tensor, size: int) -> torch.Tensor:
+        """A projection's rows, ``size`` a head, with zero rows up to ``head_cols`` a head."""
+        if size == self.head_cols:
+            return w
+        out = torch.zeros((self.n_heads, self.head_cols, w.shape[1]), dtype=w.dtype, device=w.device)
+        out[:, :size] = w.view(self.n_heads, size, w.shape[1])
+        return out.view(self.n_heads * self.head_cols, w.shape[1])
+
+    def load(self, tensors):
+        # one product reads the mixer's input for queries, latent and gate; one expands the latents
+        self.w_in = _stack_rows([self._padded_heads(tensors["q"], self.dim), tensors["dkv"], tensors["g"]], self.width)
+        uk = self._padded_heads(tensors["uk"], self.dim)
+        self.w_ukv = torch.cat([uk, self._padded_heads(tensors["uv"], self.vdim)], 0).contiguous()
+        self.w_uk_t = uk.view(self.n_heads, self.head_cols, self.kv_rank).transpose(1, 2).contiguous()
+        self.wo = tensors["o"].contiguous()
+        self.norm_kv = tensors["dkv.norm"].float().contiguous()
+        self.sinks = tensors["sink"].float().contiguous() if self.sink else None
+
+    def streamed_matrices(self):
+        return [self.w_in, self.w_ukv, self.wo]
+
+    def problems(self, dtype, page_size):
+        if self.kv_rank > ops.LATENT_MAX_RANK:
+            return [("kv_rank", f"{self.kv_rank} is above {ops.LATENT_MAX_RANK}, the widest latent the attention kernels take")]
+        return []
+
+    def forward(self, ctx, h, residual, cache: Optional[LayerCache], store: bool = False):
+        """Adds the mixed rows into ``residual``; with ``store`` writes them there instead (float32 either way) or leaves
+        them in slices, and returns what ``product_in_slices`` does."""
+        if cache is None or cache.k_pages is None or not cache.writable:
+            raise ValueError("LatentCacheAttention needs a layer cache of its own with pages")
+        n = h.shape[0]
+        H, V, R, hc = self.n_heads, self.vdim, self.kv_rank, self.head_cols
+        first = ctx.buffer("latent_in", (n, self.w_in.shape[0]), ctx.dtype)     # [query heads | latent | gate]
+        product(ctx, h, self.w_in, first)
+        gate = first[:, H * hc + R:H * hc + R + H * V]
+        ops.latent_store(first[:, H * hc:H * hc + R], self.norm_kv, self.eps, ctx.slots[cache.group], cache.k_pages)
+        mixed = ctx.buffer("latent_mixed", (n, H * V), ctx.dtype)
+        # (heads that no attention kernel takes: every row as if it came alone)
+        alone = ctx.host["n_decode"] if hc <= ops.MAX_HEAD_DIM else n
+        if alone:
+            tuned = (ctx.tuned and alone == ctx.host["n_decode"] and ops.latent_tuned_takes(ctx.dtype, R, ctx.page_size))
+            q = ctx.buffer("latent_q", (alone, H * R), ctx.dtype)
+            ops.latent_absorb(first[:alone, :H * hc], self.w_ukv, self.w_uk_t if tuned else None, hc, self.dim, q, H)
+            ops.latent_decode(q, cache.k_pages, ctx.tables[cache.group], ctx.positions[:alone], ctx.tok_seq[:alone], H, self.scale,
+                              int(ctx.host["max_context"]), self.sinks, self.w_ukv[H * hc:], hc, V,
+                              gate[:alone], mixed[:alone], ctx.buffer, plain=not tuned)
+        if alone < n:
+            self._portions(ctx, first, gate, mixed, cache, alone)
+        if store:   # the caller's pass over the rows adds the slices of a product that divides k
+            return product_in_slices(ctx, mixed, self.wo, residual)
+        product(ctx, mixed, self.wo, residual, accumulate=True)
+        return None
+
+    def _portions(self, ctx, first, gate, mixed, cache: LayerCache, a: int) -> None:
+        """Rows a .. of the step, prompt portions: attention over keys and values expanded from their contexts' latents."""
+        n = first.shape[0]
+        H, V, hc, P = self.n_heads, self.vdim, self.head_cols, ctx.page_size
+        tables, source = self._scratch_tables(ctx)
+        total = source.shape[0]
+        c = ctx.buffer("latent_rows", (total * P, self.kv_rank), ctx.dtype)
+        ops.latent_gather(cache.k_pages, ctx.tables[cache.group], source, ctx, c)
+        kv = ctx.buffer("latent_kv", (total * P, 2 * H * hc), ctx.dtype)
+        product(ctx, c, self.w_ukv, kv)
+        scratch = LayerCache(ctx.buffer("latent_k_pages", ops.key_pages_shape(total, H, P, hc), ctx.dtype),
+                             ctx.buffer("latent_v_pages", (total, H, hc, P), ctx.dtype))
+        ops.latent_expand(kv, scratch.k_pages, scratch.v_pages)
+        q = first[:, :H * hc]
+        att = ctx.buffer("att", (n, H * hc), ctx.dtype)
+        if ctx.tuned and ops.tuned_attention_supports(scratch.k_pages, H, 0):
+            ops.attention_prefill(q, att, ctx, scratch, H, self.scale, 0, sinks=self.sinks, tables=tables)
+        else:
+            ops.attention_plain(q[a:], att[a:], ctx.positions[a:], ctx.tok_seq[a:], tables, scratch.k_pages, scratch.v_pages, H,
+                                self.scale, max_context=int(ctx.host["max_context"]), grouped=n - a >= ops.PLAIN_GROUP_MIN_ROWS,
+                                sinks=self.sinks)
+        ops.gate_heads(att[a:], hc, gate[a:], mixed[a:], H, V)
+
+    def _scratch_tables(self, ctx):
+        """Once a step for all layers: block tables of the scratch pages, and the page of latents behind each."""
+        a, P = ctx.host["n_decode"], ctx.page_size
+        key = ("latent scratch", P)
+        hit = ctx.memo.get(key)
+        if hit is None:
+            pages = [-(-(p + l) // P) for p, l in zip(ctx.host["pos0"][a:], ctx.host["q_len"][a:])]
+            table = ctx.buffer("latent_table", (ctx.num_seqs, max(pages)), torch.int32)
+            source = ctx.buffer("latent_source", (sum(pages), 2), torch.int32)
+            ops.latent_tables(ctx, a, P, table, source)
+            hit = ctx.memo[key] = (table, source)
+        return hit

@@ -59,12 +59,14 @@ class TensorSpec:
 class CacheSpec:
     """Paged keys and values of one layer.  kind FULL keeps every position, WINDOW the last ``window`` and, with
     ``keep_first``, the first so many as well; RUNS the positions of the run of ``window`` (runs counted from the
-    request's first position) that holds the next query."""
+    request's first position) that holds the next query.  ``values`` False: pages of keys alone, for a mixer that caches one
+    row a position and makes everything else of it."""
     num_kv_heads: int
     head_dim: int
     kind: int = FULL
     window: int = 0
     keep_first: int = 0
+    values: bool = True
 
     @property
     def group_key(self) -> Tuple[int, int, int]:
@@ -85,7 +87,7 @@ class StateSpec:
 class LayerCache:
     """What the engine hands a mixer: its layer's pages, the index of their page group, its state."""
     k_pages: Optional[torch.Tensor] = None   # [pages, kv heads, head size / piece, page size, piece] (ops.key_pages_shape)
-    v_pages: Optional[torch.Tensor] = None   # [pages, kv heads, head size, page size] (transposed)
+    v_pages: Optional[torch.Tensor] = None   # [pages, kv heads, head size, page size] (transposed); None: keys alone
     group: int = 0
     state: Optional[torch.Tensor] = None     # [slots, *state shape]
     state_initial: float = 0.0               # what a slot holds when its request starts
@@ -282,6 +284,12 @@ class Mixer(Part):
 class FeedForward(Part):
     def forward(self, ctx, h: torch.Tensor, residual: torch.Tensor) -> None:
         raise NotImplementedError
+
+    def adds_in_place(self, ctx, n: int) -> bool:
+        """For a block that would otherwise have the rows stored (``accepts_store``) and add them in its own next pass:
+        whether in a step of n rows this feed-forward's last pass reads and writes whole rows anyway, so that adding them
+        into the residual there is the cheaper way."""
+        return False
 
 
 class Block(Part):

@@ -246,3 +246,50 @@ class SandwichBlock(Block):
         made, slices = self.ffn.forward(ctx, rows, y, store=True) or (y, 1)
         self.norm2b.add_normed(ctx, made, x, slices=slices, then=emit, rounded=handed)
         return handed
+
+
+class ConvNormBlock(Block):
+    """Pre-norm sublayers that read the normed residual plus a convolution of it over time (``ConvolvedNorm``): x += mixer(in1(x)),
+    then x += feed-forward(in2(x)); the feed-forward may be absent.  Both convolutions keep their rows in one slot.  The
+    sublayers write their rows into a 32-bit buffer or leave them in the slices of a product that divides k, and the pass
+    that adds them into the residual is the pass of the norm that reads it next: in2's inside the block, and behind the last
+    sublayer the one of whoever called the block (``forward`` returns what is still to be added, or None)."""
+    replayable = True
+    taped = True
+
+    def __init__(self, in1, mixer: Mixer, in2=None, ffn: Optional[FeedForward] = None, names=("in1", "mix", "in2", "mlp")):
+        for part in (mixer, ffn):
+            if part is not None and not getattr(part, "accepts_store", False):
+                raise ValueError(f"{type(part).__name__} cannot write its rows instead of adding them (accepts_store)")
+        if (ffn is None) != (in2 is None):
+            raise ValueError("a feed-forward and the norm and convolution before it come together")
+        if mixer.state_spec is not None and in1.taps > 1:
+            raise ValueError("the convolutions and the mixer both keep state: a cache layer has one state")
+        self.in1, self.mixer, self.in2, self.ffn = in1, mixer, in2, ffn
+        self.names = tuple(names)
+
+    def children(self) -> Dict[str, Part]:
+        parts = (self.in1, self.mixer, self.in2, self.ffn)
+        return {name: part for name, part in zip(self.names, parts) if part is not None}
+
+    def cache_spec(self) -> Optional[CacheSpec]:
+        return self.mixer.cache_spec
+
+    def state_spec(self) -> Optional[StateSpec]:
+        if self.in1.taps > 1:
+            return StateSpec((1 if self.in2 is None else 2, self.in1.taps - 1, self.in1.width), torch.float32, 0.0)
+        return self.mixer.state_spec
+
+    def forward(self, ctx, x, cache: Optional[LayerCache], pre):
+        """``pre``: the rows the mixer reads (``in1.after``).  Returns ``(y, slices)``, the last sublayer's rows that are still to
+        be added into x, or None if they have been."""
+        n, width = x.shape
+        y = ctx.buffer("sublayer_y", (n, width), torch.float32)
+        made = self.mixer.forward(ctx, pre, y, cache, store=True) or (y, 1)
+        if self.ffn is None:
+            return made
+        h = self.in2.after(ctx, x, cache, *made, out_name="h2")
+        if self.ffn.adds_in_place(ctx, n):
+            self.ffn.forward(ctx, h, x)
+            return None
+        return self.ffn.forward(ctx, h, y, store=True) or (y, 1)

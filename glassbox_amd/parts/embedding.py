@@ -3,6 +3,7 @@
 the embedding table when tied, model.rs:190-192)."""
 from __future__ import annotations
 
+import math
 from typing import Dict, Optional
 
 import torch
@@ -36,6 +37,22 @@ class Embedding(Part):
             if out.dim() != 2:
                 raise ValueError("a normed embedding fills one residual, not several streams")
             self.norm.in_place(ctx, out)
+
+
+class SinusoidEmbedding(Embedding):
+    """The token's row (times ``scale``) plus a vector of its position p: channels 2i and 2i + 1 are sine and cosine of
+    p * base^(-2i / width).  Angles are taken in 64-bit as far as whole turns go, sine and cosine in 32-bit."""
+
+    def __init__(self, vocab: int, width: int, base: float = 10000.0, scale: float = 1.0):
+        super().__init__(vocab, width, scale)
+        self.base = float(base)
+        self._turns: Optional[torch.Tensor] = None   # turns a position, a number a pair of channels
+
+    def forward(self, ctx, out):
+        if self._turns is None or self._turns.device != self.table.device:
+            i = torch.arange((self.width + 1) // 2, dtype=torch.float64)
+            self._turns = (self.base ** (-2.0 * i / self.width) / (2.0 * math.pi)).to(self.table.device)
+        ops.embed_sinusoid(self.table, ctx.token_ids, ctx.positions, self._turns, out, self.scale)
 
 
 class PairHashEmbedding(Embedding):

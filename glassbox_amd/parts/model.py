@@ -17,6 +17,7 @@ import torch
 
 from .. import ops
 from .base import CacheSpec, LayerCache, Norm, Normed, Part, PreNormed, StateSpec, TensorSpec
+from .depth import DepthAverage
 from .embedding import Embedding, LMHead
 from .tape import LayerTapes
 
@@ -57,12 +58,19 @@ class DecoderModel(Part):
     def __init__(self, config, embedding: Embedding, blocks: Sequence[Part], schedule: Sequence[LayerCall],
                  final_norm: Norm, head: LMHead, names=("model.embed_tokens", "model.layers.{}", "model.norm", "lm_head"),
                  ignorable: Sequence[str] = (), arg_keys: Optional[Dict[str, str]] = None, sources=None,
-                 streams: Optional[int] = None, passes: Optional[PassEntry] = None, passes_name: str = "loop"):
+                 streams: Optional[int] = None, passes: Optional[PassEntry] = None, passes_name: str = "loop",
+                 depth: Optional[Sequence[DepthAverage]] = None, depth_name: str = "depth{}"):
         self.config = config
         #: what is added to the residual where a pass over a repeated run begins (``LayerCall.enter``), or None
         self.passes, self.passes_name = passes, passes_name
         if passes is not None and streams is not None:
             raise ValueError("a residual of several streams has no pass entries")
+        #: one ``DepthAverage`` a schedule entry: what goes on behind it is a sum over all results so far.  The blocks are
+        #: then ``ConvNormBlock``s (or anything with ``in1.after`` and a ``forward`` that returns what is still to be added)
+        self.depth, self.depth_name = None if depth is None else list(depth), depth_name
+        if self.depth is not None and (streams is not None or passes is not None or len(self.depth) != len(schedule)
+                                       or any(a.inputs != i + 2 for i, a in enumerate(self.depth))):
+            raise ValueError("sums over depth: one for every schedule entry, over its number + 2 inputs, on a single residual")
         #: None: one residual [n, width]; a number: the residual is so many streams, [streams, n, width], which the
         #: embedding fills alike and the blocks and the final norm take as such (parts.streams)
         self.streams = streams
@@ -91,6 +99,8 @@ class DecoderModel(Part):
         out[self.names[3]] = self.head
         if self.passes is not None:
             out[self.passes_name] = self.passes
+        for i, average in enumerate(self.depth or ()):
+            out[self.depth_name.format(i)] = average
         return out
 
     def source_of(self, name: str):
@@ -134,6 +144,8 @@ class DecoderModel(Part):
     # the step ---------------------------------------------------------------------
     def forward(self, ctx, caches: Sequence[LayerCache]) -> torch.Tensor:
         """Runs the tokens of ``ctx`` through every scheduled layer; logits [wanted, vocab] float32."""
+        if self.depth is not None:
+            return self._forward_averaged(ctx, caches)
         shape = (ctx.n, self.width) if self.streams is None else (self.streams, ctx.n, self.width)
         embedded = None
         keep = self.passes is not None and self.passes.add_embedding
@@ -194,6 +206,36 @@ class DecoderModel(Part):
             return self.head.forward(ctx, pre.rows, prepared=pre if isinstance(pre, PreNormed) else None)
         rows = self.final_norm.forward(ctx, x, rows=ctx.want, out_name="h_out")
         return self.head.forward(ctx, rows)
+
+    def _forward_averaged(self, ctx, caches: Sequence[LayerCache]) -> torch.Tensor:
+        """The same for a model with sums over depth.  The step's rows keep every layer's result: x[i + 1] is the residual that
+        layer i reads and adds into, X_(i + 1) from then on, and the sum behind it begins x[i + 2].  One pass over the rows
+        adds a layer's last sublayer, forms the sum and makes the rows that the next layer's mixer reads."""
+        x = ctx.buffer("x_by_depth", (len(self.schedule) + 2, ctx.n, self.width), torch.float32)
+        self.embedding.forward(ctx, x[:2])
+        if self._taped is None:
+            self._taped = [b.all_taped() for b in self.blocks]
+        tapes = None
+        if getattr(ctx, "layer_tapes", False) and any(self._taped):
+            tapes = LayerTapes(ctx, ctx.workspace.tape_sites, self.loads, moving=True)
+        cache_of = lambda call: caches[call.cache] if call.cache is not None else None
+        h = self.blocks[self.schedule[0].block].in1.after(ctx, x[1], cache_of(self.schedule[0]))
+        for i, call in enumerate(self.schedule):
+            block, cache = self.blocks[call.block], cache_of(call)
+            if tapes is not None and self._taped[call.block]:
+                made = tapes.forward(i, block, x[i + 1], cache, {"pre": h})
+            else:
+                made = block.forward(ctx, x[i + 1], cache, pre=h)
+            y, slices = made if made is not None else (None, 1)
+            if i + 1 < len(self.schedule):
+                after = self.schedule[i + 1]
+                h = self.blocks[after.block].in1.after(ctx, x[i + 1], cache_of(after), y, slices,
+                                                       self.depth[i].spec(x, x[i + 2]))
+            else:
+                self.depth[i].forward(ctx, x[i + 1], x, x[i + 2], y, slices)
+        if ctx.want.numel() == 0:
+            return ctx.buffer("logits", (0, self.vocab_size), torch.float32)
+        return self.head.forward(ctx, self.final_norm.forward(ctx, x[-1], rows=ctx.want, out_name="h_out"))
 
     def _head_takes_prepared(self, ctx) -> bool:
         """Whether the product that ends the last block may prepare the final norm for the vocabulary product: every

@@ -17,7 +17,9 @@ Other routers and units are options of the same part: ``scoring="softmax"`` (s =
 ``renorm=False`` (a_e = scale * s_e as it stands); ``groups=(count, keep)`` (the experts form ``count`` equal runs of
 neighbours, and only experts of the ``keep`` runs whose best s + correction is largest can be chosen);
 ``unit="relu2"`` (an expert is W_down relu(W_up h)^2: one matrix in, no gate half); ``shared_gate=False`` (the shared
-expert's result is added as it is).
+expert's result is added as it is); ``scoring="chosen"`` (the ``top`` largest of the logits themselves, with ``bias`` z = W_router
+h + ``router.b``, and the softmax over the chosen logits alone as weights); ``unit="clamped"`` (g = min(W_gate h, limit), u =
+clamp(W_up h, -limit, limit), y = W_down (g sigmoid(alpha g) (u + 1))).
 """
 from __future__ import annotations
 
@@ -26,7 +28,7 @@ from typing import Dict, Optional
 import torch
 
 from .. import ops
-from .base import FeedForward, TensorSpec, product, split_workspace
+from .base import FeedForward, TensorSpec, product, product_in_slices, split_workspace
 
 
 class RoutedExperts(FeedForward):
@@ -36,11 +38,18 @@ class RoutedExperts(FeedForward):
 
     def __init__(self, width: int, n_experts: int, top: int, expert_ff: int, router_scale: float = 1.0,
                  shared_ff: int = 0, correction: bool = True, scoring: str = "sigmoid", renorm: bool = True,
-                 groups=None, unit: str = "swiglu", shared_gate: bool = True):
+                 groups=None, unit: str = "swiglu", shared_gate: bool = True, bias: bool = False, limit: Optional[float] = None,
+                 alpha: float = 1.702):
         if not 1 <= top <= n_experts:
             raise ValueError(f"{top} experts a token out of {n_experts}")
-        if scoring not in ("sigmoid", "softmax") or unit not in ("swiglu", "relu2"):
-            raise ValueError("scoring: sigmoid | softmax; unit: swiglu | relu2")
+        if scoring not in ("sigmoid", "softmax", "chosen") or unit not in ("swiglu", "relu2", "clamped"):
+            raise ValueError("scoring: sigmoid | softmax | chosen; unit: swiglu | relu2 | clamped")
+        if scoring == "chosen" and (correction or groups or not renorm):
+            raise ValueError("a choice by the logits themselves has no correction and no groups, and its weights add up to the scale")
+        if bias and scoring != "chosen":
+            raise ValueError("a bias on the router's logits goes with the choice by them (scoring='chosen')")
+        if unit == "clamped" and not (limit is not None and limit > 0):
+            raise ValueError(f"clamped units need a positive limit, got {limit}")
         self.width, self.n_experts, self.top, self.expert_ff = width, int(n_experts), int(top), int(expert_ff)
         self.router_scale, self.shared_ff, self.has_correction = float(router_scale), int(shared_ff), bool(correction)
         self.scoring, self.renorm, self.unit, self.shared_gate = scoring, bool(renorm), unit, bool(shared_gate)
@@ -50,12 +59,14 @@ class RoutedExperts(FeedForward):
             if count < 1 or n_experts % count or not 1 <= keep <= count or keep * (n_experts // count) < top:
                 raise ValueError(f"{n_experts} experts in {count} groups of which {keep} are kept, {top} experts a token")
         self.inter = self.n_experts * self.expert_ff + self.shared_ff
-        self.halves = 2 if unit == "swiglu" else 1      # matrices on the way in: gate and up, or up alone
+        self.halves = 1 if unit == "relu2" else 2      # matrices on the way in: gate and up, or up alone
+        self.has_bias = bool(bias)
+        self.gate_unit = (float(limit), float(alpha), 1.0) if unit == "clamped" else ops.SILU_UNIT   # (limit, alpha, plus)
         self.w_router = self.correction = self.w_gate_up = self.w_down = None
 
     def tensor_specs(self) -> Dict[str, TensorSpec]:
         specs: Dict[str, TensorSpec] = {}
-        ins = ("gate", "up") if self.unit == "swiglu" else ("up",)
+        ins = ("gate", "up") if self.halves == 2 else ("up",)
         for e in range(self.n_experts):
             for m in ins:
                 specs[f"e{e}.{m}"] = TensorSpec((self.expert_ff, self.width))
@@ -63,6 +74,8 @@ class RoutedExperts(FeedForward):
         specs["router"] = TensorSpec((self.n_experts, self.width))
         if self.has_correction:
             specs["correction"] = TensorSpec((self.n_experts,), kind="f32", init="normal")
+        if self.has_bias:
+            specs["router.b"] = TensorSpec((self.n_experts,), kind="f32", init="normal")
         if self.shared_ff:
             for m in ins:
                 specs[f"shared.{m}"] = TensorSpec((self.shared_ff, self.width))
@@ -74,7 +87,7 @@ class RoutedExperts(FeedForward):
     def load(self, tensors):
         names = [f"e{e}" for e in range(self.n_experts)]
         shared = ["shared"] if self.shared_ff else []
-        ins = ("gate", "up") if self.unit == "swiglu" else ("up",)
+        ins = ("gate", "up") if self.halves == 2 else ("up",)
         # every expert's gate rows, then their up rows, then the shared expert's gate and up rows (with one matrix in: the
         # experts' up rows, then the shared expert's)
         self.w_gate_up = torch.cat([tensors[f"{n}.{m}"] for m in ins for n in names] +
@@ -82,7 +95,9 @@ class RoutedExperts(FeedForward):
         self.w_down = torch.cat([tensors[f"{n}.down"] for n in names + shared], 1).contiguous()
         router = [tensors["router"]] + ([tensors["shared.sg"]] if self.shared_ff and self.shared_gate else [])
         self.w_router = torch.cat(router, 0).contiguous()
-        self.correction = tensors["correction"].contiguous() if self.has_correction else None
+        # what the route kernel adds before it chooses: to the scores, or (scoring "chosen") to the logits
+        added = "correction" if self.has_correction else "router.b" if self.has_bias else None
+        self.correction = tensors[added].contiguous() if added is not None else None
 
     def streamed_matrices(self):
         return [self.w_router, self.w_gate_up, self.w_down]
@@ -96,6 +111,8 @@ class RoutedExperts(FeedForward):
         return out
 
     def forward(self, ctx, h, residual, store: bool = False):
+        """Adds the experts' rows into ``residual``; with ``store`` writes them there instead (float32 either way) or leaves
+        them in slices, and returns what ``product_in_slices`` does."""
         n, E = h.shape[0], self.n_experts
         cols = E + (1 if self.shared_ff else 0)
         z = ctx.buffer("moe_z", (n, self.w_router.shape[0]), torch.float32)
@@ -106,18 +123,23 @@ class RoutedExperts(FeedForward):
         shared = False if not self.shared_ff else True if self.shared_gate else "whole"
         count, keep = self.groups if self.groups is not None else (0, 0)
         ops.moe_route(z, E, self.correction, self.top, self.router_scale, shared, combine, ids, weights,
-                      softmax=self.scoring == "softmax", renorm=self.renorm, groups=count, keep_groups=keep)
+                      softmax="chosen" if self.scoring == "chosen" else self.scoring == "softmax", renorm=self.renorm, groups=count, keep_groups=keep)
         if self.routed(ctx, n):
             return self._routed(ctx, h, residual, store, combine, ids, weights)
         gate_up = ctx.buffer("moe_gate_up", (n, self.halves * self.inter), torch.float32)
         product(ctx, h, self.w_gate_up, gate_up)
         act = ctx.buffer("act", (n, self.inter), ctx.dtype)
-        if self.unit == "swiglu":
-            ops.moe_gated_units(gate_up, combine, act, E, self.expert_ff)
+        if self.halves == 2:
+            ops.moe_gated_units(gate_up, combine, act, E, self.expert_ff, self.gate_unit)
         else:
             ops.moe_relu2_units(gate_up, combine, act, E, self.expert_ff)
-        product(ctx, act, self.w_down, residual, accumulate=not store)
+        if store:   # the caller's pass over the rows adds the slices of a product that divides k
+            return product_in_slices(ctx, act, self.w_down, residual)
+        product(ctx, act, self.w_down, residual, accumulate=True)
         return None
+
+    def adds_in_place(self, ctx, n: int) -> bool:
+        return self.routed(ctx, n)   # (the pass that adds up the chosen experts' rows)
 
     def routed(self, ctx, n: int) -> bool:
         """Whether a step of n tokens runs the experts on their own tokens: where the sorted rows, every expert's last
@@ -138,9 +160,9 @@ class RoutedExperts(FeedForward):
         tile_map = ctx.buffer("moe_tiles", (tiles, 3), torch.int32)
         ops.moe_sort(ids, E, tile_rows, counts, rows, pos, tile_map)
         act = ctx.buffer("act", (entries, ff), torch.bfloat16)
-        if self.unit == "swiglu":
+        if self.halves == 2:
             ops.gemm_grouped(h, rows, self.w_gate_up, ff * self.w_gate_up.stride(0), 2 * ff, tile_map, tile_rows, act,
-                             silu_mul=True, up_offset=E * ff)
+                             silu_mul=True, up_offset=E * ff, unit=self.gate_unit)
         else:   # the unit in a pass of its own over the experts' rows, in place
             ops.gemm_grouped(h, rows, self.w_gate_up, ff * self.w_gate_up.stride(0), ff, tile_map, tile_rows, act)
             ops.moe_relu2_units(act, None, act, 0, ff)
@@ -150,7 +172,9 @@ class RoutedExperts(FeedForward):
         if self.shared_ff:
             act_shared = ctx.buffer("moe_act_shared", (n, self.shared_ff), torch.bfloat16)
             w = self.w_gate_up[self.halves * E * ff:]
-            if self.unit == "swiglu":
+            if self.unit == "clamped":
+                ops.gemm_glu(h, w, act_shared, *self.gate_unit)
+            elif self.unit == "swiglu":
                 ops.gemm(h, w, act_shared, silu_mul=True, workspace=split_workspace(ctx, n, 2 * self.shared_ff, d))
             else:
                 ops.gemm(h, w, act_shared, workspace=split_workspace(ctx, n, self.shared_ff, d))

@@ -2,7 +2,8 @@
 (crates/glassbox-core/src/model.rs:94-100).  With ``offset`` the checkpoint holds the weight minus ``offset`` and
 g = offset + w, added in 32-bit when the weights are loaded and kept in 32-bit.  ``ScalarRMSNorm`` has one number for all
 coordinates and can also norm a sublayer's *output* on its way into the residual.  ``TanhNorm`` computes no statistic
-of the row at all: out = tanh(alpha x) * w + b with one number alpha."""
+of the row at all: out = tanh(alpha x) * w + b with one number alpha.  ``GroupRMSNorm`` cuts the row into equal runs of
+channels and divides each by its own root mean square."""
 from __future__ import annotations
 
 from typing import Dict, Optional, Tuple
@@ -127,3 +128,36 @@ class TanhNorm(Norm):
         """x += norm(y) (both float32; ``slices`` > 1: y is the sum of that many pieces); with ``then`` (the ``spec()`` of
         the norm that reads x next) and ``rounded``: rounded = that norm of the new x."""
         ops.tanh_norm_add(x, y, self.spec(), slices=slices, then=then, h=rounded)
+
+
+class GroupRMSNorm(Norm):
+    """The row cut into ``groups`` equal runs of neighbouring channels, each divided by its own sqrt(mean(run^2) + eps), and the
+    whole multiplied by a weight a channel.  32-bit arithmetic in both precisions."""
+    replayable = True
+    taped = True
+
+    def __init__(self, width: int, groups: int, eps: float):
+        if groups < 1 or width % groups:
+            raise ValueError(f"a row of {width} channels in {groups} equal groups")
+        self.width, self.groups, self.eps = int(width), int(groups), float(eps)
+        self.weight: Optional[torch.Tensor] = None
+
+    def tensor_specs(self) -> Dict[str, TensorSpec]:
+        return {"weight": TensorSpec((self.width,), kind="f32", init="ones")}
+
+    def load(self, tensors):
+        self.weight = tensors["weight"].float().contiguous()
+
+    def problems(self, dtype, page_size):
+        out = []
+        if self.groups > ops.GROUP_NORM_MAX_GROUPS:
+            out.append(("groups", f"{self.groups} is above {ops.GROUP_NORM_MAX_GROUPS}, the most groups the norm's kernel takes"))
+        if self.width > ops.RESIDUAL_ROWS_MAX:
+            out.append(("width", f"{self.width} is above {ops.RESIDUAL_ROWS_MAX}, the widest row the norm's kernel takes"))
+        return out
+
+    def forward(self, ctx, x, rows=None, out_name="h"):
+        m = x.shape[0] if rows is None else rows.numel()
+        out = ctx.buffer(out_name, (m, self.width), ctx.dtype)
+        ops.residual_rows(x, gamma=self.weight, groups=self.groups, eps=self.eps, h=out, rows=rows)
+        return out

@@ -19,7 +19,8 @@ What makes two layers of a kind is decided here, from the parts themselves, and 
 * the walk of the recorded layer added nothing to the step's memo (``ctx.memo``: what a part computes once a step
   for all layers, like the rotation's table, is not among the launches of the layers after it);
 * they are called alike: what the block before prepared of the first norm, whether the block after asks for its
-  norm to be prepared, the kind and shapes of the cache layer, the residual buffer;
+  norm to be prepared, the kind and shapes of the cache layer, the residual buffer (or, in a model that keeps every
+  layer's residual in a buffer of its own, ``moving``, its shape: the residual is then one of the tensors exchanged);
 * their tensors (the attributes of the parts that are tensors, the cache layer's pages and state, the gamma of a
   norm to prepare), listed in the same order, have the same sizes.
 
@@ -161,10 +162,14 @@ class _Site:
         self.key = (self.kind, _call_key(emit, False), _cache_key(cache))
         self.operands = None
 
-    def tensors(self) -> ops.TapeOperands:
-        """The layer's tensors: the block's, the cache layer's, those of the norm it is asked to prepare."""
+    def tensors(self, x: Optional[torch.Tensor] = None) -> ops.TapeOperands:
+        """The layer's tensors: the block's, the cache layer's, those of the norm it is asked to prepare; with ``x`` also
+        the residual it works on in this step."""
         if self.operands is None:
-            self.operands = ops.TapeOperands(tensors_of(self.block) + tensors_of(self.cache) + tensors_of(self.emit))
+            self.operands = ops.TapeOperands(tensors_of(self.block) + tensors_of(self.cache) + tensors_of(self.emit),
+                                             places=0 if x is None else 1)
+        if x is not None:
+            self.operands.place(0, x)
         return self.operands
 
     def forget(self) -> None:
@@ -180,10 +185,11 @@ class _Record:
 
 class LayerTapes:
     """The recorded layers of one step.  ``sites`` lives with the engine's workspace (one entry per schedule entry);
-    ``loads`` counts the times the model's weights were loaded: a site of another count holds tensors that are gone."""
+    ``loads`` counts the times the model's weights were loaded: a site of another count holds tensors that are gone.
+    ``moving``: every layer works on a residual buffer of its own."""
 
-    def __init__(self, ctx, sites: Dict[int, _Site], loads: int = 0):
-        self.ctx, self.sites, self.loads = ctx, sites, loads
+    def __init__(self, ctx, sites: Dict[int, _Site], loads: int = 0, moving: bool = False):
+        self.ctx, self.sites, self.loads, self.moving = ctx, sites, loads, moving
         self.records: Dict[tuple, _Record] = {}
         self._x = self._x_key = None
         self._pre = self._pre_key = None
@@ -197,14 +203,15 @@ class LayerTapes:
         site.bind(cache, kwargs.get("emit"))
         pre = kwargs.get("pre")
         if x is not self._x:
-            self._x, self._x_key = x, (x.data_ptr(), tuple(x.shape))
+            self._x, self._x_key = x, (0 if self.moving else x.data_ptr(), tuple(x.shape))
+        moved = x if self.moving else None
         if pre is not self._pre or self._pre_key is None:      # a replayed layer hands on what the recorded one did
             self._pre, self._pre_key = pre, _call_key(pre, True)
         key = (site.key, self._pre_key, self._x_key)
         epoch = ctx.workspace.epoch
         rec = self.records.get(key)
         if rec is not None and rec.epoch == epoch:
-            target = site.tensors()
+            target = site.tensors(moved)
             if target.sizes == rec.operands.sizes and rec.operands.maps_onto(target):
                 ops.run_tape(rec.tape, rec.operands, target)
                 return rec.result
@@ -224,6 +231,6 @@ class LayerTapes:
         # a walk that added to the step's memo did work that is done once a step (the rotation's table): its launches
         # are not those of the layers after it, so the next layer of the kind is walked and recorded instead
         if tape.usable and len(tape) and ctx.workspace.epoch == epoch and len(ctx.memo) == memo:
-            self.records[key] = _Record(tape, site.tensors(), result, epoch)
+            self.records[key] = _Record(tape, site.tensors(moved), result, epoch)
             ops.TAPE_COUNTS["recorded_layers"] += 1
         return result
