@@ -3,7 +3,7 @@
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch 8] [--context 4096] [--layers 24]
                     [--shapes smollm2-1.7b|smollm2-360m|llama-3-8b] [--reps 3]
-    python bench.py --design sagalorn|dekinex|vumalix|tekilix [--design-sizes 360m,1.7b] [--layers 12] [--batch 8] [--context 4096]
+    python bench.py --design sagalorn|dekinex|vumalix|tekilix|zakusun [--design-sizes 360m,1.7b] [--layers 12] [--batch 8] [--context 4096]
 
 ``--design sagalorn`` is another measurement with a line of its own: prefill and decode throughput of Sagalorn models
 whose layers have the sizes of the named shapes (a third of the layers each retention, windowed attention with kept
@@ -28,6 +28,11 @@ keys as values, stretched rotation and learned sinks), both within runs of 1,024
 sublayer, and in every layer routed experts of squared-ReLU units (eight in four groups of which two are kept, two a
 token, each 3/8 of the Llama's intermediate size, and a shared one of 3/4: as many multiply-adds a token as the Llama's
 three matrices).
+
+``--design zakusun`` does the same for Zakusun models: attention through a cached latent of a quarter of the width (heads of
+the Llama's head size, a sink a head, a gate a channel), norms in four groups each behind a convolution over four tokens,
+a weighted sum over all layers so far behind every layer, and in every layer routed experts of clamped gated units (eight, two
+a token, each half of the Llama's intermediate size: as many multiply-adds a token as the Llama's feed-forward).
 
 A step is one decode step of the whole batch through the path that greedy generation uses: ``Engine.step``
 (which replays steps of single tokens from HIP graphs) and the device sampler (``sampling.greedy_pending``), the
@@ -137,8 +142,21 @@ def tekilix_like(shapes: dict, layers: int, run: int = 1024, experts: int = 8, t
                 embedding={"scale": 1.0}, logit_scale=1.0, layers=[kinds[i % 2] for i in range(layers)])
 
 
+def zakusun_like(shapes: dict, layers: int, experts: int = 8, top: int = 2) -> dict:
+    """A Zakusun configuration with the widths of a Llama one: a latent of a quarter of the width, routed experts in every layer
+    with as many multiply-adds a token as the Llama's feed-forward."""
+    d, H = shapes["hidden_size"], shapes["num_attention_heads"]
+    hd = shapes.get("head_dim") or d // H
+    layer = {"type": "latent_attention",
+             "mixer": {"heads": H, "dim": hd, "vdim": hd, "kv_rank": d // 4 // 8 * 8, "scale": hd ** -0.5},
+             "mlp": {"kind": "moe", "expert": {"ff": shapes["intermediate_size"] // top // 8 * 8, "limit": 7.0},
+                     "router": {"experts": experts, "top": top}}}
+    return dict(architecture="Zakusun", vocab=shapes["vocab_size"], width=d, norm={"eps": shapes["rms_norm_eps"], "groups": 4},
+                canon={"taps": 4}, logit_scale=1.0, layers=[layer] * layers)
+
+
 DESIGNS = {"sagalorn": ("Sagalorn", sagalorn_like), "dekinex": ("Dekinex", dekinex_like), "vumalix": ("Vumalix", vumalix_like),
-           "tekilix": ("Tekilix", tekilix_like)}
+           "tekilix": ("Tekilix", tekilix_like), "zakusun": ("Zakusun", zakusun_like)}
 
 
 def design_bench(a) -> int:

@@ -68,8 +68,10 @@ def group_norm(x: torch.Tensor, weight: torch.Tensor, groups: int, eps: float) -
     return unit_rms(x.reshape(T, groups, d // groups), eps).reshape(T, d) * weight
 
 
-def with_conv(h: torch.Tensor, taps_w: torch.Tensor) -> torch.Tensor:
-    """h_t + sum_j w[:, j] h_(t - taps + 1 + j), zeros before the first token; taps_w [d, taps]."""
+def with_conv(h: torch.Tensor, taps_w: Optional[torch.Tensor]) -> torch.Tensor:
+    """h_t + sum_j w[:, j] h_(t - taps + 1 + j), zeros before the first token; taps_w [d, taps] (None: no convolution)."""
+    if taps_w is None:
+        return h
     T = h.shape[0]
     taps = taps_w.shape[1]
     y = h.clone()
@@ -184,10 +186,10 @@ def forward(cfg: dict, w: Dict[str, torch.Tensor], tokens: List[int], coarse: bo
     history = [x]
     for i, layer in enumerate(cfg["layers"]):
         name = f"l{i}."
-        h = rnd(with_conv(group_norm(x, w[name + "norm1"], groups, eps), w[name + "canon1"]))
+        h = rnd(with_conv(group_norm(x, w[name + "norm1"], groups, eps), w.get(name + "canon1")))
         x = x + latent_attention(w, name + "mix.", layer["mixer"], eps, h, rnd)
         if layer.get("mlp") is not None:
-            h = rnd(with_conv(group_norm(x, w[name + "norm2"], groups, eps), w[name + "canon2"]))
+            h = rnd(with_conv(group_norm(x, w[name + "norm2"], groups, eps), w.get(name + "canon2")))
             x = x + experts(w, name + "mlp.", layer["mlp"], h, rnd, margins)
         history.append(x)
         x = depth_average(w[name + "dwa"], history)
