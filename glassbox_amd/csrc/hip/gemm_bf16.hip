@@ -132,6 +132,7 @@ struct Groups {
   const int32_t* rows;
   long long w_stride;
   int up_off;
+  int slice_rows;   // rows of C a slice of k (the ring kernel's grouped form)
 };
 
 template <int WM, int WN, int DEPTH, int EPI, bool KFULL, typename CT, bool GROUPED = false>
@@ -437,9 +438,11 @@ template <int LEFT> __device__ __forceinline__ void vm_wait() {
   __builtin_amdgcn_s_waitcnt(0x0F70 | (LEFT & 15) | ((LEFT >> 4) << 14));
 }
 
-template <int EPI, typename CT>
+// GROUPED: as the tiled kernel's (row tiles of 256 rows); a product that divides k writes grp.slice_rows rows a slice.
+template <int EPI, typename CT, bool GROUPED = false>
 __global__ __launch_bounds__(RGM * RGN * 64, 1) void gemm_ring_kernel(const bf16* __restrict__ a, int lda, const bf16* __restrict__ w, int ldw,
-                                                           CT* __restrict__ c, int ldc, int M, int N, int K, int k_slice, Glu glu) {
+                                                           CT* __restrict__ c, int ldc, int M, int N, int K, int k_slice, Groups grp,
+                                                           Glu glu) {
   int bx = blockIdx.x, by = blockIdx.y;
   if (k_slice > 0) {  // split k: workgroup z of a tile sums its own slice of k into its own copy of C
     int z = blockIdx.z;
@@ -448,7 +451,7 @@ __global__ __launch_bounds__(RGM * RGN * 64, 1) void gemm_ring_kernel(const bf16
     // different operand pieces a k-step among its 32 workgroups); numbered anew, it holds an eighth of the grid in
     // a row: one slice, some row tiles, all column tiles (4 + 8 pieces), which its cache then serves.
     const int gx = gridDim.x, gy = gridDim.y, total = gx * gy * gridDim.z;
-    if (total % 8 == 0) {
+    if (!GROUPED && total % 8 == 0) {
       const int id = bx + gx * (by + gy * z), anew = (id % 8) * (total / 8) + id / 8;
       bx = anew % gx;
       by = (anew / gx) % gy;
@@ -456,22 +459,32 @@ __global__ __launch_bounds__(RGM * RGN * 64, 1) void gemm_ring_kernel(const bf16
     }
     a += (size_t)z * k_slice;
     w += (size_t)z * k_slice;
-    c += (size_t)z * M * ldc;
+    c += (size_t)z * (GROUPED ? grp.slice_rows : M) * ldc;
     K = min(k_slice, K - z * k_slice);
   }
   __shared__ __attribute__((aligned(16))) bf16 As[RING_STAGES][RBM * RBK];
   __shared__ __attribute__((aligned(16))) bf16 Ws[RING_STAGES][RBN * RBK];
   const int tid = threadIdx.x, lane = tid % 64, wave = tid / 64;
   const int wm = wave / RGN, wn = wave % RGN;
-  const int m0 = by * RBM;
+  int m0 = by * RBM;
   const int half = N / 2;  // EPI_SILU_MUL: number of gate rows
+  int up_off = half;       // and how far behind its gate row an up row lies
+  if constexpr (GROUPED) {
+    const int32_t* tile = grp.map + 3 * by;
+    const int group = tile[0];
+    if (group < 0) return;   // (the whole workgroup)
+    m0 = tile[1];
+    M = tile[2];
+    w += (size_t)group * grp.w_stride;
+    up_off = grp.up_off;
+  }
   // row of W behind row r of the workgroup's W tile (r = wn * 64 + j * 32 + column); with EPI_SILU_MUL a wave's
   // first column tile holds gate rows and its second the up rows that belong to them
   auto w_row = [&](int r) -> int {
     if (EPI == EPI_SILU_MUL) {
       const int j = (r % (RTN * 32)) / 32;  // column tile of its wave: even ones hold gate rows, odd ones their up rows
       const int n = bx * (RBN / 2) + (r / (RTN * 32)) * (RTN / 2 * 32) + (j / 2) * 32 + r % 32;
-      return n < half ? (j % 2 ? half + n : n) : 0;
+      return n < half ? (j % 2 ? up_off + n : n) : 0;
     }
     return min(bx * RBN + r, N - 1);
   };
@@ -481,7 +494,11 @@ __global__ __launch_bounds__(RGM * RGN * 64, 1) void gemm_ring_kernel(const bf16
 #pragma unroll
   for (int t = 0; t < RLA; ++t) {
     const int row = (wave * RLA + t) * 16 + lane / 4, piece = (lane % 4) ^ ((row >> 2) & 3);
-    asrc[t] = a + (size_t)min(m0 + row, M - 1) * lda + piece * 8;
+    int arow = min(m0 + row, M - 1);
+    if constexpr (GROUPED) {
+      if (grp.rows) arow = grp.rows[arow];
+    }
+    asrc[t] = a + (size_t)arow * lda + piece * 8;
   }
 #pragma unroll
   for (int t = 0; t < RLW; ++t) {
@@ -654,7 +671,7 @@ int launch_ring(const bf16* a, int lda, const bf16* w, int ldw, CT* c, int ldc, 
   const int cols = EPI == EPI_SILU_MUL ? N / 2 : N, bn = EPI == EPI_SILU_MUL ? RBN / 2 : RBN;
   const dim3 grid((cols + bn - 1) / bn, (M + RBM - 1) / RBM), block(RGM * RGN * 64);
   GB_REQUIRE(grid.y <= 65535, "gemm_bf16: M=%d needs more than 65535 row tiles", M);
-  hipLaunchKernelGGL((gemm_ring_kernel<EPI, CT>), grid, block, 0, stream, a, lda, w, ldw, c, ldc, M, N, K, 0, glu);
+  hipLaunchKernelGGL((gemm_ring_kernel<EPI, CT>), grid, block, 0, stream, a, lda, w, ldw, c, ldc, M, N, K, 0, Groups{}, glu);
   return launched("gemm_bf16 (ring)");
 }
 
@@ -1084,7 +1101,7 @@ int launch_split(const bf16* a, int lda, const bf16* w, int ldw, CT* c, int ldc,
   }
   if (ring)
     hipLaunchKernelGGL((gemm_ring_kernel<EPI_STORE, float>), dim3((N + RBN - 1) / RBN, (M + RBM - 1) / RBM, plan.slices), dim3(RGM * RGN * 64),
-                       0, stream, a, lda, w, ldw, ws, N, M, N, K, plan.k_slice, Glu{});
+                       0, stream, a, lda, w, ldw, ws, N, M, N, K, plan.k_slice, Groups{}, Glu{});
 #define GB_S(WM, FULL)                                                                                                   \
   if (!ring && !streams && (plan.bm == 64 * WM) && kfull == FULL)                                                                   \
     hipLaunchKernelGGL((gemm_tiled_kernel<WM, 2, 1, EPI_STORE, FULL, float>), grid, block, 0, stream, a, lda, w, ldw, ws, \
@@ -1881,12 +1898,14 @@ extern "C" int gb_gemm_bf16_glu(const void* a, int lda, const void* w, int ldw, 
 // numbers for each of `tiles` row tiles of `tile_rows` (64 or 128) rows, as a kernel on the device laid them out; a
 // group's W starts w_stride elements behind the one before.  Epilogue 0 stores (bfloat16 or float32), 2 forms
 // silu(gate) * up, or the clamped unit (limit, alpha, plus: see Glu), from the N / 2 gate rows of a group and the up rows
-// up_off rows behind them.
+// up_off rows behind them.  Tiles of 256 rows go through the ring kernel, which may divide k into `slices` (float32 results
+// without an epilogue): slice z's sums lie z * slice_rows rows further on in C.
 extern "C" int gb_gemm_bf16_grouped(const void* a, int lda, const int32_t* rows, const void* w, int ldw, long long w_stride,
                                     int up_off, void* c, int ldc, int c_dtype, const int32_t* map, int tiles, int tile_rows,
-                                    int N, int K, int epilogue, float limit, float alpha, float plus, hipStream_t stream) {
+                                    int N, int K, int epilogue, float limit, float alpha, float plus, int slices, int slice_rows,
+                                    hipStream_t stream) {
   GB_REQUIRE(limit > 0.f, "gemm_bf16_grouped: the unit's limit must be positive");
-  GB_REQUIRE(tiles >= 0 && N > 0 && K > 0 && (tile_rows == 64 || tile_rows == 128), "gemm_bf16_grouped: bad sizes tiles=%d of %d rows, N=%d K=%d",
+  GB_REQUIRE(tiles >= 0 && N > 0 && K > 0 && (tile_rows == 64 || tile_rows == 128 || tile_rows == 256), "gemm_bf16_grouped: bad sizes tiles=%d of %d rows, N=%d K=%d",
              tiles, tile_rows, N, K);
   GB_REQUIRE(K % 8 == 0 && ldw % 8 == 0 && lda % 8 == 0 && w_stride % 8 == 0 && lda >= K && ldw >= K,
              "gemm_bf16_grouped: the inner size, the row strides and the distance between groups (%d, %d, %d, %lld) must keep rows 16-byte aligned",
@@ -1898,10 +1917,26 @@ extern "C" int gb_gemm_bf16_grouped(const void* a, int lda, const int32_t* rows,
   const int cols = epilogue == EPI_SILU_MUL ? N / 2 : N, bn = epilogue == EPI_SILU_MUL ? 64 : 128;
   GB_REQUIRE(ldc >= cols && tiles <= 65535, "gemm_bf16_grouped: rows of C are shorter than the product's, or more than 65535 row tiles");
   if (tiles == 0) return 0;
-  const Groups grp{map, rows, w_stride, up_off};
-  const dim3 grid((cols + bn - 1) / bn, tiles), block(256);
+  GB_REQUIRE(slices >= 1 && (slices == 1 || (tile_rows == 256 && epilogue == EPI_STORE && c_dtype == kF32 && slice_rows > 0)),
+             "gemm_bf16_grouped: %d slices of k go with tiles of 256 rows and float32 results", slices);
+  const Groups grp{map, rows, w_stride, up_off, slice_rows};
   const bf16* A = (const bf16*)a;
   const bf16* W = (const bf16*)w;
+  if (tile_rows == 256) {
+    GB_REQUIRE(ring_takes(a, lda, w, ldw, K), "gemm_bf16_grouped: tiles of 256 rows need an inner size of whole 32s, %d and more, not %d", RBK * RING_STAGES, K);
+    const int k_slice = slices == 1 ? 0 : (K / RBK + slices - 1) / slices * RBK;
+    GB_REQUIRE(slices == 1 || (slices - 1) * (long long)k_slice < K, "gemm_bf16_grouped: %d slices of k=%d leave some without a step", slices, K);
+    const int rbn = epilogue == EPI_SILU_MUL ? RBN / 2 : RBN;
+    const dim3 rgrid((cols + rbn - 1) / rbn, tiles, slices), rblock(RGM * RGN * 64);
+    if (epilogue == EPI_SILU_MUL)
+      hipLaunchKernelGGL((gemm_ring_kernel<EPI_SILU_MUL, bf16, true>), rgrid, rblock, 0, stream, A, lda, W, ldw, (bf16*)c, ldc, 0, N, K, 0, grp, Glu{limit, alpha, plus});
+    else if (c_dtype == kF32)
+      hipLaunchKernelGGL((gemm_ring_kernel<EPI_STORE, float, true>), rgrid, rblock, 0, stream, A, lda, W, ldw, (float*)c, ldc, 0, N, K, k_slice, grp, Glu{});
+    else
+      hipLaunchKernelGGL((gemm_ring_kernel<EPI_STORE, bf16, true>), rgrid, rblock, 0, stream, A, lda, W, ldw, (bf16*)c, ldc, 0, N, K, 0, grp, Glu{});
+    return launched("gemm_bf16 (grouped ring)");
+  }
+  const dim3 grid((cols + bn - 1) / bn, tiles), block(256);
   const bool kfull = K % TBK == 0;
 #define GB_G(WM, EPI, CT, FULL)                                                                                              \
   if (tile_rows == 64 * WM && epilogue == EPI && kfull == FULL && (EPI == EPI_SILU_MUL || (c_dtype == kF32) == std::is_same_v<CT, float>)) \

@@ -106,6 +106,26 @@ __global__ __launch_bounds__(THREADS) void residual_rows_kernel(RowPass p, T* __
   const int t = blockIdx.x;
   float* xr = p.x + (size_t)(p.rows ? p.rows[t] : t) * d;
   f32x4 v[WORDS];
+  const int K = p.taps - 1;
+  int pos = 0;
+  float* st = nullptr;
+  if (p.conv_w && K > 0) {
+    const int seq = p.tok_seq[t];
+    pos = p.pos0[seq];
+    st = p.state + (size_t)p.state_slots[seq] * p.slot_stride;
+  }
+  // a step of single tokens is a few of these workgroups, whose time is round trips to memory: what the convolution reads (up
+  // to four taps) is on its way from the start
+  constexpr int AHEAD = WORDS == 1 ? 4 : 0;
+  f32x4 ahead_w[AHEAD > 0 ? AHEAD : 1], ahead_s[AHEAD > 0 ? AHEAD : 1];
+  const bool ahead = AHEAD > 0 && p.conv_w && p.taps <= AHEAD && 4 * (int)threadIdx.x < d;
+  if (AHEAD > 0 && ahead) {
+#pragma unroll
+    for (int j = 0; j < AHEAD; ++j) {
+      if (j < p.taps) ahead_w[j] = load4(p.conv_w + (size_t)j * d + 4 * threadIdx.x);
+      if (j < K) ahead_s[j] = load4(st + (size_t)j * d + 4 * threadIdx.x);
+    }
+  }
 #pragma unroll
   for (int i = 0; i < WORDS; ++i) {
     const int c = (threadIdx.x + i * THREADS) * 4;
@@ -122,7 +142,7 @@ __global__ __launch_bounds__(THREADS) void residual_rows_kernel(RowPass p, T* __
     f32x4 acc[WORDS];
 #pragma unroll
     for (int i = 0; i < WORDS; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
+#pragma unroll(WORDS == 1 ? 8 : 4)
     for (int j = 0; j < p.count; ++j) {
       const float a = p.coef[j];
       const float* hr = p.hist + (size_t)j * p.hist_stride + (size_t)t * d;
@@ -157,14 +177,6 @@ __global__ __launch_bounds__(THREADS) void residual_rows_kernel(RowPass p, T* __
   __syncthreads();
   if (p.scales && (int)threadIdx.x < p.groups) p.scales[(size_t)t * p.groups + threadIdx.x] = inv[threadIdx.x];
   if (!h) return;
-  const int K = p.taps - 1;
-  int pos = 0;
-  float* st = nullptr;
-  if (p.conv_w && K > 0) {
-    const int seq = p.tok_seq[t];
-    pos = p.pos0[seq];
-    st = p.state + (size_t)p.state_slots[seq] * p.slot_stride;
-  }
 #pragma unroll
   for (int i = 0; i < WORDS; ++i) {
     const int q = threadIdx.x + i * THREADS, c = 4 * q;
@@ -175,20 +187,23 @@ __global__ __launch_bounds__(THREADS) void residual_rows_kernel(RowPass p, T* __
 #pragma unroll
     for (int e = 0; e < 4; ++e) cur[e] = v[i][e] * r * g[e];
     f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-    if (p.conv_w) {
-      for (int j = 0; j < p.taps; ++j) {
-        f32x4 in = cur;
-        if (j < K) {   // index j of the slot is the row of position pos - (K - j); it moves to index j - 1
-          in = load4(st + (size_t)j * d + c);
-          if (j > 0) store4(st + (size_t)(j - 1) * d + c, in);
-          if (pos - (K - j) < 0) in = f32x4{0.f, 0.f, 0.f, 0.f};   // before the request's first token
-        }
-        const f32x4 wj = load4(p.conv_w + (size_t)j * d + c);
-#pragma unroll
-        for (int e = 0; e < 4; ++e) acc[e] = fmaf(wj[e], in[e], acc[e]);
+    // index j of the slot is the row of position pos - (K - j); it moves to index j - 1
+    auto tap = [&](int j, f32x4 in, const f32x4& wj) {
+      if (j < K) {
+        if (j > 0) store4(st + (size_t)(j - 1) * d + c, in);
+        if (pos - (K - j) < 0) in = f32x4{0.f, 0.f, 0.f, 0.f};   // before the request's first token
       }
-      if (K > 0) store4(st + (size_t)(K - 1) * d + c, cur);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) acc[e] = fmaf(wj[e], in[e], acc[e]);
+    };
+    if (AHEAD > 0 && ahead) {
+#pragma unroll
+      for (int j = 0; j < AHEAD; ++j)
+        if (j < p.taps) tap(j, j < K ? ahead_s[j] : cur, ahead_w[j]);
+    } else if (p.conv_w) {
+      for (int j = 0; j < p.taps; ++j) tap(j, j < K ? load4(st + (size_t)j * d + c) : cur, load4(p.conv_w + (size_t)j * d + c));
     }
+    if (p.conv_w && K > 0) store4(st + (size_t)(K - 1) * d + c, cur);
     store4(h + (size_t)t * d + c, cur + acc);
   }
 }

@@ -126,28 +126,35 @@ __global__ void latent_absorb_plain_kernel(const T* __restrict__ q, int ldq, con
 }
 
 // ------------------------------------------------------------------------------------------------ latent_decode
-// Four waves; a step takes 64 latents of the context.  Each wave reads 16 of them from their page straight into MFMA operands
-// (lane (j, c): key j, channels 32 ks + 8 c .. + 7, as the pages' pieces lie), forms the scores of its keys for all columns
-// (a column is a head), and leaves scores and latents in LDS.  Then every wave takes part of the channels of the sums: per 32
-// keys it reads 8 keys x 8 channels a lane and turns them in registers (a pair of words gives two channels' pairs of keys),
-// which makes eight operands of 16 channels, one of each run of eight; the columns' running maximum is formed by each wave for
-// itself, from the same scores in the same order.  Two buffers: one barrier a step.
+// Four waves; a step takes 128 latents of the context.  Each wave reads 32 of them from their pages straight into MFMA
+// operands (lane (j, c): key j, channels 32 ks + 8 c .. + 7, as the pages' pieces lie), forms the scores of its keys for all
+// columns (a column is a head), and leaves scores and latents in LDS.  Then every wave takes part of the sums: per 32 keys it
+// reads 8 keys x 8 channels a lane and turns them in registers (a pair of words gives two channels' pairs of keys), which makes
+// eight operands of 16 channels, one of each run of eight; a column's running maximum is formed by each wave for itself, from
+// the same scores in the same order.  The latents of the next step are on their way meanwhile.
 //   S^T[key, col]     A = 16 keys x 32 channels,       B = 32 channels x 16 columns (the queries, in registers)
 //   O^T[chan, col]    A = 16 channels x 32 keys,       B = 32 keys x 16 columns (the weights, as the lanes form them)
-// KS: k-steps of 32 channels that hold R; CT: tiles of 16 columns.
-template <int KS, int CT>
+// KS: k-steps of 32 channels that hold R (FULL: exactly); CT: tiles of 16 columns.  The sums fall into units of (128 channels, tile of columns);
+// with more waves than units the waves of a unit take its runs of 32 keys in turn, and their sums meet in LDS at the end.
+template <int KS, int CT, bool FULL>
 __global__ __launch_bounds__(256, 1) void latent_decode_kernel(const bf16* __restrict__ q, const bf16* __restrict__ pages,
                                                                const int32_t* __restrict__ tables, int table_stride,
                                                                const int32_t* __restrict__ positions, int H, int R, int P, float scale2,
                                                                int chunk, int splits, float* __restrict__ ws_acc,
                                                                float* __restrict__ ws_ml) {
+  constexpr int KEYS = 128, KT = 2;         // keys a step; tiles of 16 of them a wave
   constexpr int ROW = KS * 32 + 8;          // a latent in LDS, with 16 bytes between rows so that 16 rows' words spread over the banks
-  constexpr int SROW = 68;                  // a column's 64 scores
+  constexpr int SROW = KEYS + 4;            // a column's scores
+  constexpr int OROW = KS * 32 + 4;         // a column's sums, at the end
   constexpr int NB = KS / 4;                // blocks of 128 channels
-  constexpr int UNITS = NB * CT, UPW = (UNITS + 3) / 4;   // (block, column tile) pairs, and how many a wave takes
-  static_assert(UPW == 1 || NB == 4, "a wave's pairs share their block");
-  __shared__ __align__(16) bf16 cbuf[2][64 * ROW];
-  __shared__ __align__(16) float sbuf[2][CT * 16 * SROW];
+  constexpr int UNITS = NB * CT, UPW = (UNITS + 3) / 4;   // units, and how many a wave takes
+  constexpr int PARTS = UNITS >= 4 ? 1 : 4 / UNITS;       // waves that share a unit
+  constexpr int RUNS = KEYS / 32 / PARTS;   // runs of 32 keys a wave takes of a step
+  static_assert(UPW == 1 || NB == 4, "a wave's units share their block");
+  static_assert(CT * 16 * OROW * 4 <= KEYS * ROW * 2, "the sums take the latents' place");
+  __shared__ __align__(16) bf16 cbuf[KEYS * ROW];
+  __shared__ __align__(16) float sbuf[CT * 16 * SROW];
+  __shared__ float lbuf[CT * 16];
   const int row = blockIdx.z, hg = blockIdx.y, split = blockIdx.x;
   const int pos = positions[row];
   const int c0 = split * chunk;
@@ -157,16 +164,24 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(const bf16* __res
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int32_t* table = tables + (size_t)row * table_stride;
 
-  bf16x8 kf[KS];
+  // Nothing is loaded behind a condition: lanes beyond the last key read the last key again (their scores are masked), pieces
+  // beyond the latent's read its last one again (the queries hold zeros there, and such channels' sums go nowhere), columns
+  // beyond the heads the last head.
+  const int pieces = R / 8;
+  bf16x8 kf[KT][KS];
   auto load_tile = [&](int kb) {
-    const int key0 = kb + wave * 16;        // 16 keys in a row lie in one page
-    const bool valid = key0 + j <= last;
-    const int page = key0 <= last ? table[key0 / P] : 0;
-    const bf16* b = pages + (size_t)page * P * R + (size_t)(key0 % P + j) * 8;
 #pragma unroll
-    for (int ks = 0; ks < KS; ++ks) {
-      const int piece = ks * 4 + c;
-      kf[ks] = (valid && piece * 8 < R) ? load8_once(b + (size_t)piece * P * 8) : zero8();
+    for (int t = 0; t < KT; ++t) {
+      const int key0 = min(kb + wave * 16 * KT + 16 * t, last & ~15);        // 16 keys in a row lie in one page
+      const bf16* b = pages + (size_t)table[key0 / P] * P * R;
+      const int slot = key0 % P + min(j, last - key0);
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks) {
+        if (FULL)
+          kf[t][ks] = load8_once(b + (size_t)(ks * 4 * P) * 8 + (c * P + slot) * 8);
+        else
+          kf[t][ks] = load8_once(b + (size_t)(min(ks * 4 + c, pieces - 1) * P + slot) * 8);
+      }
     }
   };
   load_tile(c0);
@@ -174,11 +189,13 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(const bf16* __res
   bf16x8 qf[CT][KS];
 #pragma unroll
   for (int ct = 0; ct < CT; ++ct) {
-    const int head = (hg * CT + ct) * 16 + j;
+    const bf16* qr = q + ((size_t)row * H + min((hg * CT + ct) * 16 + j, H - 1)) * R + 8 * c;
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) {
-      const int ch = ks * 32 + 8 * c;
-      qf[ct][ks] = (head < H && ch < R) ? load8(q + ((size_t)row * H + head) * R + ch) : zero8();
+      if (FULL)
+        qf[ct][ks] = load8(qr + ks * 32);
+      else
+        qf[ct][ks] = ks * 32 + 8 * c < R ? load8(qr + ks * 32) : zero8();
     }
   }
   f32x4 acc[UPW][8];
@@ -190,112 +207,137 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(const bf16* __res
 #pragma unroll
     for (int i = 0; i < 8; ++i) acc[u][i] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
-  const int block = wave % NB;              // this wave's channels: pieces 16 block .. 16 block + 15
+  // this wave's units: block of channels `block` (pieces 16 block .. 16 block + 15) with column tile (unit + 4 u) / NB; its part
+  // of a unit's runs of keys
+  const int unit = wave % (UNITS < 4 ? UNITS : 4), part = wave / (UNITS < 4 ? UNITS : 4);
+  const int block = unit % NB;
 
-  int buf = 0;
-  for (int kb = c0; kb <= last; kb += 64, buf ^= 1) {
-    bf16* cb = cbuf[buf];
-    float* sb = sbuf[buf];
+  for (int kb = c0; kb <= last; kb += KEYS) {
+    f32x4 s[KT][CT];
 #pragma unroll
-    for (int ct = 0; ct < CT; ++ct) {
-      f32x4 s = {0.f, 0.f, 0.f, 0.f};
+    for (int t = 0; t < KT; ++t)
 #pragma unroll
-      for (int ks = 0; ks < KS; ++ks) s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[ks], qf[ct][ks], s, 0, 0, 0);
+      for (int ct = 0; ct < CT; ++ct) s[t][ct] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int r = 0; r < 4; ++r) s[r] = kb + wave * 16 + 4 * c + r <= last ? s[r] * scale2 : -INFINITY;
-      *reinterpret_cast<f32x4*>(&sb[(ct * 16 + j) * SROW + wave * 16 + 4 * c]) = s;
-    }
+    for (int ks = 0; ks < KS; ++ks)
 #pragma unroll
-    for (int ks = 0; ks < KS; ++ks) *reinterpret_cast<bf16x8*>(&cb[(wave * 16 + j) * ROW + (ks * 4 + c) * 8]) = kf[ks];
-    if (kb + 64 <= last) load_tile(kb + 64);
-    // what this wave wrote is in LDS, and every wave is past its reads of this buffer (two steps ago); the loads on their way
-    // go on
-    asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
-    if (wave < UNITS) {
-      bf16x8 pf[UPW][2];
+      for (int t = 0; t < KT; ++t)
 #pragma unroll
-      for (int u = 0; u < UPW; ++u) {
-        const int ct = (wave + 4 * u) / NB;
-        float sv[2][8];
-        float mx = -INFINITY;
+        for (int ct = 0; ct < CT; ++ct) s[t][ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[t][ks], qf[ct][ks], s[t][ct], 0, 0, 0);
+    // every wave is through with the last step's latents and scores
+    if (kb > c0) asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
 #pragma unroll
-        for (int g = 0; g < 2; ++g) {
-          const float* sp = &sb[(ct * 16 + j) * SROW + 32 * g + 8 * c];
-          const f32x4 a = *reinterpret_cast<const f32x4*>(sp), b = *reinterpret_cast<const f32x4*>(sp + 4);
+    for (int t = 0; t < KT; ++t) {
+      const int k0 = (wave * KT + t) * 16;
 #pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            sv[g][e] = a[e];
-            sv[g][4 + e] = b[e];
-            mx = fmaxf(mx, fmaxf(a[e], b[e]));
-          }
-        }
-        mx = fmaxf(mx, __shfl_xor(mx, 16, kWave));
-        mx = fmaxf(mx, __shfl_xor(mx, 32, kWave));
-        const float m_new = fmaxf(m[u], mx);   // (a step holds at least one key: finite)
-        const float alpha = __builtin_amdgcn_exp2f(m[u] - m_new);
-        float sum = 0.f;
+      for (int ct = 0; ct < CT; ++ct) {
 #pragma unroll
-        for (int g = 0; g < 2; ++g)
-#pragma unroll
-          for (int e = 0; e < 8; ++e) {
-            const float w = __builtin_amdgcn_exp2f(sv[g][e] - m_new);
-            sum += w;
-            pf[u][g][e] = (bf16)w;
-          }
-        l[u] = l[u] * alpha + sum;
-        m[u] = m_new;
-        if (__any(alpha != 1.f)) {
-#pragma unroll
-          for (int i = 0; i < 8; ++i)
-#pragma unroll
-            for (int r = 0; r < 4; ++r) acc[u][i][r] *= alpha;
-        }
+        for (int r = 0; r < 4; ++r) s[t][ct][r] = kb + k0 + 4 * c + r <= last ? s[t][ct][r] * scale2 : -INFINITY;
+        *reinterpret_cast<f32x4*>(&sbuf[(ct * 16 + j) * SROW + k0 + 4 * c]) = s[t][ct];
       }
 #pragma unroll
-      for (int g = 0; g < 2; ++g) {
-        uint32_t in[8][4];   // key 32 g + 8 c + e, channels 8 piece .. + 7
+      for (int ks = 0; ks < KS; ++ks) *reinterpret_cast<bf16x8*>(&cbuf[(k0 + j) * ROW + (ks * 4 + c) * 8]) = kf[t][ks];
+    }
+    if (kb + KEYS <= last) load_tile(kb + KEYS);
+    // what this wave wrote is in LDS; its loads on their way go on
+    asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+    bf16x8 pf[UPW][RUNS];
 #pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          const uint4 v = *reinterpret_cast<const uint4*>(&cb[(32 * g + 8 * c + e) * ROW + (block * 16 + j) * 8]);
-          in[e][0] = v.x, in[e][1] = v.y, in[e][2] = v.z, in[e][3] = v.w;
+    for (int u = 0; u < UPW; ++u) {
+      const float* sc = &sbuf[((unit + 4 * u) / NB * 16 + j) * SROW + 8 * c];
+      float mx = -INFINITY;
+#pragma unroll
+      for (int g = 0; g < KEYS / 32; ++g) {
+        const f32x4 a = *reinterpret_cast<const f32x4*>(sc + 32 * g), b = *reinterpret_cast<const f32x4*>(sc + 32 * g + 4);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) mx = fmaxf(mx, fmaxf(a[e], b[e]));
+      }
+      mx = fmaxf(mx, __shfl_xor(mx, 16, kWave));
+      mx = fmaxf(mx, __shfl_xor(mx, 32, kWave));
+      const float m_new = fmaxf(m[u], mx);   // (a step holds at least one key: finite)
+      const float alpha = __builtin_amdgcn_exp2f(m[u] - m_new);
+      float sum = 0.f;
+#pragma unroll
+      for (int g = 0; g < RUNS; ++g) {
+        const float* sp = sc + 32 * (g * PARTS + part);
+        const f32x4 a = *reinterpret_cast<const f32x4*>(sp), b = *reinterpret_cast<const f32x4*>(sp + 4);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const float w0 = __builtin_amdgcn_exp2f(a[e] - m_new), w1 = __builtin_amdgcn_exp2f(b[e] - m_new);
+          sum += w0 + w1;
+          pf[u][g][e] = (bf16)w0;
+          pf[u][g][4 + e] = (bf16)w1;
         }
+      }
+      l[u] = l[u] * alpha + sum;
+      m[u] = m_new;
+      if (__any(alpha != 1.f)) {
 #pragma unroll
-        for (int i = 0; i < 8; ++i) {
-          union {
-            uint32_t w[4];
-            bf16x8 v;
-          } af;   // channel 8 piece + i, keys 8 c .. 8 c + 7
+        for (int i = 0; i < 8; ++i)
 #pragma unroll
-          for (int k = 0; k < 4; ++k)
-            af.w[k] = __builtin_amdgcn_perm(in[2 * k + 1][i / 2], in[2 * k][i / 2], (i & 1) ? 0x07060302u : 0x05040100u);
+          for (int r = 0; r < 4; ++r) acc[u][i][r] *= alpha;
+      }
+    }
 #pragma unroll
-          for (int u = 0; u < UPW; ++u) acc[u][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(af.v, pf[u][g], acc[u][i], 0, 0, 0);
-        }
+    for (int g = 0; g < RUNS; ++g) {
+      uint32_t in[8][4];   // key 8 c + e of the run, channels 8 piece .. + 7
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const uint4 v = *reinterpret_cast<const uint4*>(&cbuf[(32 * (g * PARTS + part) + 8 * c + e) * ROW + (block * 16 + j) * 8]);
+        in[e][0] = v.x, in[e][1] = v.y, in[e][2] = v.z, in[e][3] = v.w;
+      }
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        union {
+          uint32_t w[4];
+          bf16x8 v;
+        } af;   // channel 8 piece + i, keys 8 c .. 8 c + 7
+#pragma unroll
+        for (int k = 0; k < 4; ++k)
+          af.w[k] = __builtin_amdgcn_perm(in[2 * k + 1][i / 2], in[2 * k][i / 2], (i & 1) ? 0x07060302u : 0x05040100u);
+#pragma unroll
+        for (int u = 0; u < UPW; ++u) acc[u][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(af.v, pf[u][g], acc[u][i], 0, 0, 0);
       }
     }
   }
-  if (wave >= UNITS) return;
+  // the sums go out through LDS, so that a column's channels leave in whole lines; the waves of a unit add theirs up in order
+  float* obuf = reinterpret_cast<float*>(cbuf);
 #pragma unroll
-  for (int u = 0; u < UPW; ++u) {
-    const int ct = (wave + 4 * u) / NB, head = (hg * CT + ct) * 16 + j;
-    float total = l[u] + __shfl_xor(l[u], 16, kWave);
-    total += __shfl_xor(total, 32, kWave);
-    if (head >= H) continue;
-    const size_t cell = ((size_t)row * H + head) * splits + split;
-    if (block == 0 && c == 0) {
-      ws_ml[cell * 2] = m[u];
-      ws_ml[cell * 2 + 1] = total;
+  for (int turn = 0; turn < PARTS; ++turn) {
+    __syncthreads();
+    if (part != turn) continue;
+#pragma unroll
+    for (int u = 0; u < UPW; ++u) {
+      const int col = (unit + 4 * u) / NB * 16 + j;
+      float total = l[u] + __shfl_xor(l[u], 16, kWave);
+      total += __shfl_xor(total, 32, kWave);
+      if (block == 0 && c == 0) {
+        lbuf[col] = turn == 0 ? total : lbuf[col] + total;
+        const int head = hg * CT * 16 + col;
+        if (turn == 0 && head < H) ws_ml[(((size_t)row * H + head) * splits + split) * 2] = m[u];   // (the same in every part)
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        float* o = obuf + col * OROW + (block * 16 + 4 * c + r) * 8;
+        f32x4 a, b;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) a[e] = acc[u][e][r], b[e] = acc[u][4 + e][r];
+        if (turn > 0) {
+          a += *reinterpret_cast<const f32x4*>(o);
+          b += *reinterpret_cast<const f32x4*>(o + 4);
+        }
+        *reinterpret_cast<f32x4*>(o) = a;
+        *reinterpret_cast<f32x4*>(o + 4) = b;
+      }
     }
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int ch = (block * 16 + 4 * c + r) * 8;
-      if (ch >= R) continue;
-      f32x4 a, b;
-#pragma unroll
-      for (int e = 0; e < 4; ++e) a[e] = acc[u][e][r], b[e] = acc[u][4 + e][r];
-      *reinterpret_cast<f32x4*>(ws_acc + cell * R + ch) = a;
-      *reinterpret_cast<f32x4*>(ws_acc + cell * R + ch + 4) = b;
-    }
+  }
+  __syncthreads();
+  const int heads = min(CT * 16, H - hg * CT * 16), quads = R / 4;
+  for (int i = threadIdx.x; i < heads * quads; i += 256) {
+    const int col = i / quads, ch = (i % quads) * 4;
+    const size_t cell = ((size_t)row * H + hg * CT * 16 + col) * splits + split;
+    *reinterpret_cast<f32x4*>(ws_acc + cell * R + ch) = *reinterpret_cast<const f32x4*>(obuf + col * OROW + ch);
+    if (ch == 0) ws_ml[cell * 2 + 1] = lbuf[col];
   }
 }
 
@@ -365,19 +407,46 @@ __global__ __launch_bounds__(256) void latent_decode_plain_kernel(const T* __res
 }
 
 // ------------------------------------------------------------------------------------------------ latent_finish
-// A workgroup a (token, head): uv [H * hc, R] (the first vdim rows of a head), gate [n, ldg] (or nullptr: none).
-template <typename T>
+// A workgroup a (token, head): uv [H * hc, R] (the first vdim rows of a head), gate [n, ldg].  WORDS (bfloat16, R a multiple of
+// 8): sixteen lanes a channel of the value, 16 bytes of a row of W_uv a lane.  The first 64 rows' first 512 channels, and the
+// first partial sums of every thread's channels, are asked for before anything is known of the chunks: the kernel is short, and
+// round trips to memory are what it consists of.
+template <typename T, bool WORDS>
 __global__ __launch_bounds__(256) void latent_finish_kernel(const float* __restrict__ ws_acc, const float* __restrict__ ws_ml,
                                                             const int32_t* __restrict__ positions, int chunk, int splits,
                                                             const float* __restrict__ sinks, const T* __restrict__ uv, int hc,
                                                             const T* __restrict__ gate, int ldg, T* __restrict__ out, int ldo, int H,
-                                                            int R, int vdim, int words) {
+                                                            int R, int vdim) {
   __shared__ float weight[kMaxSplits];
   __shared__ __align__(16) float o[kMaxRank];
+  __shared__ __align__(16) float half_sums[1024];
   __shared__ float scratch[17];
   const int t = blockIdx.x / H, h = blockIdx.x % H, tid = threadIdx.x;
-  const int count = min(positions[t] / chunk + 1, splits);   // chunks that hold keys
+  const int g16 = tid / 16, l16 = tid % 16;
+  const T* w = uv + (size_t)h * hc * R;
+  bf16x8 early[4][4];
+  if constexpr (WORDS) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int k = 0; k < 4; ++k) {
+        const int d = g16 + 16 * i, p = l16 + 16 * k;
+        early[i][k] = (d < vdim && p * 8 < R) ? load8(w + (size_t)d * R + 8 * p) : zero8();
+      }
+  }
+  constexpr int EARLY = 8;
   const size_t cell0 = ((size_t)t * H + h) * splits;
+  // four channels a thread; where that leaves threads over, groups of them take the chunks in turn
+  const bool by_quads = R % 4 == 0 && R <= 1024;
+  const int quads = by_quads ? R / 4 : 256, groups = 256 / quads, group = tid / quads, q4 = (tid % quads) * 4;
+  f32x4 sums[EARLY];
+#pragma unroll
+  for (int i = 0; i < EARLY; ++i) {
+    const int k = group + i * groups;
+    sums[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (by_quads && group < groups && k < splits) sums[i] = *reinterpret_cast<const f32x4*>(ws_acc + (cell0 + k) * R + q4);
+  }
+  const int count = min(positions[t] / chunk + 1, splits);   // chunks that hold keys (the others' sums are not of this step)
   const float mine = tid < count ? ws_ml[(cell0 + tid) * 2] : -INFINITY, mine_l = tid < count ? ws_ml[(cell0 + tid) * 2 + 1] : 0.f;
   const float top = block_max(mine, scratch);
   const float f = tid < count ? exp2f(mine - top) : 0.f;
@@ -385,38 +454,70 @@ __global__ __launch_bounds__(256) void latent_finish_kernel(const float* __restr
   float total = block_sum(f * mine_l, scratch);   // (also orders the writes of weight before the reads below)
   if (sinks) total += exp2f(fmaf(sinks[h], kLog2e, -top));
   const float inv = 1.0f / total;
-  for (int r = tid; r < R; r += 256) {
-    float s = 0.f;
+  if (by_quads) {
+    f32x4 s = {0.f, 0.f, 0.f, 0.f};
+    if (group < groups) {
+#pragma unroll
+      for (int i = 0; i < EARLY; ++i) {
+        const int k = group + i * groups;
+        if (k < count) s += sums[i] * weight[k];
+      }
 #pragma unroll 8
-    for (int k = 0; k < count; ++k) s = fmaf(ws_acc[(cell0 + k) * R + r], weight[k], s);
-    o[r] = s * inv;
+      for (int k = group + EARLY * groups; k < count; k += groups) s += *reinterpret_cast<const f32x4*>(ws_acc + (cell0 + k) * R + q4) * weight[k];
+      *reinterpret_cast<f32x4*>(&half_sums[group * R + q4]) = s;
+    }
+    __syncthreads();
+    for (int r = tid; r < R; r += 256) {
+      float v = 0.f;
+      for (int k = 0; k < groups; ++k) v += half_sums[k * R + r];
+      o[r] = v * inv;
+    }
+  } else {
+    for (int r = tid; r < R; r += 256) {
+      float s = 0.f;
+      for (int k = 0; k < count; ++k) s = fmaf(ws_acc[(cell0 + k) * R + r], weight[k], s);
+      o[r] = s * inv;
+    }
   }
   __syncthreads();
-  const int g16 = tid / 16, l16 = tid % 16;   // sixteen lanes a channel of the value
-  for (int d = g16; d < vdim; d += 16) {
-    const T* w = uv + ((size_t)h * hc + d) * R;
-    float s = 0.f;
-    bool done = false;
-    if constexpr (std::is_same<T, bf16>::value) {
-      if (words) {
-        for (int p = l16; p < R / 8; p += 16) {
-          const bf16x8 v = load8(w + 8 * p);
-          const f32x4 a = *reinterpret_cast<const f32x4*>(&o[8 * p]), b = *reinterpret_cast<const f32x4*>(&o[8 * p + 4]);
-#pragma unroll
-          for (int e = 0; e < 4; ++e) s = fmaf((float)v[e], a[e], s);
-#pragma unroll
-          for (int e = 0; e < 4; ++e) s = fmaf((float)v[4 + e], b[e], s);
-        }
-        done = true;
-      }
-    }
-    if (!done)
-      for (int r = l16; r < R; r += 16) s = fmaf(to_f(w[r]), o[r], s);
+  auto finish = [&](int d, float s) {   // the sixteen lanes' sums of channel d
 #pragma unroll
     for (int off = 8; off >= 1; off >>= 1) s += __shfl_xor(s, off, 16);
-    if (l16 == 0) {
-      if (gate) s = s / (1.0f + expf(-to_f(gate[(size_t)t * ldg + (size_t)h * vdim + d])));
+    if (l16 == 0 && d < vdim) {
+      s = s / (1.0f + expf(-to_f(gate[(size_t)t * ldg + (size_t)h * vdim + d])));
       out[(size_t)t * ldo + (size_t)h * vdim + d] = from_f<T>(s);
+    }
+  };
+  auto dot8 = [&](const bf16x8& v, int p, float s) {
+    const f32x4 a = *reinterpret_cast<const f32x4*>(&o[8 * p]), b = *reinterpret_cast<const f32x4*>(&o[8 * p + 4]);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) s = fmaf((float)v[e], a[e], s);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) s = fmaf((float)v[4 + e], b[e], s);
+    return s;
+  };
+  if constexpr (WORDS) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int d = g16 + 16 * i;
+      float s = 0.f;
+#pragma unroll
+      for (int k = 0; k < 4; ++k)
+        if ((l16 + 16 * k) * 8 < R) s = dot8(early[i][k], l16 + 16 * k, s);
+      if (d < vdim)
+        for (int p = l16 + 64; p < R / 8; p += 16) s = dot8(load8(w + (size_t)d * R + 8 * p), p, s);
+      finish(d, s);
+    }
+    for (int d = g16 + 64; d < vdim; d += 16) {
+      float s = 0.f;
+      for (int p = l16; p < R / 8; p += 16) s = dot8(load8(w + (size_t)d * R + 8 * p), p, s);
+      finish(d, s);
+    }
+  } else {
+    for (int d = g16; d < vdim; d += 16) {
+      float s = 0.f;
+      for (int r = l16; r < R; r += 16) s = fmaf(to_f(w[(size_t)d * R + r]), o[r], s);
+      finish(d, s);
     }
   }
 }
@@ -572,20 +673,22 @@ extern "C" int gb_latent_decode(const void* q, int dtype, const void* pages, con
   const float scale2 = scale * kLog2e;
   if (!plain) {
     GB_REQUIRE(dtype == kBF16 && gb_latent_decode_takes(R, P), "latent_decode: R=%d in pages of %d goes through the plain kernel", R, P);
-    GB_REQUIRE(chunk % 64 == 0 && n <= 65535 && words16(q) && words16(pages) && words16(ws_acc), "latent_decode: chunks of whole 64 keys, aligned operands");
+    GB_REQUIRE(chunk % 128 == 0 && n <= 65535 && words16(q) && words16(pages) && words16(ws_acc), "latent_decode: chunks of whole 128 keys, aligned operands");
     const int ct = H > 16 ? 2 : 1;
     const dim3 grid((unsigned)splits, (unsigned)((H + 16 * ct - 1) / (16 * ct)), (unsigned)n);
-#define GB_LATENT(KS, CT)                                                                                                       \
-  if (ct == CT)                                                                                                                 \
-    hipLaunchKernelGGL((latent_decode_kernel<KS, CT>), grid, dim3(256), 0, stream, (const bf16*)q, (const bf16*)pages, tables, \
-                       table_stride, positions, H, R, P, scale2, chunk, splits, ws_acc, ws_ml);
+#define GB_LATENT_AS(KS, CT, FULL)                                                                                              \
+  if (ct == CT && (R == KS * 32) == FULL)                                                                                       \
+    hipLaunchKernelGGL((latent_decode_kernel<KS, CT, FULL>), grid, dim3(256), 0, stream, (const bf16*)q, (const bf16*)pages,     \
+                       tables, table_stride, positions, H, R, P, scale2, chunk, splits, ws_acc, ws_ml);
+#define GB_LATENT(KS) GB_LATENT_AS(KS, 1, true) GB_LATENT_AS(KS, 1, false) GB_LATENT_AS(KS, 2, true) GB_LATENT_AS(KS, 2, false)
     if (R <= 128) {
-      GB_LATENT(4, 1) GB_LATENT(4, 2)
+      GB_LATENT(4)
     } else if (R <= 256) {
-      GB_LATENT(8, 1) GB_LATENT(8, 2)
+      GB_LATENT(8)
     } else {
-      GB_LATENT(16, 1) GB_LATENT(16, 2)
+      GB_LATENT(16)
     }
+#undef GB_LATENT_AS
 #undef GB_LATENT
     return launched("latent_decode");
   }
@@ -608,15 +711,24 @@ extern "C" int gb_latent_decode(const void* q, int dtype, const void* pages, con
 extern "C" int gb_latent_finish(const float* ws_acc, const float* ws_ml, const int32_t* positions, int chunk, int splits,
                                 const float* sinks, const void* uv, int hc, const void* gate, int ldg, void* out, int ldo, int dtype,
                                 int n, int H, int R, int vdim, hipStream_t stream) {
-  GB_REQUIRE(n >= 0 && H > 0 && R > 0 && R <= kMaxRank && vdim > 0 && hc >= vdim && ldo >= H * vdim && (!gate || ldg >= H * vdim),
+  GB_REQUIRE(n >= 0 && H > 0 && R > 0 && R <= kMaxRank && vdim > 0 && hc >= vdim && ldo >= H * vdim && gate && ldg >= H * vdim,
              "latent_finish: bad sizes n=%d heads=%d R=%d vdim=%d", n, H, R, vdim);
   GB_REQUIRE(chunk > 0 && splits >= 1 && splits <= kMaxSplits && ws_acc && ws_ml && positions && uv && out, "latent_finish: %d chunks, or operands are missing", splits);
   if (n == 0) return 0;
   GB_REQUIRE((long long)n * H < (1ll << 31), "latent_finish: too many (token, head) pairs");
-  const int words = dtype == kBF16 && R % 8 == 0 && words16(uv);
-  GB_BY_DTYPE(dtype, "latent_finish",
-              hipLaunchKernelGGL(latent_finish_kernel<TT>, dim3((unsigned)(n * H)), dim3(256), 0, stream, ws_acc, ws_ml, positions, chunk,
-                                 splits, sinks, (const TT*)uv, hc, (const TT*)gate, ldg, (TT*)out, ldo, H, R, vdim, words))
+  GB_REQUIRE(R % 4 != 0 || words16(ws_acc), "latent_finish: the partial sums must be 16-byte aligned");
+#define GB_FINISH(T, WORDS)                                                                                                     \
+  hipLaunchKernelGGL((latent_finish_kernel<T, WORDS>), dim3((unsigned)(n * H)), dim3(256), 0, stream, ws_acc, ws_ml, positions, \
+                     chunk, splits, sinks, (const T*)uv, hc, (const T*)gate, ldg, (T*)out, ldo, H, R, vdim)
+  if (dtype == kBF16 && R % 8 == 0 && words16(uv))
+    GB_FINISH(bf16, true);
+  else if (dtype == kBF16)
+    GB_FINISH(bf16, false);
+  else if (dtype == kF32)
+    GB_FINISH(float, false);
+  else
+    return fail("latent_finish: unknown dtype %d", dtype);
+#undef GB_FINISH
   return launched("latent_finish");
 }
 

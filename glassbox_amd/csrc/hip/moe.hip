@@ -165,6 +165,54 @@ __global__ __launch_bounds__(4 * kWave) void route_kernel(const float* __restric
     }
 }
 
+// Logits and route in one kernel, for the router that chooses by z = W h + bias and weighs by the softmax over the chosen (up to
+// kWave experts): a workgroup a token, its waves take the experts in turn, a wave a dot product; then lane e of the first wave
+// holds expert e, and the number of experts that go before it (a larger logit, or the same and a lower number) is its place.
+template <typename T>
+__global__ __launch_bounds__(256) void router_kernel(const T* __restrict__ h, int ldh, const T* __restrict__ w, int ldw, int d, int words,
+                                                     int E, const float* __restrict__ bias, int top, float scale,
+                                                     float* __restrict__ combine, int32_t* __restrict__ ids, float* __restrict__ wts) {
+  __shared__ float z[kWave];
+  const int t = blockIdx.x, lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
+  const T* row = h + (size_t)t * ldh;
+  for (int e = wave; e < E; e += 4) {
+    const T* we = w + (size_t)e * ldw;
+    float s = 0.f;
+    bool done = false;
+    if constexpr (std::is_same<T, bf16>::value) {
+      if (words) {
+#pragma unroll 4
+        for (int c = lane * 8; c < d; c += kWave * 8) {
+          const bf16x8 a = *reinterpret_cast<const bf16x8*>(row + c), b = *reinterpret_cast<const bf16x8*>(we + c);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) s = fmaf((float)a[i], (float)b[i], s);
+        }
+        done = true;
+      }
+    }
+    if (!done)
+      for (int c = lane; c < d; c += kWave) s = fmaf(to_f(row[c]), to_f(we[c]), s);
+    s = wave_sum(s);
+    if (lane == 0) z[e] = s + (bias ? bias[e] : 0.f);
+  }
+  __syncthreads();
+  if (wave > 0) return;
+  const float mine = lane < E ? z[lane] : -INFINITY;
+  int ahead = 0;
+  for (int o = 0; o < E; ++o) {
+    const float v = z[o];
+    ahead += (v > mine || (v == mine && o < lane)) ? 1 : 0;
+  }
+  const bool chosen = lane < E && ahead < top;
+  const float s = expf(mine - wave_max(mine));
+  const float a = s * (scale / (wave_sum(chosen ? s : 0.f) + 1e-20f));
+  if (lane < E) combine[(size_t)t * E + lane] = chosen ? a : 0.f;
+  if (chosen) {
+    ids[(size_t)t * top + ahead] = lane;
+    wts[(size_t)t * top + ahead] = a;
+  }
+}
+
 // The unit: g' = min(g, limit), u' = clamp(u, -limit, limit), g' sigmoid(alpha g') (u' + plus); as it stands here silu(g) u.
 struct UnitOf {
   float limit = INFINITY, alpha = 1.0f, plus = 0.0f;
@@ -342,11 +390,13 @@ __global__ __launch_bounds__(256) void place_kernel(const int32_t* __restrict__ 
     }
 }
 
-// out[t] (+)= sum over k of wts[t, k] * y[pos[t, k]]  +  gates[t * ldg] * y_shared[t]; four columns a thread.
+// out[t] (+)= sum over k of wts[t, k] * y[pos[t, k]]  +  gates[t * ldg] * y_shared[t]; four columns a thread.  y is the sum of
+// `slices` pieces, slice_stride floats apart (what a product that divides k leaves), added in their order.
 __global__ __launch_bounds__(256) void combine_kernel(const float* __restrict__ y, int ldy, const int32_t* __restrict__ pos,
                                                       const float* __restrict__ wts, int top, const float* __restrict__ ysh,
                                                       int ldsh, const float* __restrict__ gates, int ldg, float* __restrict__ out,
-                                                      int ldo, int accumulate, int n, int quads, int y_rows) {
+                                                      int ldo, int accumulate, int n, int quads, int y_rows, int slices,
+                                                      long long slice_stride) {
   const long long idx = (long long)blockIdx.x * 256 + threadIdx.x;
   if (idx >= (long long)n * quads) return;
   const int t = (int)(idx / quads), c = (int)(idx % quads) * 4;
@@ -355,7 +405,14 @@ __global__ __launch_bounds__(256) void combine_kernel(const float* __restrict__ 
     const float w = wts[(size_t)t * top + k];
     // an entry whose expert is none (a row of logits that are no numbers) was never placed: any row will do for it
     const int r = min(max(pos[(size_t)t * top + k], 0), y_rows - 1);
-    const float4 v = *reinterpret_cast<const float4*>(y + (size_t)r * ldy + c);
+    float4 v = *reinterpret_cast<const float4*>(y + (size_t)r * ldy + c);
+    for (int z = 1; z < slices; ++z) {
+      const float4 o = *reinterpret_cast<const float4*>(y + (size_t)z * slice_stride + (size_t)r * ldy + c);
+      v.x += o.x;
+      v.y += o.y;
+      v.z += o.z;
+      v.w += o.w;
+    }
     acc.x += w * v.x;
     acc.y += w * v.y;
     acc.z += w * v.z;
@@ -400,6 +457,24 @@ extern "C" int gb_moe_route_by(const float* z, int ldz, int n, int E, const floa
 extern "C" int gb_moe_route(const float* z, int ldz, int n, int E, const float* correction, int top, float scale, int shared,
                             float* combine, int32_t* ids, float* wts, hipStream_t stream) {
   return gb_moe_route_by(z, ldz, n, E, correction, top, scale, shared ? 1 : 0, 0, 1, 0, 0, combine, ids, wts, stream);
+}
+
+// h [n, ldh] and w [E, ldw] of `dtype`, d columns each; bias float32 [E] or nullptr; combine [n, E], ids and wts [n, top].
+extern "C" int gb_moe_router(const void* h, int dtype, int ldh, const void* w, int ldw, int n, int d, int E, const float* bias, int top,
+                             float scale, float* combine, int32_t* ids, float* wts, hipStream_t stream) {
+  GB_REQUIRE(n >= 0 && d > 0 && ldh >= d && ldw >= d && h && w && combine && ids && wts, "moe_router: bad sizes n=%d d=%d", n, d);
+  GB_REQUIRE(E > 0 && E <= kWave && top > 0 && top <= E, "moe_router: %d chosen experts of %d (at most %d)", top, E, kWave);
+  if (n == 0) return 0;
+  const int words = dtype == kBF16 && d % 8 == 0 && ldh % 8 == 0 && ldw % 8 == 0 && (uintptr_t)h % 16 == 0 && (uintptr_t)w % 16 == 0;
+  if (dtype == kF32)
+    hipLaunchKernelGGL(router_kernel<float>, dim3((unsigned)n), dim3(256), 0, stream, (const float*)h, ldh, (const float*)w, ldw, d, words, E,
+                       bias, top, scale, combine, ids, wts);
+  else if (dtype == kBF16)
+    hipLaunchKernelGGL(router_kernel<bf16>, dim3((unsigned)n), dim3(256), 0, stream, (const bf16*)h, ldh, (const bf16*)w, ldw, d, words, E,
+                       bias, top, scale, combine, ids, wts);
+  else
+    return fail("moe_router: unknown dtype %d", dtype);
+  return launched("moe_router");
 }
 
 extern "C" int gb_moe_relu2_units(const void* z, int in_dtype, int ld, const float* combine, int cols, void* act, int out_dtype,
@@ -472,7 +547,9 @@ extern "C" int gb_moe_sort(const int32_t* ids, int n, int top, int E, int tile_r
 }
 
 extern "C" int gb_moe_combine(const float* y, int ldy, const int32_t* pos, const float* wts, int top, const float* ysh, int ldsh,
-                              const float* gates, int ldg, float* out, int ldo, int accumulate, int n, int d, int y_rows, hipStream_t stream) {
+                              const float* gates, int ldg, float* out, int ldo, int accumulate, int n, int d, int y_rows, int slices,
+                              long long slice_stride, hipStream_t stream) {
+  GB_REQUIRE(slices >= 1 && slice_stride % 4 == 0 && (slices == 1 || slice_stride >= (long long)y_rows * ldy), "moe_combine: %d slices of y", slices);
   GB_REQUIRE(y_rows >= (long long)n * top, "moe_combine: y holds %d rows for %d tokens of %d choices", y_rows, n, top);
   GB_REQUIRE(n >= 0 && d > 0 && d % 4 == 0 && ldy % 4 == 0 && ldo % 4 == 0 && (!ysh || (ldsh % 4 == 0 && gates)) && ldy >= d && ldo >= d,
              "moe_combine: rows of %d columns (strides %d, %d, %d) must be whole groups of four", d, ldy, ldsh, ldo);
@@ -481,12 +558,13 @@ extern "C" int gb_moe_combine(const float* y, int ldy, const int32_t* pos, const
   const long long count = (long long)n * (d / 4);
   GB_REQUIRE((count + 255) / 256 < (1ll << 31), "moe_combine: too many elements");
   hipLaunchKernelGGL(combine_kernel, dim3((unsigned)((count + 255) / 256)), dim3(256), 0, stream, y, ldy, pos, wts, top, ysh, ldsh,
-                     gates, ldg, out, ldo, accumulate, n, d / 4, y_rows);
+                     gates, ldg, out, ldo, accumulate, n, d / 4, y_rows, slices, slice_stride);
   return launched("moe_combine");
 }
 
 GB_TAPED(gb_moe_sort)
 GB_TAPED(gb_moe_combine)
+GB_TAPED(gb_moe_router)
 GB_TAPED(gb_moe_route)
 GB_TAPED(gb_moe_route_by)
 GB_TAPED(gb_moe_relu2_units)

@@ -144,8 +144,11 @@ _SIGS = {
         "gb_moe_gated_units": [_vp, _i, _i, _vp, _i, _vp, _i, _i, _i, _i, _i, _f, _f, _f, _vp],
         # ids, n, top, experts, rows a tile, tiles, counts, rows, pos, map, stream
         "gb_moe_sort": [_vp, _i, _i, _i, _i, _i, _vp, _vp, _vp, _vp, _vp],
-        # y, ldy, pos, weights, top, y_shared, its stride, gates, their stride, out, ldo, accumulate, n, d, rows of y, stream
-        "gb_moe_combine": [_vp, _i, _vp, _vp, _i, _vp, _i, _vp, _i, _vp, _i, _i, _i, _i, _i, _vp],
+        # y, ldy, pos, weights, top, y_shared, its stride, gates, their stride, out, ldo, accumulate, n, d, rows of y, slices
+        # of y, their distance, stream
+        "gb_moe_combine": [_vp, _i, _vp, _vp, _i, _vp, _i, _vp, _i, _vp, _i, _i, _i, _i, _i, _i, C.c_longlong, _vp],
+        # h, dtype, ldh, w, ldw, n, d, experts, bias, top, scale, combine, ids, weights, stream
+        "gb_moe_router": [_vp, _i, _i, _vp, _i, _i, _i, _i, _vp, _i, _f, _vp, _vp, _vp, _vp],
     },
     "streams": {
         # X, stream stride, streams, w_in, gamma, gamma dtype, rows, out, out dtype, sum, m, d, eps, mix, w_out, y, stream
@@ -181,8 +184,8 @@ _SIGS = {
         "gb_gemm_bf16": [_vp, _i, _vp, _i, _vp, _i, _i, _i, _i, _i, _i, _vp, _i, _f, _vp, _i, _vp, _i, _vp, _vp, _i, _vp,
                          C.c_longlong, _vp],
         # a, lda, rows, w, ldw, distance between groups, up_off, c, ldc, c_dtype, map, tiles, rows a tile, N, K, epilogue,
-        # limit, alpha, plus, stream
-        "gb_gemm_bf16_grouped": [_vp, _i, _vp, _vp, _i, C.c_longlong, _i, _vp, _i, _i, _vp, _i, _i, _i, _i, _i, _f, _f, _f, _vp],
+        # limit, alpha, plus, slices of k, rows of c a slice, stream
+        "gb_gemm_bf16_grouped": [_vp, _i, _vp, _vp, _i, C.c_longlong, _i, _vp, _i, _i, _vp, _i, _i, _i, _i, _i, _f, _f, _f, _i, _i, _vp],
         # a, lda, w, ldw, c, ldc, M, N, K, limit, alpha, plus, stream
         "gb_gemm_bf16_glu": [_vp, _i, _vp, _i, _vp, _i, _i, _i, _i, _f, _f, _f, _vp],
         "gb_gemm_bf16_split_floats": [_i, _i, _i],
@@ -1263,10 +1266,14 @@ def moe_sort(ids: torch.Tensor, n_experts: int, tile_rows: int, counts: torch.Te
 def moe_combine(y: torch.Tensor, pos: torch.Tensor, weights: torch.Tensor, y_shared: Optional[torch.Tensor],
                 gates: Optional[torch.Tensor], out: torch.Tensor, accumulate: bool) -> None:
     """out[t] (+)= sum over k of weights[t, k] * y[pos[t, k]] + gates[t] * y_shared[t], all float32; ``gates`` may be a
-    column of a wider tensor."""
+    column of a wider tensor; a ``y`` of [slices, rows, d] is the sum of its slices."""
     _dev(y, pos, weights, y_shared, gates, out)
     n, top = weights.shape
     d = out.shape[1]
+    slices, slice_stride = 1, 0
+    if y.dim() == 3:
+        slices, slice_stride = y.shape[0], y.stride(0)
+        y = y[0]
     for t, what in ((y, "y"), (out, "out"), (y_shared, "y_shared")):
         if t is not None and (t.dtype != torch.float32 or t.dim() != 2 or t.stride(1) != 1 or t.shape[1] != d):
             raise KernelError(f"moe_combine: {what} must be float32 [rows, {d}] with dense rows")
@@ -1277,7 +1284,38 @@ def moe_combine(y: torch.Tensor, pos: torch.Tensor, weights: torch.Tensor, y_sha
     lib = _lib("moe")
     _launch(lib, lib.gb_moe_combine, _p(y), y.stride(0), _p(pos), _p(weights), top, _p(y_shared),
             y_shared.stride(0) if y_shared is not None else 0, _p(gates), gates.stride(0) if gates is not None else 0,
-            _p(out), out.stride(0), 1 if accumulate else 0, n, d, y.shape[0], _stream())
+            _p(out), out.stride(0), 1 if accumulate else 0, n, d, y.shape[0], slices, slice_stride, _stream())
+
+
+MOE_ROUTER_MAX_EXPERTS = 64   # moe.hip: a lane an expert
+
+
+def moe_router(h: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], top: int, scale: float, combine: torch.Tensor,
+               ids: torch.Tensor, weights: torch.Tensor) -> None:
+    """Logits z = h . w^T + bias and the route by them in one kernel (``moe_route`` with ``softmax="chosen"``): ``h`` [n, d] and
+    ``w`` [experts, d] of one type, up to ``MOE_ROUTER_MAX_EXPERTS`` experts."""
+    _dev(h, w, bias, combine, ids, weights)
+    n, d = h.shape
+    E = w.shape[0]
+    if w.dtype != h.dtype or w.shape[1] != d or E > MOE_ROUTER_MAX_EXPERTS:
+        raise KernelError(f"moe_router: w must be [at most {MOE_ROUTER_MAX_EXPERTS}, d] of h's type")
+    _f32_rows(combine, (n, E), "combine")
+    _f32_rows(weights, (n, top), "weights")
+    _i32(ids, "ids", n * top)
+    if bias is not None:
+        _f32_rows(bias, (E,), "bias")
+    lib = _lib("moe")
+    _launch(lib, lib.gb_moe_router, _p(h), dtype_code(h), _rows(h, "h"), _p(w), _rows(w, "w"), n, d, E, _p(bias), int(top), float(scale),
+            _p(combine), _p(ids), _p(weights), _stream())
+
+
+@functools.lru_cache(maxsize=4096)
+def grouped_ring_slices(entries: int, groups: int, n_out: int, k: int) -> int:
+    """Slices of k for a grouped product with tiles of 256 rows and columns: as many (up to four) as leave the compute units
+    busy to the end, if the tiles' number is what one expects of so many entries."""
+    tiles = (entries // 256 + groups // 2) * -(-n_out // 256)
+    cost = lambda s: -(-tiles * s // 256) / s
+    return min((s for s in (1, 2, 3, 4) if k // s >= 512 or s == 1), key=cost)
 
 
 def gemm_grouped_takes(a: torch.Tensor, w: torch.Tensor, group_stride: int) -> bool:
@@ -1293,12 +1331,17 @@ def gemm_grouped(a: torch.Tensor, rows: Optional[torch.Tensor], w: torch.Tensor,
     ``a`` (row r without ``rows``); ``tile_map`` (as ``moe_sort`` writes it) names each row tile's group and rows; group g
     uses the ``n_out`` rows of ``w`` that begin ``g * group_stride`` elements into it.  ``silu_mul``: the group's rows
     are n_out / 2 gate rows, with the up row of each ``up_offset`` rows behind it, and out = silu(gate) * up, or another
-    ``unit = (limit, alpha, plus)`` as ``moe_gated_units`` takes it."""
+    ``unit = (limit, alpha, plus)`` as ``moe_gated_units`` takes it.  Row tiles are of 64, 128 or 256 rows; with 256 (the inner
+    size a multiple of 32) a float32 ``out`` may be [slices, rows, n_out]: k is divided, and out's sum over the slices is the
+    result."""
     _dev(a, rows, w, tile_map, out)
     K = a.shape[1]
     cols = n_out // 2 if silu_mul else n_out
     if not gemm_grouped_takes(a, w, group_stride) or a.stride(1) != 1 or w.stride(1) != 1 or w.shape[1] < K:
         raise KernelError("gemm_grouped: operands must be bfloat16 with dense, 16-byte aligned rows")
+    slices = 1
+    if out.dim() == 3 and out.is_contiguous():
+        slices, out = out.shape[0], out[0]
     if out.dim() != 2 or out.stride(1) != 1 or out.shape[1] != cols or (silu_mul and out.dtype != torch.bfloat16):
         raise KernelError(f"gemm_grouped: out must be [rows, {cols}] with dense rows (bfloat16 behind silu(gate) * up)")
     tiles = tile_map.shape[0]
@@ -1308,7 +1351,7 @@ def gemm_grouped(a: torch.Tensor, rows: Optional[torch.Tensor], w: torch.Tensor,
     lib = _lib("gemm_bf16")
     _launch(lib, lib.gb_gemm_bf16_grouped, _p(a), a.stride(0), _p(rows), _p(w), w.stride(0), int(group_stride), int(up_offset),
             _p(out), out.stride(0), dtype_code(out), _p(tile_map), tiles, tile_rows, n_out, K, 2 if silu_mul else 0,
-            *map(float, unit), _stream())
+            *map(float, unit), slices, out.shape[0], _stream())
 
 
 # ------------------------------------------------------------------- small residual operations
@@ -2102,7 +2145,7 @@ def latent_chunk(rows: int, n_heads: int, max_context: int, tuned: bool) -> int:
     all of one), at least 128 keys each, since every chunk leaves a row of sums a head for the last pass."""
     if tuned:
         groups = rows * -(-n_heads // (32 if n_heads > 16 else 16))
-        want, step, least = max(1, 256 // groups), 64, 128
+        want, step, least = max(1, 256 // groups), 128, 128
     else:
         want, step, least = max(1, 1024 // (rows * n_heads)), 256, 256
     chunk = -(-max_context // min(want, 256))
@@ -2111,7 +2154,7 @@ def latent_chunk(rows: int, n_heads: int, max_context: int, tuned: bool) -> int:
 
 def latent_decode(q: torch.Tensor, pages: torch.Tensor, tables: torch.Tensor, positions: torch.Tensor, tok_seq: torch.Tensor,
                   n_heads: int, scale: float, max_context: int, sinks: Optional[torch.Tensor], uv: torch.Tensor, head_cols: int,
-                  vdim: int, gate: Optional[torch.Tensor], out: torch.Tensor, buffer, plain: bool = False) -> None:
+                  vdim: int, gate: torch.Tensor, out: torch.Tensor, buffer, plain: bool = False) -> None:
     """Attention of rows with absorbed queries ``q`` ([n, heads * R]) over their requests' cached latents: out [n, heads * vdim] =
     sigmoid(gate) * W_uv (softmax(scale * q . c, with a sink a head) c).  ``uv`` [>= heads * head_cols, R], the first ``vdim`` rows
     of a head.  The matrix-core kernel takes row t for request t's single token; ``plain``: any rows, by ``tok_seq``.
@@ -2135,7 +2178,7 @@ def latent_decode(q: torch.Tensor, pages: torch.Tensor, tables: torch.Tensor, po
     _launch(lib, lib.gb_latent_decode, _p(q), dtype_code(q), _p(pages), _p(tables), tables.stride(0), _p(positions), _p(tok_seq), n,
             n_heads, R, P, float(scale), chunk, splits, _p(acc), _p(ml), 1 if plain else 0, _stream())
     _launch(lib, lib.gb_latent_finish, _p(acc), _p(ml), _p(positions), chunk, splits, _p(_sinks(sinks, n_heads)), _p(uv), head_cols,
-            _p(gate), _act_rows(gate, q.dtype, n_heads * vdim, "gate") if gate is not None else 0, _p(out),
+            _p(gate), _act_rows(gate, q.dtype, n_heads * vdim, "gate"), _p(out),
             _act_rows(out, q.dtype, n_heads * vdim, "out"), dtype_code(out), n, n_heads, R, vdim, _stream())
 
 

@@ -115,15 +115,13 @@ class RoutedExperts(FeedForward):
         them in slices, and returns what ``product_in_slices`` does."""
         n, E = h.shape[0], self.n_experts
         cols = E + (1 if self.shared_ff else 0)
-        z = ctx.buffer("moe_z", (n, self.w_router.shape[0]), torch.float32)
-        product(ctx, h, self.w_router, z)
         combine = ctx.buffer("moe_combine", (n, cols), torch.float32)
         ids = ctx.buffer("moe_ids", (n, self.top), torch.int32)
         weights = ctx.buffer("moe_weights", (n, self.top), torch.float32)
-        shared = False if not self.shared_ff else True if self.shared_gate else "whole"
-        count, keep = self.groups if self.groups is not None else (0, 0)
-        ops.moe_route(z, E, self.correction, self.top, self.router_scale, shared, combine, ids, weights,
-                      softmax="chosen" if self.scoring == "chosen" else self.scoring == "softmax", renorm=self.renorm, groups=count, keep_groups=keep)
+        if self.scoring == "chosen" and not self.shared_ff and E <= ops.MOE_ROUTER_MAX_EXPERTS and ctx.tuned:
+            ops.moe_router(h, self.w_router, self.correction, self.top, self.router_scale, combine, ids, weights)
+        else:
+            self._route(ctx, h, combine, ids, weights)
         if self.routed(ctx, n):
             return self._routed(ctx, h, residual, store, combine, ids, weights)
         gate_up = ctx.buffer("moe_gate_up", (n, self.halves * self.inter), torch.float32)
@@ -137,6 +135,15 @@ class RoutedExperts(FeedForward):
             return product_in_slices(ctx, act, self.w_down, residual)
         product(ctx, act, self.w_down, residual, accumulate=True)
         return None
+
+    def _route(self, ctx, h, combine, ids, weights) -> None:
+        n, E = h.shape[0], self.n_experts
+        z = ctx.buffer("moe_z", (n, self.w_router.shape[0]), torch.float32)
+        product(ctx, h, self.w_router, z)
+        shared = False if not self.shared_ff else True if self.shared_gate else "whole"
+        count, keep = self.groups if self.groups is not None else (0, 0)
+        ops.moe_route(z, E, self.correction, self.top, self.router_scale, shared, combine, ids, weights,
+                      softmax="chosen" if self.scoring == "chosen" else self.scoring == "softmax", renorm=self.renorm, groups=count, keep_groups=keep)
 
     def adds_in_place(self, ctx, n: int) -> bool:
         return self.routed(ctx, n)   # (the pass that adds up the chosen experts' rows)
@@ -153,6 +160,10 @@ class RoutedExperts(FeedForward):
         n, E, ff, d, top = h.shape[0], self.n_experts, self.expert_ff, self.width, self.top
         entries = n * top
         tile_rows = 128 if entries >= 256 * E else 64
+        # many rows an expert: the ring kernel's tiles of 256 rows, where these fill the chip
+        if (entries >= 512 * E and d % 32 == 0 and ff % 32 == 0 and min(d, ff) >= 128
+                and (entries // 256) * -(-ff * self.halves // 256) >= 192):
+            tile_rows = 256
         tiles = ops.moe_sort_tiles(entries, E, tile_rows)
         counts = ctx.buffer("moe_counts", (E,), torch.int32)
         rows = ctx.buffer("moe_rows", (entries,), torch.int32)
@@ -166,7 +177,8 @@ class RoutedExperts(FeedForward):
         else:   # the unit in a pass of its own over the experts' rows, in place
             ops.gemm_grouped(h, rows, self.w_gate_up, ff * self.w_gate_up.stride(0), ff, tile_map, tile_rows, act)
             ops.moe_relu2_units(act, None, act, 0, ff)
-        y = ctx.buffer("moe_y", (entries, d), torch.float32)
+        slices = ops.grouped_ring_slices(entries, E, d, ff) if tile_rows == 256 else 1
+        y = ctx.buffer("moe_y", (slices, entries, d) if slices > 1 else (entries, d), torch.float32)
         ops.gemm_grouped(act, None, self.w_down, ff, d, tile_map, tile_rows, y)
         y_shared = gates = None
         if self.shared_ff:

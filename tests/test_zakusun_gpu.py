@@ -394,6 +394,73 @@ def test_the_router_chooses_by_logits_with_bias(E, top):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("E, top, d", [(6, 2, 64), (64, 16, 40), (3, 3, 50), (12, 4, 2048), (1, 1, 8)])
+def test_logits_and_route_in_one_kernel(E, top, d, dtype):
+    """The same choice and weights as the product and the route kernel give, for rows of one to hundreds of tokens."""
+    from glassbox_amd import ops
+    torch.manual_seed(E + d)
+    for n in (1, 9, 300):
+        h, w, bias = torch.randn(n, d).to(dtype), (torch.randn(E, d) * 3 / d ** 0.5).to(dtype), torch.randn(E)
+        z = h.to(F64) @ w.to(F64).T + bias.to(F64)
+        ids_w, wts_w = pz.route(z, top)
+        combine = torch.full((n, E), 9.0, device=DEV)
+        ids, wts = torch.empty(n, top, dtype=torch.int32, device=DEV), torch.empty(n, top, device=DEV)
+        ops.moe_router(h.to(DEV), w.to(DEV), _dev(bias), top, 0.5, combine, ids, wts)
+        clear = pz.route_margin(z, top) > 1e-4
+        assert clear.sum() > 0.9 * n
+        dense = torch.zeros(n, E, dtype=F64).scatter_(1, ids_w, 0.5 * wts_w)
+        assert (combine.cpu().to(F64) - dense)[clear].abs().max() < 5e-5
+        given = torch.zeros(n, E, dtype=F64).scatter_(1, ids.cpu().long(), wts.cpu().to(F64))
+        assert torch.equal(given, combine.cpu().to(F64))
+        ordered = wts.cpu()
+        assert torch.all(ordered[:, :-1] >= ordered[:, 1:])      # the largest logit's expert first
+
+
+def test_grouped_products_by_tiles_of_256_rows_with_k_divided():
+    """Rows of groups of very unequal size (none, one, a tile and a row more, several tiles) through the ring kernel: stored,
+    behind the clamped unit, and with k divided into slices that are added, against the product by tiles of 128 rows."""
+    from glassbox_amd import ops
+    torch.manual_seed(6)
+    d, ff, E = 256, 320, 5
+    sizes = [0, 1, 257, 900, 300]
+    n = sum(sizes)
+    ids = torch.cat([torch.full((s,), e) for e, s in enumerate(sizes)])[torch.randperm(n)].int().view(n, 1)
+    h = torch.randn(n, d).bfloat16().to(DEV)
+    up = (torch.randn(2 * E * ff, d) * 0.1).bfloat16().to(DEV)
+    down = (torch.randn(d, E * ff) * 0.1).bfloat16().to(DEV)
+    got = {}
+    for rows in (128, 256):
+        tiles = ops.moe_sort_tiles(n, E, rows)
+        counts, order = torch.empty(E, dtype=torch.int32, device=DEV), torch.empty(n, dtype=torch.int32, device=DEV)
+        pos, tile_map = torch.empty(n, 1, dtype=torch.int32, device=DEV), torch.empty(tiles, 3, dtype=torch.int32, device=DEV)
+        ops.moe_sort(ids.to(DEV), E, rows, counts, order, pos, tile_map)
+        act = torch.full((n, ff), 7.0, dtype=torch.bfloat16, device=DEV)
+        ops.gemm_grouped(h, order, up, ff * d, 2 * ff, tile_map, rows, act, silu_mul=True, up_offset=E * ff, unit=(1.0, 1.702, 1.0))
+        plain = torch.full((n, ff), 7.0, dtype=torch.bfloat16, device=DEV)
+        ops.gemm_grouped(h, order, up, ff * d, ff, tile_map, rows, plain)
+        y = torch.full((n, d), 7.0, device=DEV)
+        ops.gemm_grouped(act, None, down, ff, d, tile_map, rows, y)
+        got[rows] = (act.float(), plain.float(), y)
+        if rows == 256:
+            for slices in (2, 3):
+                parts = torch.full((slices, n, d), 7.0, device=DEV)
+                ops.gemm_grouped(act, None, down, ff, d, tile_map, rows, parts)
+                assert (parts.sum(0) - y).abs().max() < 1e-4 * float(y.abs().max())
+                one, two = torch.zeros(n, d, device=DEV), torch.zeros(n, d, device=DEV)
+                wts = torch.rand(n, 1, device=DEV)
+                ops.moe_combine(y, pos, wts, None, None, one, False)
+                ops.moe_combine(parts, pos, wts, None, None, two, False)
+                assert (one - two).abs().max() < 1e-4 * float(one.abs().max())
+    for a, b in zip(got[128], got[256]):
+        assert (a - b).abs().max() <= 1e-2 * float(b.abs().max())
+    # one group's rows against the product written out
+    order = torch.argsort(ids[:, 0].to(DEV), stable=True)
+    rows = order[sizes[1] + sizes[2]:sizes[1] + sizes[2] + sizes[3]]
+    want = h[rows].float() @ up[3 * ff:4 * ff].float().t()
+    assert (got[256][1][258:258 + 900] - want).abs().max() < 1e-2 * float(want.abs().max())
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("ff, limit", [(12, 0.7), (30, 2.0), (7, 1.5)])
 def test_clamped_units_with_weights(ff, limit, dtype):
     from glassbox_amd import ops
@@ -412,7 +479,7 @@ def test_clamped_units_with_weights(ff, limit, dtype):
 
 
 @pytest.mark.parametrize("d, E, top, ff, sizes", [(64, 8, 2, 16, (5, 300)), (128, 4, 2, 64, (3, 2100)), (96, 12, 3, 40, (17, 65, 700)),
-                                                  (256, 2, 1, 128, (1100,))])
+                                                  (256, 2, 1, 128, (1100,)), (128, 4, 2, 4096, (2048,))])
 def test_experts_on_their_own_tokens_against_every_expert_on_every_token(d, E, top, ff, sizes):
     """The two ways through a step of the routed feed-forward (few rows: every expert on every token, zeros for the ones
     not chosen; many rows: sorted by expert) against the plain sum, with one expert's down matrix a hundred times the
