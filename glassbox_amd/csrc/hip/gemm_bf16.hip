@@ -446,6 +446,12 @@ __global__ __launch_bounds__(RGM * RGN * 64, 1) void gemm_ring_kernel(const bf16
   int bx = blockIdx.x, by = blockIdx.y;
   if (k_slice > 0) {  // split k: workgroup z of a tile sums its own slice of k into its own copy of C
     int z = blockIdx.z;
+    if (GROUPED) {  // the tiles in the map's order, all slices of a tile before the next one's
+      const int gx = gridDim.x, gz = gridDim.z, id = bx + gx * (by + (int)gridDim.y * z);
+      bx = id % gx;
+      z = id / gx % gz;
+      by = id / gx / gz;
+    }
     // The chip deals workgroups round its 8 dies by their number, and each die has a second-level cache of its
     // own.  With the grid as it stands a die would hold one column tile over all row tiles and all slices (8 + 32
     // different operand pieces a k-step among its 32 workgroups); numbered anew, it holds an eighth of the grid in
@@ -527,6 +533,9 @@ __global__ __launch_bounds__(RGM * RGN * 64, 1) void gemm_ring_kernel(const bf16
   const uint32_t wbase = (uint32_t)(uintptr_t)(lds_void*)&Ws[0][0] + 2 * wn * RTN * 32 * RBK;
   constexpr uint32_t A_STAGE = 2 * RBM * RBK, W_STAGE = 2 * RBN * RBK, TILE = 2 * 32 * RBK;
 
+  // GROUPED: a group's last tile may hold few rows: a wave leaves out the MFMAs of rows of 32 that lie beyond the group's end
+  const int live = GROUPED ? min(max((M - m0 - wm * RTM * 32 + 31) / 32, 0), RTM) : RTM;
+
   const int steps = K / RBK;
   bf16x8 fa[2][RTM], fw[2][RTN];
   auto read_operands = [&](int stage, int ks) {
@@ -540,9 +549,11 @@ __global__ __launch_bounds__(RGM * RGN * 64, 1) void gemm_ring_kernel(const bf16
   auto multiply = [&](int ks, auto more, int nstage, int nk0) {
 #pragma unroll
     for (int i = 0; i < RTM; ++i) {
+      if (!GROUPED || i < live) {
 #pragma unroll
-      for (int j = 0; j < RTN; ++j)
-        acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(fa[ks][i], fw[ks][j], acc[i][j], 0, 0, 0);
+        for (int j = 0; j < RTN; ++j)
+          acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(fa[ks][i], fw[ks][j], acc[i][j], 0, 0, 0);
+      }
       if (decltype(more)::value) {
         constexpr int SLOTS = 2 * RTM;
         const int slot = ks * RTM + i;

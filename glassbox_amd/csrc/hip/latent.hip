@@ -332,13 +332,16 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(const bf16* __res
     }
   }
   __syncthreads();
-  const int heads = min(CT * 16, H - hg * CT * 16), quads = R / 4;
-  for (int i = threadIdx.x; i < heads * quads; i += 256) {
-    const int col = i / quads, ch = (i % quads) * 4;
-    const size_t cell = ((size_t)row * H + hg * CT * 16 + col) * splits + split;
-    *reinterpret_cast<f32x4*>(ws_acc + cell * R + ch) = *reinterpret_cast<const f32x4*>(obuf + col * OROW + ch);
-    if (ch == 0) ws_ml[cell * 2 + 1] = lbuf[col];
+  const int heads = min(CT * 16, H - hg * CT * 16);
+  float* cells = ws_acc + (((size_t)row * H + hg * CT * 16) * splits + split) * R;   // a head's are splits * R apart
+  for (int col = wave; col < heads; col += 4) {
+#pragma unroll
+    for (int i = 0; i < (KS * 8 + 63) / 64; ++i) {
+      const int ch = (lane + 64 * i) * 4;
+      if (ch < R) *reinterpret_cast<f32x4*>(cells + (size_t)col * splits * R + ch) = *reinterpret_cast<const f32x4*>(obuf + col * OROW + ch);
+    }
   }
+  if ((int)threadIdx.x < heads) ws_ml[(((size_t)row * H + hg * CT * 16 + threadIdx.x) * splits + split) * 2 + 1] = lbuf[threadIdx.x];
 }
 
 // Any sizes and types: 256 threads, a thread a key for the scores and a thread a channel (and every 256th after it) for the sums.
@@ -408,9 +411,8 @@ __global__ __launch_bounds__(256) void latent_decode_plain_kernel(const T* __res
 
 // ------------------------------------------------------------------------------------------------ latent_finish
 // A workgroup a (token, head): uv [H * hc, R] (the first vdim rows of a head), gate [n, ldg].  WORDS (bfloat16, R a multiple of
-// 8): sixteen lanes a channel of the value, 16 bytes of a row of W_uv a lane.  The first 64 rows' first 512 channels, and the
-// first partial sums of every thread's channels, are asked for before anything is known of the chunks: the kernel is short, and
-// round trips to memory are what it consists of.
+// 8): sixteen lanes a channel of the value, 16 bytes of a row of W_uv a lane; the first 64 rows' first 512 channels are asked for
+// before anything else.
 template <typename T, bool WORDS>
 __global__ __launch_bounds__(256) void latent_finish_kernel(const float* __restrict__ ws_acc, const float* __restrict__ ws_ml,
                                                             const int32_t* __restrict__ positions, int chunk, int splits,
@@ -420,7 +422,6 @@ __global__ __launch_bounds__(256) void latent_finish_kernel(const float* __restr
   __shared__ float weight[kMaxSplits];
   __shared__ __align__(16) float o[kMaxRank];
   __shared__ __align__(16) float half_sums[1024];
-  __shared__ float scratch[17];
   const int t = blockIdx.x / H, h = blockIdx.x % H, tid = threadIdx.x;
   const int g16 = tid / 16, l16 = tid % 16;
   const T* w = uv + (size_t)h * hc * R;
@@ -434,36 +435,37 @@ __global__ __launch_bounds__(256) void latent_finish_kernel(const float* __restr
         early[i][k] = (d < vdim && p * 8 < R) ? load8(w + (size_t)d * R + 8 * p) : zero8();
       }
   }
-  constexpr int EARLY = 8;
   const size_t cell0 = ((size_t)t * H + h) * splits;
   // four channels a thread; where that leaves threads over, groups of them take the chunks in turn
   const bool by_quads = R % 4 == 0 && R <= 1024;
   const int quads = by_quads ? R / 4 : 256, groups = 256 / quads, group = tid / quads, q4 = (tid % quads) * 4;
-  f32x4 sums[EARLY];
+  const int count = min(positions[t] / chunk + 1, splits);   // chunks that hold keys
+  // every wave finds the maximum and the sum for itself (a lane a chunk, and every 64th after it): no barriers
+  const int lane = tid % kWave;
+  float m_of[kMaxSplits / kWave], l_of[kMaxSplits / kWave], top = -INFINITY, total = 0.f;
 #pragma unroll
-  for (int i = 0; i < EARLY; ++i) {
-    const int k = group + i * groups;
-    sums[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-    if (by_quads && group < groups && k < splits) sums[i] = *reinterpret_cast<const f32x4*>(ws_acc + (cell0 + k) * R + q4);
+  for (int i = 0; i < kMaxSplits / kWave; ++i) {
+    const int k = lane + kWave * i;
+    m_of[i] = k < count ? ws_ml[(cell0 + k) * 2] : -INFINITY;
+    l_of[i] = k < count ? ws_ml[(cell0 + k) * 2 + 1] : 0.f;
+    top = fmaxf(top, m_of[i]);
   }
-  const int count = min(positions[t] / chunk + 1, splits);   // chunks that hold keys (the others' sums are not of this step)
-  const float mine = tid < count ? ws_ml[(cell0 + tid) * 2] : -INFINITY, mine_l = tid < count ? ws_ml[(cell0 + tid) * 2 + 1] : 0.f;
-  const float top = block_max(mine, scratch);
-  const float f = tid < count ? exp2f(mine - top) : 0.f;
-  weight[tid] = f;
-  float total = block_sum(f * mine_l, scratch);   // (also orders the writes of weight before the reads below)
+  top = wave_max(top);
+#pragma unroll
+  for (int i = 0; i < kMaxSplits / kWave; ++i) {
+    const float f = m_of[i] == -INFINITY ? 0.f : exp2f(m_of[i] - top);
+    if (tid < kWave) weight[lane + kWave * i] = f;
+    total = fmaf(f, l_of[i], total);
+  }
+  total = wave_sum(total);
   if (sinks) total += exp2f(fmaf(sinks[h], kLog2e, -top));
   const float inv = 1.0f / total;
+  __syncthreads();
   if (by_quads) {
     f32x4 s = {0.f, 0.f, 0.f, 0.f};
     if (group < groups) {
-#pragma unroll
-      for (int i = 0; i < EARLY; ++i) {
-        const int k = group + i * groups;
-        if (k < count) s += sums[i] * weight[k];
-      }
 #pragma unroll 8
-      for (int k = group + EARLY * groups; k < count; k += groups) s += *reinterpret_cast<const f32x4*>(ws_acc + (cell0 + k) * R + q4) * weight[k];
+      for (int k = group; k < count; k += groups) s += *reinterpret_cast<const f32x4*>(ws_acc + (cell0 + k) * R + q4) * weight[k];
       *reinterpret_cast<f32x4*>(&half_sums[group * R + q4]) = s;
     }
     __syncthreads();

@@ -1312,8 +1312,8 @@ def moe_router(h: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], t
 @functools.lru_cache(maxsize=4096)
 def grouped_ring_slices(entries: int, groups: int, n_out: int, k: int) -> int:
     """Slices of k for a grouped product with tiles of 256 rows and columns: as many (up to four) as leave the compute units
-    busy to the end, if the tiles' number is what one expects of so many entries."""
-    tiles = (entries // 256 + groups // 2) * -(-n_out // 256)
+    busy to the end (a group's last tile, which holds few rows, costs little and is not counted)."""
+    tiles = max(entries // 256, groups) * -(-n_out // 256)
     cost = lambda s: -(-tiles * s // 256) / s
     return min((s for s in (1, 2, 3, 4) if k // s >= 512 or s == 1), key=cost)
 
