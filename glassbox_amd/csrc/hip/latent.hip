@@ -7,7 +7,7 @@
 // ordinary attention kernels.
 //
 //   latent_store    the RMS norm of a latent row and its way into the pages: [page][R / 8][slot][8] as a key head of R columns
-//   latent_absorb   q' [n, H * R] = W_uk^T q, head by head
+//   latent_absorb   q' [n, H * R] = W_uk^T q, head by head; latent_store_absorb both in one launch
 //   latent_decode   partial softmax sums of q' over a chunk of the context's latents, one workgroup a (chunk, 16 or 32 heads,
 //                   token); latent_decode_plain the same for any sizes and types, a workgroup a (chunk, token, head)
 //   latent_finish   the chunks' partial results added in their order, with the head's sink; W_uv; the sigmoid gate
@@ -42,13 +42,8 @@ inline bool grid_fits(long long count, int per_block) { return (count + per_bloc
 // ------------------------------------------------------------------------------------------------ latent_store
 // A wave a row.
 template <typename T>
-__global__ __launch_bounds__(256) void latent_store_kernel(const T* __restrict__ in, int ld, const float* __restrict__ gamma, float eps,
-                                                           const int32_t* __restrict__ slots, T* __restrict__ pages, int page_size,
-                                                           int n, int R, int words) {
-  const int t = blockIdx.x * 4 + threadIdx.x / kWave, lane = threadIdx.x % kWave;
-  if (t >= n) return;
-  const T* row = in + (size_t)t * ld;
-  const int slot = slots[t];
+__device__ __forceinline__ void store_latent(const T* __restrict__ row, const float* __restrict__ gamma, float eps, int slot,
+                                             T* __restrict__ pages, int page_size, int R, bool words, int lane) {
   T* page = pages + (size_t)(slot / page_size) * page_size * R;
   const int at = slot % page_size;
   float ss = 0.f;
@@ -77,13 +72,20 @@ __global__ __launch_bounds__(256) void latent_store_kernel(const T* __restrict__
   for (int c = lane; c < R; c += kWave) page[key_offset(at, c, page_size, piece)] = from_f<T>(to_f(row[c]) * r * gamma[c]);
 }
 
+template <typename T>
+__global__ __launch_bounds__(256) void latent_store_kernel(const T* __restrict__ in, int ld, const float* __restrict__ gamma, float eps,
+                                                           const int32_t* __restrict__ slots, T* __restrict__ pages, int page_size,
+                                                           int n, int R, int words) {
+  const int t = blockIdx.x * 4 + threadIdx.x / kWave;
+  if (t < n) store_latent(in + (size_t)t * ld, gamma, eps, slots[t], pages, page_size, R, words != 0, threadIdx.x % kWave);
+}
+
 // ------------------------------------------------------------------------------------------------ latent_absorb
 // A wave a (64 latent channels, head, 16 tokens): D[channel][token], A = rows of W_uk^T ([H][R][hc], 16 bytes a lane), B =
 // the tokens' queries.
-__global__ __launch_bounds__(64) void latent_absorb_kernel(const bf16* __restrict__ q, int ldq, const bf16* __restrict__ uk_t, int hc,
-                                                           bf16* __restrict__ out, int n, int H, int R) {
-  const int h = blockIdx.y, r0 = blockIdx.x * 64, t0 = blockIdx.z * 16;
-  const int lane = threadIdx.x, j = lane & 15, c = lane >> 4;
+__device__ __forceinline__ void absorb_tile(const bf16* __restrict__ q, int ldq, const bf16* __restrict__ uk_t, int hc,
+                                            bf16* __restrict__ out, int n, int H, int R, int h, int r0, int t0, int lane) {
+  const int j = lane & 15, c = lane >> 4;
   const int tok = t0 + j;
   f32x4 acc[4];
 #pragma unroll
@@ -108,6 +110,25 @@ __global__ __launch_bounds__(64) void latent_absorb_kernel(const bf16* __restric
     for (int e = 0; e < 4; ++e) o[e] = (bf16)acc[b][e];
     *reinterpret_cast<bf16x4*>(out + ((size_t)tok * H + h) * R + r) = o;
   }
+}
+
+__global__ __launch_bounds__(64) void latent_absorb_kernel(const bf16* __restrict__ q, int ldq, const bf16* __restrict__ uk_t, int hc,
+                                                           bf16* __restrict__ out, int n, int H, int R) {
+  absorb_tile(q, ldq, uk_t, hc, out, n, H, R, blockIdx.y, blockIdx.x * 64, blockIdx.z * 16, threadIdx.x);
+}
+
+// Both in one launch, for steps of few rows: workgroup y = H takes the latents (x counts rows), the others their tile of W_uk^T q
+// for the first n_q tokens.
+__global__ __launch_bounds__(64) void latent_store_absorb_kernel(const bf16* __restrict__ rows, int ld, int c_col, const float* __restrict__ gamma,
+                                                                 float eps, const int32_t* __restrict__ slots, bf16* __restrict__ pages,
+                                                                 int page_size, int n, const bf16* __restrict__ uk_t, int hc,
+                                                                 bf16* __restrict__ out, int n_q, int H, int R) {
+  if ((int)blockIdx.y == H) {
+    for (int t = blockIdx.x + gridDim.x * blockIdx.z; t < n; t += gridDim.x * gridDim.z)
+      store_latent(rows + (size_t)t * ld + c_col, gamma, eps, slots[t], pages, page_size, R, true, threadIdx.x);
+    return;
+  }
+  absorb_tile(rows, ld, uk_t, hc, out, n_q, H, R, blockIdx.y, blockIdx.x * 64, blockIdx.z * 16, threadIdx.x);
 }
 
 // A thread a (token, head, channel): uk [H * hc, R], the first dim rows of a head.
@@ -659,6 +680,21 @@ extern "C" int gb_latent_absorb(const void* q, int dtype, int ldq, const void* u
   return launched("latent_absorb");
 }
 
+// gb_latent_store and gb_latent_absorb of the first n_q rows in one launch: rows [n, ld] bfloat16 hold H query heads of hc columns
+// and the latent from column c_col on; R and hc multiples of 8, everything aligned.
+extern "C" int gb_latent_store_absorb(const void* rows, int ld, int c_col, const float* gamma, float eps, const int32_t* slots, void* pages,
+                                      int page_size, int n, const void* uk_t, int hc, void* out, int n_q, int H, int R,
+                                      hipStream_t stream) {
+  GB_REQUIRE(n_q > 0 && n >= n_q && H > 0 && H < 65535 && R > 0 && R % 8 == 0 && hc > 0 && hc % 8 == 0 && c_col >= H * hc && ld >= c_col + R,
+             "latent_store_absorb: bad sizes n=%d of %d heads=%d of %d R=%d", n_q, n, H, hc, R);
+  GB_REQUIRE(ld % 8 == 0 && c_col % 8 == 0 && words16(rows) && words16(pages) && words16(uk_t) && words16(out) && gamma && slots && page_size > 0 && n_q <= 65535 * 16,
+             "latent_store_absorb: operands must be 16-byte aligned rows");
+  const dim3 grid((unsigned)((R + 63) / 64), (unsigned)(H + 1), (unsigned)((n_q + 15) / 16));
+  hipLaunchKernelGGL(latent_store_absorb_kernel, grid, dim3(64), 0, stream, (const bf16*)rows, ld, c_col, gamma, eps, slots, (bf16*)pages,
+                     page_size, n, (const bf16*)uk_t, hc, (bf16*)out, n_q, H, R);
+  return launched("latent_store_absorb");
+}
+
 // Whether the matrix-core kernel takes latents of R channels in pages of P tokens.
 extern "C" int gb_latent_decode_takes(int R, int P) { return R >= 8 && R % 8 == 0 && R <= 512 && P >= 16 && P % 16 == 0; }
 
@@ -777,6 +813,7 @@ extern "C" int gb_latent_expand(const void* kv, int dtype, int ld, void* k_pages
 // the launches of a layer can be recorded and made again for the layers like it (common.h)
 GB_TAPED(gb_latent_store)
 GB_TAPED(gb_latent_absorb)
+GB_TAPED(gb_latent_store_absorb)
 GB_TAPED(gb_latent_decode)
 GB_TAPED(gb_latent_finish)
 GB_TAPED(gb_latent_tables)

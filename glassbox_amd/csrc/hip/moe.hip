@@ -19,7 +19,7 @@
 // in the order of their experts (entries of an expert in the order of the tokens): rows[r] is the token behind sorted
 // row r, pos[t * top + k] the sorted row of token t's k-th choice, and `map` cuts the sorted rows into row tiles that
 // lie in one expert each (three numbers a tile: expert, first row, end of the expert's rows; the tiles past the last one
-// carry expert -1); whole tiles come first, then the experts' last ones, so that a launch ends on the short work.  The products then go tile by tile with the tile's expert's matrices, and `combine` adds up, for
+// carry expert -1).  The products then go tile by tile with the tile's expert's matrices, and `combine` adds up, for
 // each token, its chosen experts' output rows times their weights in the order of the choices, and the shared
 // expert's row times its gate.
 #include "common.h"
@@ -339,22 +339,20 @@ __global__ __launch_bounds__(256) void place_kernel(const int32_t* __restrict__ 
                                                     int32_t* __restrict__ rows, int32_t* __restrict__ pos,
                                                     int32_t* __restrict__ map) {
   __shared__ int part[4];
-  __shared__ int first_row, first_tile, last_tile, all_tiles;
+  __shared__ int first_row, first_tile, all_tiles;
   const int e = blockIdx.x, lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
   if (threadIdx.x == 0) {
-    int r = 0, whole = 0, part = 0, mine = 0;
+    int r = 0, t = 0, all = 0;
     for (int o = 0; o < E; ++o) {
       if (o == e) {
         first_row = r;
-        first_tile = whole;
-        mine = part;
+        first_tile = t;
       }
       r += counts[o];
-      whole += counts[o] / tile_rows;
-      part += counts[o] % tile_rows != 0;
+      t += (counts[o] + tile_rows - 1) / tile_rows;
     }
-    last_tile = whole + mine;   // where this expert's last tile goes, if it is not whole
-    all_tiles = whole + part;
+    all = t;
+    all_tiles = all;
   }
   __syncthreads();
   const int base = first_row, mine = counts[e];
@@ -378,7 +376,7 @@ __global__ __launch_bounds__(256) void place_kernel(const int32_t* __restrict__ 
   }
   const int my_tiles = (mine + tile_rows - 1) / tile_rows;
   for (int j = threadIdx.x; j < my_tiles; j += 256) {
-    int32_t* t = map + 3 * (size_t)(j < mine / tile_rows ? first_tile + j : last_tile);
+    int32_t* t = map + 3 * (size_t)(first_tile + j);
     t[0] = e;
     t[1] = base + j * tile_rows;
     t[2] = base + mine;

@@ -120,6 +120,8 @@ _SIGS = {
         "gb_latent_store": [_vp, _i, _i, _vp, _f, _vp, _vp, _i, _i, _i, _vp],
         # q, dtype, ldq, uk, uk_t, head columns, dim, out, n, heads, R, stream
         "gb_latent_absorb": [_vp, _i, _i, _vp, _vp, _i, _i, _vp, _i, _i, _i, _vp],
+        # rows, ld, latent's column, gamma, eps, slots, pages, page size, n, uk_t, head columns, out, absorbed rows, heads, R, stream
+        "gb_latent_store_absorb": [_vp, _i, _i, _vp, _f, _vp, _vp, _i, _i, _vp, _i, _vp, _i, _i, _i, _vp],
         "gb_latent_decode_takes": [_i, _i],
         # q, dtype, pages, tables, stride, positions, tok_seq, n, heads, R, page size, scale, chunk, splits, acc, ml, plain, stream
         "gb_latent_decode": [_vp, _i, _vp, _vp, _i, _vp, _vp, _i, _i, _i, _i, _f, _i, _i, _vp, _vp, _i, _vp],
@@ -2131,6 +2133,24 @@ def latent_absorb(q: torch.Tensor, uk: torch.Tensor, uk_t: Optional[torch.Tensor
     lib = _lib("latent")
     _launch(lib, lib.gb_latent_absorb, _p(q), dtype_code(q), _act_rows(q, q.dtype, n_heads * head_cols, "q"), _p(uk), _p(uk_t),
             head_cols, dim, _p(out), n, n_heads, R, _stream())
+
+
+def latent_store_absorb(rows: torch.Tensor, latent_col: int, gamma: torch.Tensor, eps: float, slots: torch.Tensor, pages: torch.Tensor,
+                        uk_t: torch.Tensor, out: torch.Tensor) -> None:
+    """``latent_store`` of the latents that begin at column ``latent_col`` of ``rows`` (bfloat16, 16-byte aligned, query heads
+    first) and ``latent_absorb`` of the first ``out.shape[0]`` rows' heads, in one launch."""
+    _dev(rows, gamma, slots, pages, uk_t, out)
+    P, R = _latent_pages(pages, torch.bfloat16, "latent_store_absorb")
+    n, n_q = rows.shape[0], out.shape[0]
+    H, _, hc = uk_t.shape
+    _f32_rows(gamma, (R,), "gamma")
+    _i32(slots, "slots", n)
+    if (rows.dtype != torch.bfloat16 or uk_t.dtype != torch.bfloat16 or uk_t.shape[1] != R or not uk_t.is_contiguous()
+            or tuple(out.shape) != (n_q, H * R) or not out.is_contiguous() or out.dtype != torch.bfloat16 or n_q > n):
+        raise KernelError("latent_store_absorb: uk_t must be contiguous [heads, R, head columns], out contiguous [rows, heads * R]")
+    lib = _lib("latent")
+    _launch(lib, lib.gb_latent_store_absorb, _p(rows), _act_rows(rows, torch.bfloat16, latent_col + R, "rows"), int(latent_col), _p(gamma),
+            float(eps), _p(slots), _p(pages), P, n, _p(uk_t), hc, _p(out), n_q, H, R, _stream())
 
 
 @functools.lru_cache(maxsize=4096)

@@ -737,14 +737,19 @@ class LatentCacheAttention(Mixer):
         first = ctx.buffer("latent_in", (n, self.w_in.shape[0]), ctx.dtype)     # [query heads | latent | gate]
         product(ctx, h, self.w_in, first)
         gate = first[:, H * hc + R:H * hc + R + H * V]
-        ops.latent_store(first[:, H * hc:H * hc + R], self.norm_kv, self.eps, ctx.slots[cache.group], cache.k_pages)
+        slots = ctx.slots[cache.group]
         mixed = ctx.buffer("latent_mixed", (n, H * V), ctx.dtype)
         # (heads that no attention kernel takes: every row as if it came alone)
         alone = ctx.host["n_decode"] if hc <= ops.MAX_HEAD_DIM else n
+        tuned = ctx.tuned and alone == ctx.host["n_decode"] and ops.latent_tuned_takes(ctx.dtype, R, ctx.page_size)
+        q = ctx.buffer("latent_q", (alone, H * R), ctx.dtype) if alone else None
+        if alone and tuned and n <= ops.ROPE_PRODUCT_MAX_ROWS:
+            ops.latent_store_absorb(first, H * hc, self.norm_kv, self.eps, slots, cache.k_pages, self.w_uk_t, q)
+        else:
+            ops.latent_store(first[:, H * hc:H * hc + R], self.norm_kv, self.eps, slots, cache.k_pages)
+            if alone:
+                ops.latent_absorb(first[:alone, :H * hc], self.w_ukv, self.w_uk_t if tuned else None, hc, self.dim, q, H)
         if alone:
-            tuned = (ctx.tuned and alone == ctx.host["n_decode"] and ops.latent_tuned_takes(ctx.dtype, R, ctx.page_size))
-            q = ctx.buffer("latent_q", (alone, H * R), ctx.dtype)
-            ops.latent_absorb(first[:alone, :H * hc], self.w_ukv, self.w_uk_t if tuned else None, hc, self.dim, q, H)
             ops.latent_decode(q, cache.k_pages, ctx.tables[cache.group], ctx.positions[:alone], ctx.tok_seq[:alone], H, self.scale,
                               int(ctx.host["max_context"]), self.sinks, self.w_ukv[H * hc:], hc, V,
                               gate[:alone], mixed[:alone], ctx.buffer, plain=not tuned)
