@@ -155,8 +155,26 @@ def zakusun_like(shapes: dict, layers: int, experts: int = 8, top: int = 2) -> d
                 canon={"taps": 4}, logit_scale=1.0, layers=[layer] * layers)
 
 
+def zumizen_like(shapes: dict, layers: int, run: int = 1024, experts: int = 8, top: int = 2) -> dict:
+    """A Zumizen configuration with the widths of a Llama one: the two mixers in turn (side by side, attention and delta rule have
+    half of the heads each), routed experts in every layer with as many multiply-adds a token as the Llama's feed-forward."""
+    d, H, G = shapes["hidden_size"], shapes["num_attention_heads"], shapes["num_key_value_heads"]
+    hd = shapes.get("head_dim") or d // H
+    half = lambda n: max(1, n // 2)
+    moe = {"kind": "moe", "expert": {"ff": shapes["intermediate_size"] // top // 8 * 8}, "router": {"experts": experts, "top": top}}
+    left = {"heads": half(G) * (H // G), "kv_heads": half(G), "dim": hd, "vdim": hd, "scale": hd ** -0.5, "mask": {"size": run}}
+    right = {"heads": half(G) * (H // G), "kv_heads": half(G), "dim": hd, "vdim": hd, "conv": 4}
+    channel = {"heads": H, "kv_heads": G, "dim": hd, "vdim": hd, "conv": 4, "decay_rank": hd, "gate_rank": hd}
+    kinds = [{"type": "parallel", "mixer": {"left": left, "left_scale": 0.7, "right": right, "right_scale": 0.8}, "mlp": moe},
+             {"type": "channel_delta", "mixer": channel, "mlp": moe}]
+    return dict(architecture="Zumizen", vocab=shapes["vocab_size"], width=d, norm={"eps": shapes["rms_norm_eps"]}, logit_softcap=30.0,
+                embedding={"scale": 1.0, "bigram": {"buckets": 65536, "mul_prev": 1000003, "mul_cur": 31}},
+                layers=[kinds[i % 2] for i in range(layers)])
+
+
 DESIGNS = {"sagalorn": ("Sagalorn", sagalorn_like), "dekinex": ("Dekinex", dekinex_like), "vumalix": ("Vumalix", vumalix_like),
-           "tekilix": ("Tekilix", tekilix_like), "zakusun": ("Zakusun", zakusun_like)}
+           "tekilix": ("Tekilix", tekilix_like), "zakusun": ("Zakusun", zakusun_like),
+           "zumizen": ("Zumizen", zumizen_like)}
 
 
 def design_bench(a) -> int:

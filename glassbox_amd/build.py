@@ -53,6 +53,7 @@ LIBRARIES: Dict[str, tuple] = {
     "headmix": ("hip", ["hip/headmix.hip"], ["hip/common.h"]),
     "tanhmix": ("hip", ["hip/tanhmix.hip"], ["hip/common.h"]),
     "groupmix": ("hip", ["hip/groupmix.hip"], ["hip/common.h"]),
+    "delta": ("hip", ["hip/delta.hip"], ["hip/common.h"]),
     "latent": ("hip", ["hip/latent.hip"], ["hip/common.h"]),
 }
 

@@ -47,12 +47,16 @@ __device__ __forceinline__ bf16x8 zero8() {
 
 // What a mixer may ask of the softmax beyond a window: `span` > 0: positions are cut into runs of `span` from 0 on and a
 // token sees the keys of its own run up to itself (no window then); `softcap` > 0: score = softcap * tanh(score /
-// softcap); `sinks` [nh]: exp(sinks[h]) joins the denominator of head h and has no value.
+// softcap); `sinks` [nh]: exp(sinks[h]) joins the denominator of head h and has no value; `slopes` [nh]: slopes[h] times the
+// key's distance is taken off the score.  Caps and slopes are kernels of their own (MODE), so that the others' score loops
+// stay as they were.
 struct Extra {
   int span;
   float softcap;
   const float* __restrict__ sinks;
+  const float* __restrict__ slopes;
 };
+enum : int { kPlainScores = 0, kCapped = 1, kSloped = 2 };
 
 __device__ __forceinline__ int first_key(int pos, int window, int span) {
   return span > 0 ? pos - pos % span : window > 0 ? max(0, pos - window + 1) : 0;
@@ -87,11 +91,11 @@ __device__ __forceinline__ void reset(Running<HD>& st) {
 // their keys are masked anyway.
 // WIDE: the softmax weights enter the value product in two bfloat16 parts, p = hi + lo (two products), which keeps 16
 // bits of them instead of 8: for results that go on in 32-bit.
-template <int HD, bool WIDE = false, bool CAP = false>
+template <int HD, bool WIDE = false, int MODE = kPlainScores>
 __device__ __forceinline__ void attend64(Running<HD>& st, const bf16x8* qf, const bf16* __restrict__ kp,
                                          const bf16* __restrict__ vp, const int32_t* __restrict__ table, int nkv, int kvh,
                                          int P, int kbase, int lo, int hi, int clamp_lo, int clamp_hi, float scale,
-                                         int lane, float softcap = 0.f) {
+                                         int lane, float softcap = 0.f, float slope = 0.f, int pos = 0) {
   constexpr int KS = (HD + 31) / 32, DB = HD / 16;
   const int j = lane & 15, c = lane >> 4;
   bf16x8 kf[4][KS];
@@ -125,7 +129,8 @@ __device__ __forceinline__ void attend64(Running<HD>& st, const bf16x8* qf, cons
     for (int r = 0; r < 4; ++r) {
       const int key = kbase + 16 * t + 4 * c + r;
       float sc = a[r] * scale;
-      if (CAP) sc = capped_fast(a[r], scale / softcap, softcap);   // (a kernel of its own: the others' score loops stay as they were)
+      if (MODE == kCapped) sc = capped_fast(a[r], scale / softcap, softcap);
+      if (MODE == kSloped) sc = fmaf(slope, (float)(key - pos), sc);
       s[t][r] = (key >= lo && key <= hi) ? sc : -INFINITY;
       mx = fmaxf(mx, s[t][r]);
     }
@@ -190,7 +195,7 @@ __device__ __forceinline__ void store_out4(float* p, const f32x4& v) { *reinterp
 // grid (chunks, kv heads, requests); request s is row s of q and out, at position positions[s].
 // WAVES waves take 64 keys each in turn; dynamic LDS holds their partial results for the merge:
 // WAVES * (32 + HD * G) floats, G the query heads per kv head.
-template <int HD, int WAVES, typename OT, bool CAP = false>
+template <int HD, int WAVES, typename OT, int MODE = kPlainScores>
 __global__ __launch_bounds__(WAVES * 64) void decode_kernel(const bf16* __restrict__ q, int q_stride, OT* __restrict__ out,
                                                             int out_stride, float* __restrict__ ws_acc,
                                                             float* __restrict__ ws_ml, const int32_t* __restrict__ positions,
@@ -224,12 +229,13 @@ __global__ __launch_bounds__(WAVES * 64) void decode_kernel(const bf16* __restri
   Running<HD> st;
   reset(st);
   const int col_lo = col < G ? lo : 1, col_hi = col < G ? pos : 0;
+  const float slope = MODE == kSloped && col < G ? ex.slopes[kvh * G + col] : 0.f;
   const int end = min(c0 + chunk, pos + 1);
   for (int kb = c0 + wave * 64; kb < end; kb += 64 * WAVES) {
     // the kept first keys of these 64, then those inside the window (a tile can hold both kinds)
-    if (kb < kept) attend64<HD, WIDE, CAP>(st, qf, kp, vp, table, nkv, kvh, P, kb, col < G ? 0 : 1, col < G ? kept - 1 : 0, 0, kept - 1, scale, lane, ex.softcap);
+    if (kb < kept) attend64<HD, WIDE, MODE>(st, qf, kp, vp, table, nkv, kvh, P, kb, col < G ? 0 : 1, col < G ? kept - 1 : 0, 0, kept - 1, scale, lane, ex.softcap, slope, pos);
     if (kb + 64 <= lo) continue;
-    attend64<HD, WIDE, CAP>(st, qf, kp, vp, table, nkv, kvh, P, kb, col_lo, col_hi, lo, pos, scale, lane, ex.softcap);
+    attend64<HD, WIDE, MODE>(st, qf, kp, vp, table, nkv, kvh, P, kb, col_lo, col_hi, lo, pos, scale, lane, ex.softcap, slope, pos);
   }
   st.l += __shfl_xor(st.l, 16, kWave);
   st.l += __shfl_xor(st.l, 32, kWave);
@@ -421,12 +427,12 @@ __device__ __forceinline__ void load_values(bf16x8 (&vf)[(HD + 31) / 32][2 * T],
 // registers at a time; as soon as the last block's score products have read kf it is loaded again
 // for the keys from `next`, and vf likewise after the last value products, so that those loads are
 // in flight during the arithmetic in between.
-template <int HD, int QB, int ACT, int T = 2, bool WIDE = false, bool CAP = false>
+template <int HD, int QB, int ACT, int T = 2, bool WIDE = false, int MODE = kPlainScores>
 __device__ __forceinline__ void attend64_q32(float (&m)[QB], float (&l)[QB], f32x16 (&acc)[QB][(HD + 31) / 32],
                                              const bf16x8* __restrict__ q_lds, int q_at, bf16x8 (&kf)[T][HD / 16],
                                              bf16x8 (&vf)[(HD + 31) / 32][2 * T], const PageSource& src, int kbase, int next,
                                              const int (&lo)[QB], const int (&hi)[QB], bool mask, float c, int lane,
-                                             int keep = 0, float cap_in = 0.f, float cap_out = 0.f) {
+                                             int keep = 0, float cap_in = 0.f, float cap_out = 0.f, const int* pos = nullptr) {
   constexpr int KS = HD / 16, DB = (HD + 31) / 32;
   constexpr int LAST = (ACT & 2) ? 1 : 0;
   const int g = lane >> 5;
@@ -451,11 +457,19 @@ __device__ __forceinline__ void attend64_q32(float (&m)[QB], float (&l)[QB], f32
       __builtin_amdgcn_sched_barrier(0);
       load_keys<HD, T>(kf, src, next, lane);
     }
-    if (CAP) {  // capped scores, kept in the raw scores' unit (a kernel of its own: the others stay as they were)
+    if (MODE == kCapped) {  // capped scores, kept in the raw scores' unit
 #pragma unroll
       for (int t = 0; t < T; ++t)
 #pragma unroll
         for (int r = 0; r < 16; ++r) s[t][r] = capped_fast(s[t][r], cap_in, cap_out);
+    }
+    if (MODE == kSloped) {  // the distances' share, in the raw scores' unit (cap_in: slope / scale)
+      const float base = (float)(kbase + 8 * g - pos[qb]);
+#pragma unroll
+      for (int t = 0; t < T; ++t)
+#pragma unroll
+        for (int r = 0; r < 16; ++r)
+          s[t][r] = fmaf(cap_in, base + (float)(32 * t + 16 * (r >> 3) + 4 * ((r >> 2) & 1) + (r & 3)), s[t][r]);
     }
     if (mask) {  // the same for the whole wave
 #pragma unroll
@@ -636,7 +650,7 @@ __device__ __forceinline__ void hand_over(float& m, float& l, f32x16 (&acc)[DB],
 // blocks w and n-1-w of 32 tokens.  SPLIT waves share a pair: they take its tiles of 64 keys in turn, and at the
 // end the others hand their sums to the first through LDS.  One wave a pair is best when the pairs alone give
 // every SIMD a wave; short portions and few heads do not, and then the keys are what is left to divide.
-template <int HD, int QB, int PAIRS, int SPLIT, typename OT, bool CAP = false>
+template <int HD, int QB, int PAIRS, int SPLIT, typename OT, int MODE = kPlainScores>
 __global__ __launch_bounds__(64 * PAIRS * SPLIT, 2) void prefill_kernel(const bf16* __restrict__ q, int q_stride, OT* __restrict__ out,
                                                       int out_stride, const int32_t* __restrict__ q_start,
                                                       const int32_t* __restrict__ q_len, const int32_t* __restrict__ pos0,
@@ -675,7 +689,7 @@ __global__ __launch_bounds__(64 * PAIRS * SPLIT, 2) void prefill_kernel(const bf
   PageSource src{kp, vp, tables + (size_t)seq * table_stride, nkv, kvh, page_shift, 0, 0, (keep + 15) & ~15};
   const size_t row0 = (size_t)q_start[seq];
   const float c = scale * 1.4426950408889634f;
-  const float cap_in = ex.softcap > 0.f ? scale / ex.softcap : 0.f, cap_out = ex.softcap > 0.f ? ex.softcap / scale : 0.f;
+  const float cap_in = MODE == kSloped ? ex.slopes[head] / scale : ex.softcap > 0.f ? scale / ex.softcap : 0.f, cap_out = ex.softcap > 0.f ? ex.softcap / scale : 0.f;
   // a sink's share of a token's denominator, given the token's running maximum (in the raw scores' unit)
   auto sink_of = [&](float m) { return ex.sinks ? __builtin_amdgcn_exp2f(ex.sinks[head] * 1.4426950408889634f - m * c) : 0.f; };
   constexpr int T = QB == 2 ? 2 : 1;  // tiles of 32 keys a step: with one block live at a time (the larger head
@@ -694,7 +708,7 @@ __global__ __launch_bounds__(64 * PAIRS * SPLIT, 2) void prefill_kernel(const bf
   const bool has_second = blocks - 1 - w > w;
 
   if constexpr (QB == 2) {
-    int lo[2], hi[2];
+    int lo[2], hi[2], at[2];   // at: the tokens' positions
     float m[2], l[2];
     f32x16 acc[2][DB];
     BlockRange range[2];
@@ -705,6 +719,7 @@ __global__ __launch_bounds__(64 * PAIRS * SPLIT, 2) void prefill_kernel(const bf
       const int p = p0 + tok;
       lo[qb] = valid ? first_key(p, window, ex.span) : 1;
       hi[qb] = valid ? p : 0;
+      at[qb] = p;
 #pragma unroll
       for (int ks = 0; ks < KS; ++ks)
         qf[(qb * KS + ks) * 64] = valid ? load8(q + (row0 + tok) * q_stride + (size_t)head * HD + 16 * ks + 8 * g) : zero8();
@@ -745,29 +760,29 @@ __global__ __launch_bounds__(64 * PAIRS * SPLIT, 2) void prefill_kernel(const bf
       const int kept_tiles = (keep + 63) & ~63;
       while (kb <= range[0].last && kb < kept_tiles) {
         const int next = my_next(kb);
-        attend64_q32<HD, 2, 3, 2, WIDE, CAP>(m, l, acc, q_lds, q_at, kf, vf, src, kb, next, lo, hi, true, c, lane, keep, cap_in, cap_out);
+        attend64_q32<HD, 2, 3, 2, WIDE, MODE>(m, l, acc, q_lds, q_at, kf, vf, src, kb, next, lo, hi, true, c, lane, keep, cap_in, cap_out, at);
         kb = next;
       }
       while (kb <= range[0].last && kb + 63 < range[1].first) {
         const int next = my_next(kb);
-        attend64_q32<HD, 2, 1, 2, WIDE, CAP>(m, l, acc, q_lds, q_at, kf, vf, src, kb, next, lo, hi, !range[0].unmasked(kb), c, lane, keep, cap_in, cap_out);
+        attend64_q32<HD, 2, 1, 2, WIDE, MODE>(m, l, acc, q_lds, q_at, kf, vf, src, kb, next, lo, hi, !range[0].unmasked(kb), c, lane, keep, cap_in, cap_out, at);
         kb = next;
       }
       while (kb <= range[0].last) {
         const int next = my_next(kb);
         const bool mask = !(range[0].unmasked(kb) && range[1].unmasked(kb));
-        attend64_q32<HD, 2, 3, 2, WIDE, CAP>(m, l, acc, q_lds, q_at, kf, vf, src, kb, next, lo, hi, mask, c, lane, keep, cap_in, cap_out);
+        attend64_q32<HD, 2, 3, 2, WIDE, MODE>(m, l, acc, q_lds, q_at, kf, vf, src, kb, next, lo, hi, mask, c, lane, keep, cap_in, cap_out, at);
         kb = next;
       }
       while (kb <= range[1].last) {
         const int next = my_next(kb);
-        attend64_q32<HD, 2, 2, 2, WIDE, CAP>(m, l, acc, q_lds, q_at, kf, vf, src, kb, next, lo, hi, !range[1].unmasked(kb), c, lane, keep, cap_in, cap_out);
+        attend64_q32<HD, 2, 2, 2, WIDE, MODE>(m, l, acc, q_lds, q_at, kf, vf, src, kb, next, lo, hi, !range[1].unmasked(kb), c, lane, keep, cap_in, cap_out, at);
         kb = next;
       }
     } else {
       while (kb <= range[0].last) {
         const int next = my_next(kb);
-        attend64_q32<HD, 2, 1, 2, WIDE, CAP>(m, l, acc, q_lds, q_at, kf, vf, src, kb, next, lo, hi, !range[0].unmasked(kb), c, lane, keep, cap_in, cap_out);
+        attend64_q32<HD, 2, 1, 2, WIDE, MODE>(m, l, acc, q_lds, q_at, kf, vf, src, kb, next, lo, hi, !range[0].unmasked(kb), c, lane, keep, cap_in, cap_out, at);
         kb = next;
       }
     }
@@ -795,6 +810,7 @@ __global__ __launch_bounds__(64 * PAIRS * SPLIT, 2) void prefill_kernel(const bf
       const bool valid = tok < qlen;
       const int p = p0 + tok;
       int lo[1] = {valid ? first_key(p, window, ex.span) : 1}, hi[1] = {valid ? p : 0};
+      const int at[1] = {p};
       float m[1] = {-INFINITY}, l[1] = {0.f};
       f32x16 acc[1][DB];
 #pragma unroll
@@ -816,8 +832,8 @@ __global__ __launch_bounds__(64 * PAIRS * SPLIT, 2) void prefill_kernel(const bf
       load_keys<HD, T>(kf, src, key_of(i0), lane);
       load_values<HD, T>(vf, src, key_of(i0), lane);
       for (int i = i0; key_of(i) <= range.last; i += stride)
-        attend64_q32<HD, 1, 1, T, WIDE, CAP>(m, l, acc, q_lds, q_at, kf, vf, src, key_of(i), key_of(i + stride), lo, hi,
-                                  !range.unmasked(key_of(i), SPAN), c, lane, keep, cap_in, cap_out);
+        attend64_q32<HD, 1, 1, T, WIDE, MODE>(m, l, acc, q_lds, q_at, kf, vf, src, key_of(i), key_of(i + stride), lo, hi,
+                                  !range.unmasked(key_of(i), SPAN), c, lane, keep, cap_in, cap_out, at);
       if constexpr (SPLIT > 1) {
         hand_over<DB, SPLIT>(m[0], l[0], acc[0], handed[wave], handed_ml[wave], half, lane, c, which > 0);
         if (half != 0) continue;
@@ -846,7 +862,7 @@ template <typename OT>
 static int decode_launch(const void* q, int q_stride, OT* out, int out_stride, void* ws_acc, void* ws_ml,
                          const int32_t* positions, const int32_t* tables, int table_stride, const void* k_pages,
                          const void* v_pages, int n_decode, int nh, int nkv, int hd, int page_size, float scale, int window,
-                         int keep_first, int chunk, int max_context, hipStream_t stream, Extra ex = Extra{0, 0.f, nullptr}) {
+                         int keep_first, int chunk, int max_context, hipStream_t stream, Extra ex = Extra{0, 0.f, nullptr, nullptr}) {
   GB_REQUIRE(keep_first >= 0 && (keep_first == 0 || window > 0), "attention_decode: kept first keys go with a window");
   GB_REQUIRE(ex.span >= 0 && (ex.span == 0 || window == 0) && ex.softcap >= 0.f, "attention_decode: runs of positions exclude a window; a cap is positive or 0");
   GB_REQUIRE(n_decode >= 0 && nh > 0 && nkv > 0 && nh % nkv == 0, "attention_decode: bad head counts nh=%d nkv=%d", nh, nkv);
@@ -868,25 +884,31 @@ static int decode_launch(const void* q, int q_stride, OT* out, int out_stride, v
   const int waves = (splits == 1 && max_context > 512 && hd <= 64 && 16 * (32 + (size_t)hd * G) * sizeof(float) <= 65536) ? 16 : 4;
   const size_t lds = (size_t)waves * (32 + (size_t)hd * G) * sizeof(float);
   const dim3 grid(splits, nkv, n_decode), block(waves * 64);
-  // capped scores are a kernel of their own (bfloat16 results only), so that the others' score loops are what they were
+  // capped and sloped scores are kernels of their own (bfloat16 results only), so that the others' score loops are what they were
   constexpr bool kCanCap = std::is_same<OT, bf16>::value;
-  const bool cap = ex.softcap > 0.f;
-  GB_REQUIRE(!cap || kCanCap, "attention_decode: capped scores with float32 result rows are not served");
-#define GB_DECODE(HD, WAVES, CAP)                                                                                          \
-  hipLaunchKernelGGL((decode_kernel<HD, WAVES, OT, CAP>), grid, block, lds, stream, (const bf16*)q, q_stride, out, out_stride, \
+  const bool cap = ex.softcap > 0.f, sloped = ex.slopes != nullptr;
+  GB_REQUIRE(!(cap || sloped) || kCanCap, "attention_decode: capped or sloped scores with float32 result rows are not served");
+  GB_REQUIRE(!(cap && sloped), "attention_decode: scores with a cap and slopes are not served");
+#define GB_DECODE(HD, WAVES, MODE)                                                                                         \
+  hipLaunchKernelGGL((decode_kernel<HD, WAVES, OT, MODE>), grid, block, lds, stream, (const bf16*)q, q_stride, out, out_stride, \
                      (float*)ws_acc, (float*)ws_ml, positions, tables, table_stride, (const bf16*)k_pages,                  \
                      (const bf16*)v_pages, nh, nkv, page_size, scale, window, keep_first, chunk, splits, ex)
 #define GB_CASE(HD)                                                 \
   if (hd == HD) {                                                   \
     if (cap) {                                                      \
       if constexpr (kCanCap) {                                      \
-        if (waves == 16) GB_DECODE(HD, 16, true);                   \
-        else GB_DECODE(HD, 4, true);                                \
+        if (waves == 16) GB_DECODE(HD, 16, kCapped);                \
+        else GB_DECODE(HD, 4, kCapped);                             \
+      }                                                             \
+    } else if (sloped) {                                            \
+      if constexpr (kCanCap) {                                      \
+        if (waves == 16) GB_DECODE(HD, 16, kSloped);                \
+        else GB_DECODE(HD, 4, kSloped);                             \
       }                                                             \
     } else if (waves == 16) {                                       \
-      GB_DECODE(HD, 16, false);                                     \
+      GB_DECODE(HD, 16, kPlainScores);                                   \
     } else {                                                        \
-      GB_DECODE(HD, 4, false);                                      \
+      GB_DECODE(HD, 4, kPlainScores);                                    \
     }                                                               \
   }
   GB_FOR_HEAD_SIZES(GB_CASE)
@@ -1031,7 +1053,7 @@ static int prefill_launch(const void* q, int q_stride, OT* out, int out_stride, 
                           const int32_t* pos0, int seq_base, int n_seqs, int max_q_len, int max_context, const int32_t* tables,
                           int table_stride, const void* k_pages, const void* v_pages, int nh, int nkv, int hd, int page_size,
                           float scale, int window, int keep_first, int first_row, int n_rows, float* part_ws,
-                          long long part_floats, hipStream_t stream, Extra ex = Extra{0, 0.f, nullptr}) {
+                          long long part_floats, hipStream_t stream, Extra ex = Extra{0, 0.f, nullptr, nullptr}) {
   GB_REQUIRE(keep_first >= 0 && (keep_first == 0 || window > 0), "attention_prefill: kept first keys go with a window");
   GB_REQUIRE(ex.span >= 0 && (ex.span == 0 || window == 0) && ex.softcap >= 0.f, "attention_prefill: runs of positions exclude a window; a cap is positive or 0");
   GB_REQUIRE(n_seqs >= 0 && nh > 0 && nkv > 0 && nh % nkv == 0, "attention_prefill: bad head counts nh=%d nkv=%d", nh, nkv);
@@ -1055,21 +1077,25 @@ static int prefill_launch(const void* q, int q_stride, OT* out, int out_stride, 
     part_ml = part_ws + cells * hd;
   }
   const dim3 grid((max_q_len + 64 * per_group - 1) / (64 * per_group) * parts, nh, n_seqs), block(64 * per_group * split);
-  // capped scores are a kernel of their own (bfloat16 results only), so that the others' score loops are what they were
+  // capped and sloped scores are kernels of their own (bfloat16 results only), so that the others' score loops are what they were
   constexpr bool kCanCap = std::is_same<OT, bf16>::value;
-  const bool cap = ex.softcap > 0.f;
-  GB_REQUIRE(!cap || kCanCap, "attention_prefill: capped scores with float32 result rows are not served");
-#define GB_LAUNCH_AS(HD, QB, PAIRS, SPLIT, CAP)                                                                             \
-  hipLaunchKernelGGL((prefill_kernel<HD, QB, PAIRS, SPLIT, OT, CAP>), grid, block, 0, stream, (const bf16*)q, q_stride, out, \
+  const bool cap = ex.softcap > 0.f, sloped = ex.slopes != nullptr;
+  GB_REQUIRE(!(cap || sloped) || kCanCap, "attention_prefill: capped or sloped scores with float32 result rows are not served");
+  GB_REQUIRE(!(cap && sloped), "attention_prefill: scores with a cap and slopes are not served");
+  GB_REQUIRE(!sloped || scale > 0.f, "attention_prefill: slopes need a positive scale");
+#define GB_LAUNCH_AS(HD, QB, PAIRS, SPLIT, MODE)                                                                            \
+  hipLaunchKernelGGL((prefill_kernel<HD, QB, PAIRS, SPLIT, OT, MODE>), grid, block, 0, stream, (const bf16*)q, q_stride, out, \
                      out_stride, q_start, q_len, pos0, seq_base, tables, table_stride, (const bf16*)k_pages,               \
                      (const bf16*)v_pages, nh, nkv, page_shift, scale, window, keep_first, part_acc, part_ml, parts, first_row, \
                      n_rows, ex)
 #define GB_LAUNCH(HD, QB, PAIRS, SPLIT)                            \
   do {                                                             \
     if (cap) {                                                     \
-      if constexpr (kCanCap) GB_LAUNCH_AS(HD, QB, PAIRS, SPLIT, true); \
+      if constexpr (kCanCap) GB_LAUNCH_AS(HD, QB, PAIRS, SPLIT, kCapped); \
+    } else if (sloped) {                                           \
+      if constexpr (kCanCap) GB_LAUNCH_AS(HD, QB, PAIRS, SPLIT, kSloped); \
     } else {                                                       \
-      GB_LAUNCH_AS(HD, QB, PAIRS, SPLIT, false);                   \
+      GB_LAUNCH_AS(HD, QB, PAIRS, SPLIT, kPlainScores);                  \
     }                                                              \
   } while (0)
 #define GB_CASE(HD)                                        \
@@ -1134,13 +1160,13 @@ extern "C" int gb_attention_prefill_bf16(const void* q, int q_stride, void* out,
 }
 
 // The same two with everything a mixer may ask of the softmax: a window with kept first keys, or runs of `span`
-// positions; capped scores; sinks [nh] (see Extra).  out32 != 0: float32 result rows.
+// positions; capped scores; sinks [nh]; slopes [nh] (see Extra).  out32 != 0: float32 result rows.
 extern "C" int gb_attention_decode_bf16_by(const void* q, int q_stride, void* out, int out_stride, int out32, void* ws_acc,
                                            void* ws_ml, const int32_t* positions, const int32_t* tables, int table_stride,
                                            const void* k_pages, const void* v_pages, int n_decode, int nh, int nkv, int hd,
                                            int page_size, float scale, int window, int keep_first, int span, float softcap,
-                                           const float* sinks, int chunk, int max_context, hipStream_t stream) {
-  const Extra ex{span, softcap, sinks};
+                                           const float* sinks, const float* slopes, int chunk, int max_context, hipStream_t stream) {
+  const Extra ex{span, softcap, sinks, slopes};
   if (out32) {
     GB_REQUIRE((uintptr_t)out % 16 == 0, "attention_decode: float32 result rows must be 16-byte aligned");
     return decode_launch<float>(q, q_stride, (float*)out, out_stride, ws_acc, ws_ml, positions, tables, table_stride, k_pages,
@@ -1155,9 +1181,9 @@ extern "C" int gb_attention_prefill_bf16_by(const void* q, int q_stride, void* o
                                             int n_seqs, int max_q_len, int max_context, const int32_t* tables, int table_stride,
                                             const void* k_pages, const void* v_pages, int nh, int nkv, int hd, int page_size,
                                             float scale, int window, int keep_first, int span, float softcap,
-                                            const float* sinks, int first_row, int n_rows, float* part_ws,
+                                            const float* sinks, const float* slopes, int first_row, int n_rows, float* part_ws,
                                             long long part_floats, hipStream_t stream) {
-  const Extra ex{span, softcap, sinks};
+  const Extra ex{span, softcap, sinks, slopes};
   if (out32) {
     GB_REQUIRE((uintptr_t)out % 16 == 0, "attention_prefill: float32 result rows must be 16-byte aligned");
     return prefill_launch<float>(q, q_stride, (float*)out, out_stride, q_start, q_len, pos0, seq_base, n_seqs, max_q_len,

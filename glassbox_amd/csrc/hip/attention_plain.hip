@@ -7,7 +7,8 @@
 // table, lo = 0 or p - window + 1 (crates/glassbox-core/src/model.rs:285-312):
 //   score = dot(q, k) * scale ; prob = softmax(score) ; out = sum prob * v
 // Options: `span` > 0: positions are cut into runs of `span` from 0 on and lo is the first position of p's run (a token
-// sees its own run only); `softcap` > 0: score = softcap * tanh(score / softcap); `sinks`: one number a query head whose
+// sees its own run only); `softcap` > 0: score = softcap * tanh(score / softcap); `slopes`: one number a query head,
+// slopes[h] * (p - key's position) is taken off the score (behind the cap); `sinks`: one number a query head whose
 // exponential joins the softmax's denominator and which has no value (the weights then sum to less than one).
 //
 // The order of every addition depends on the token's position alone, not on the batch and not
@@ -99,9 +100,12 @@ struct Shape {
   int span;   // > 0: a token sees the keys of its own run of `span` positions (runs counted from position 0)
   float softcap;        // > 0: scores pass softcap * tanh(score / softcap)
   const float* sinks;   // [nh] or null: exp(sinks[h]) is added to the softmax's denominator of head h
-  __device__ __forceinline__ float score(float dot) const {
-    const float s = dot * scale;
-    return softcap > 0.f ? softcap * tanhf(s / softcap) : s;
+  const float* slopes;  // [nh] or null: slopes[h] * (distance of the key) is taken off the score
+  __device__ __forceinline__ float slope(int h) const { return slopes ? slopes[h] : 0.f; }
+  __device__ __forceinline__ float score(float dot, float slope, int distance) const {
+    float s = dot * scale;
+    if (softcap > 0.f) s = softcap * tanhf(s / softcap);
+    return slopes ? fmaf(-slope, (float)distance, s) : s;
   }
 };
 
@@ -127,8 +131,8 @@ struct Chunks {
 template <typename T, int PER>
 __device__ __forceinline__ void chunk_alone(const Shape& sh, const float* qs, float* es, float* scratch,
                                             const int32_t* __restrict__ table, const T* __restrict__ k_pages,
-                                            const T* __restrict__ v_pages, int kvh, int c0, int hi, float& m_c, float& l_c,
-                                            float (&a_c)[PER]) {
+                                            const T* __restrict__ v_pages, int kvh, float slope, int pos, int c0, int hi, float& m_c,
+                                            float& l_c, float (&a_c)[PER]) {
   const int tid = threadIdx.x;
   const int ps = sh.page_size, hd = sh.hd;
   const int p = c0 + tid;
@@ -136,7 +140,7 @@ __device__ __forceinline__ void chunk_alone(const Shape& sh, const float* qs, fl
   if (p <= hi) {
     const int page = table[p / ps];
     const T* kb = k_pages + ((size_t)page * sh.nkv + kvh) * ps * hd;
-    s = sh.score(key_dot<T>(qs, kb, p % ps, hd, ps, key_piece(hd)));
+    s = sh.score(key_dot<T>(qs, kb, p % ps, hd, ps, key_piece(hd)), slope, pos - p);
   }
   m_c = block_max(s, scratch);
   const float e = p <= hi ? expf(s - m_c) : 0.f;
@@ -206,6 +210,7 @@ __global__ __launch_bounds__(kChunk) void attention_plain_kernel(
   const Chunks ch(sh, pos);
   const int n_chunks = ch.n;
   const int tid = threadIdx.x;
+  const float slope = sh.slope(h);
   if (SPLIT && (int)blockIdx.y >= n_chunks) return;
 
   for (int d = tid; d < sh.hd; d += kChunk) qs[d] = to_f(q[(size_t)t * q_stride + (size_t)h * sh.hd + d]);
@@ -214,7 +219,7 @@ __global__ __launch_bounds__(kChunk) void attention_plain_kernel(
   if (SPLIT) {
     const int c = blockIdx.y, c0 = ch.first(c);
     float m_c, l_c, a_c[PER];
-    chunk_alone<T, PER>(sh, qs, es, scratch, table, k_pages, v_pages, kvh, c0, ch.last(c, pos), m_c, l_c, a_c);
+    chunk_alone<T, PER>(sh, qs, es, scratch, table, k_pages, v_pages, kvh, slope, pos, c0, ch.last(c, pos), m_c, l_c, a_c);
     float* cell = ws + ((size_t)blockIdx.x * max_chunks + c) * ws_stride(PER);
 #pragma unroll
     for (int u = 0; u < PER; ++u) cell[u * kChunk + tid] = a_c[u];
@@ -231,7 +236,7 @@ __global__ __launch_bounds__(kChunk) void attention_plain_kernel(
   for (int c = 0; c < n_chunks; ++c) {
     const int c0 = ch.first(c);
     float m_c, l_c, a_c[PER];
-    chunk_alone<T, PER>(sh, qs, es, scratch, table, k_pages, v_pages, kvh, c0, ch.last(c, pos), m_c, l_c, a_c);
+    chunk_alone<T, PER>(sh, qs, es, scratch, table, k_pages, v_pages, kvh, slope, pos, c0, ch.last(c, pos), m_c, l_c, a_c);
     merge_chunk<PER>(r, acc, m_c, l_c, a_c);
   }
   finish<T, PER>(sh, comb, acc, r, h, out + (size_t)t * out_stride + (size_t)h * sh.hd);
@@ -310,8 +315,8 @@ static_assert(kChunk / kWave == 4, "block_reduce keeps four waves' parts a value
 template <typename T, int PER, int Q>
 __device__ __forceinline__ void chunk_together(const Shape& sh, const T* __restrict__ q0, int q_stride, float* es, float* scratch,
                                                const int32_t* __restrict__ table, const T* __restrict__ k_pages,
-                                               const T* __restrict__ v_pages, int kvh, int c0, const int (&hi)[Q],
-                                               float (&m_c)[Q], float (&l_c)[Q], float (&a_c)[Q][PER]) {
+                                               const T* __restrict__ v_pages, int kvh, float slope, int pos0, int c0,
+                                               const int (&hi)[Q], float (&m_c)[Q], float (&l_c)[Q], float (&a_c)[Q][PER]) {
   const int tid = threadIdx.x;
   const int ps = sh.page_size, hd = sh.hd;
   const int p = c0 + tid;
@@ -326,7 +331,7 @@ __device__ __forceinline__ void chunk_together(const Shape& sh, const T* __restr
     key_dots<T, Q>(q0, q_stride, kb, p % ps, hd, ps, key_piece(hd), dot);
 #pragma unroll
     for (int j = 0; j < Q; ++j)
-      if (p <= hi[j]) s[j] = sh.score(dot[j]);
+      if (p <= hi[j]) s[j] = sh.score(dot[j], slope, pos0 + j - p);
   }
 #pragma unroll
   for (int j = 0; j < Q; ++j) m_c[j] = s[j];
@@ -391,7 +396,7 @@ __device__ __forceinline__ void walk_together(const Shape& sh, const T* __restri
 #pragma unroll
     for (int j = 0; j < Q; ++j) hi[j] = min(c0 + kChunk - 1, pos0 + j);
     float m_c[Q], l_c[Q], a_c[Q][PER];
-    chunk_together<T, PER, Q>(sh, q0, q_stride, es, scratch, table, k_pages, v_pages, kvh, c0, hi, m_c, l_c, a_c);
+    chunk_together<T, PER, Q>(sh, q0, q_stride, es, scratch, table, k_pages, v_pages, kvh, sh.slope(h), pos0, c0, hi, m_c, l_c, a_c);
 #pragma unroll
     for (int j = 0; j < Q; ++j)
       if (c0 <= pos0 + j) merge_chunk<PER>(r[j], acc[j], m_c[j], l_c[j], a_c[j]);
@@ -431,6 +436,7 @@ __global__ __launch_bounds__(kChunk) void attention_plain_group_kernel(
     qs[e] = to_f(q[(size_t)(first + j) * q_stride + (size_t)h * sh.hd + d]);
   }
   __syncthreads();
+  const float slope = sh.slope(h);
   for (int j = 0; j < count; ++j) {   // one after the other, as a workgroup of the one-token form would
     const int t = first + j;
     const int pos = positions[t];
@@ -444,7 +450,7 @@ __global__ __launch_bounds__(kChunk) void attention_plain_group_kernel(
     for (int c = 0; c < n_chunks; ++c) {
       const int c0 = ch.first(c);
       float m_c, l_c, a_c[PER];
-      chunk_alone<T, PER>(sh, qs + j * sh.hd, es, scratch + kGroup * 4, table, k_pages, v_pages, kvh, c0,
+      chunk_alone<T, PER>(sh, qs + j * sh.hd, es, scratch + kGroup * 4, table, k_pages, v_pages, kvh, slope, pos, c0,
                           ch.last(c, pos), m_c, l_c, a_c);
       merge_chunk<PER>(r, acc, m_c, l_c, a_c);
     }
@@ -549,7 +555,7 @@ extern "C" int gb_attention_plain(const void* q, int q_stride, void* out, int ou
                                   const int32_t* positions, const int32_t* tok_seq, const int32_t* tables,
                                   int table_stride, const void* k_pages, const void* v_pages, int n, int nh, int nkv,
                                   int hd, int page_size, float scale, int window, int keep_first, int span,
-                                  float softcap, const float* sinks, float* ws, long long ws_floats, int max_context,
+                                  float softcap, const float* sinks, const float* slopes, float* ws, long long ws_floats, int max_context,
                                   int grouped, hipStream_t stream) {
   GB_REQUIRE(n >= 0 && nh > 0 && nkv > 0 && hd > 0, "attention_plain: bad sizes n=%d nh=%d nkv=%d hd=%d", n, nh, nkv, hd);
   GB_REQUIRE(nh % nkv == 0, "attention_plain: %d query heads are not a multiple of %d key heads", nh, nkv);
@@ -575,7 +581,7 @@ extern "C" int gb_attention_plain(const void* q, int q_stride, void* out, int ou
                "attention_plain: the workspace holds %lld floats, %lld are needed", ws_floats,
                gb_attention_plain_split_floats(n, nh, hd, page_size, max_context, keep_first));
   }
-  const Shape sh{nh, nkv, hd, page_size, window, table_stride, scale, keep_first, span, softcap, sinks};
+  const Shape sh{nh, nkv, hd, page_size, window, table_stride, scale, keep_first, span, softcap, sinks, slopes};
   if (dtype == kF32)
     return launch_by_pairs<float>(per, q, q_stride, out, out_stride, positions, tok_seq, tables, k_pages, v_pages, n, sh, ws,
                                   max_chunks, grouped != 0, stream);

@@ -811,6 +811,20 @@ __global__ void scale_rows_kernel(float* __restrict__ x, float s, long long coun
   if (i < count) x[i] *= s;
 }
 
+// x = cap * tanh(scale * x / cap)   (float32: logits that a model bounds)
+__global__ void cap_rows_kernel(float* __restrict__ x, float scale, float cap, long long count) {
+  const long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i < count) x[i] = cap * tanhf(x[i] * scale / cap);
+}
+
+extern "C" int gb_cap_rows(float* x, float scale, float cap, long long count, hipStream_t stream) {
+  GB_REQUIRE(count >= 0 && (count + 255) / 256 < (1ll << 31), "cap_rows: bad size %lld", count);
+  GB_REQUIRE(cap > 0.f, "cap_rows: the cap must be positive");
+  if (count == 0) return 0;
+  hipLaunchKernelGGL(cap_rows_kernel, dim3((unsigned)((count + 255) / 256)), dim3(256), 0, stream, x, scale, cap, count);
+  return launched("cap_rows");
+}
+
 extern "C" int gb_scale_rows(float* x, float s, long long count, hipStream_t stream) {
   GB_REQUIRE(count >= 0 && (count + 255) / 256 < (1ll << 31), "scale_rows: bad size %lld", count);
   if (count == 0) return 0;
@@ -833,7 +847,7 @@ extern "C" int gb_add_bias(float* x, const float* bias, int n, int d, hipStream_
 }
 
 // ------------------------------------------------------------------------ embedding with a hashed pair table
-// x[c, i, :] = table[ids[i], :] + pairs[row, :], row = (previous token * mul_prev + ids[i] * mul_cur) mod buckets, and
+// x[c, i, :] = scale * table[ids[i], :] + pairs[row, :], row = (previous token * mul_prev + ids[i] * mul_cur) mod buckets, and
 // row `buckets` (the table's last) for a request's first token.  The token before a step's first row of a request is
 // kept in the request's state slot (`prev`, one int32 a slot): the block of that first row reads it, unless the request
 // starts at position 0, and leaves the request's last token of this step there; no other block touches the slot.
@@ -842,7 +856,8 @@ __global__ void embed_pairs_kernel(const T* __restrict__ table, const T* __restr
                                    float* __restrict__ x, int n, int d, int vocab, int buckets, long long mul_prev,
                                    long long mul_cur, const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ q_start,
                                    const int32_t* __restrict__ q_len, const int32_t* __restrict__ pos0,
-                                   const int32_t* __restrict__ state_slots, int32_t* __restrict__ prev, int copies) {
+                                   const int32_t* __restrict__ state_slots, int32_t* __restrict__ prev, int copies,
+                                   float scale) {
   __shared__ int s_before;
   const int i = blockIdx.x;
   const int id = ids[i];
@@ -869,7 +884,7 @@ __global__ void embed_pairs_kernel(const T* __restrict__ table, const T* __restr
   const T* trow = table + (size_t)(ok ? id : 0) * d;
   const T* prow = pairs + (size_t)(ok ? row : 0) * d;
   for (int c = threadIdx.x; c < d; c += blockDim.x) {
-    const float v = ok ? to_f(trow[c]) + to_f(prow[c]) : __builtin_nanf("");  // a bad id must not pass silently
+    const float v = ok ? fmaf(scale, to_f(trow[c]), to_f(prow[c])) : __builtin_nanf("");  // a bad id must not pass silently
     for (int k = 0; k < copies; ++k) x[((size_t)k * n + i) * d + c] = v;
   }
 }
@@ -877,7 +892,7 @@ __global__ void embed_pairs_kernel(const T* __restrict__ table, const T* __restr
 extern "C" int gb_embed_pairs(const void* table, const void* pairs, int dtype, const int32_t* ids, float* x, int n, int d,
                               int vocab, int buckets, long long mul_prev, long long mul_cur, const int32_t* tok_seq,
                               const int32_t* q_start, const int32_t* q_len, const int32_t* pos0, const int32_t* state_slots,
-                              int32_t* prev, int copies, hipStream_t stream) {
+                              int32_t* prev, int copies, float scale, hipStream_t stream) {
   GB_REQUIRE(n >= 0 && d > 0 && vocab > 0 && buckets > 0 && copies > 0, "embed_pairs: bad sizes n=%d d=%d vocab=%d buckets=%d",
              n, d, vocab, buckets);
   GB_REQUIRE(tok_seq && q_start && q_len && pos0 && state_slots && prev, "embed_pairs: the step's tables and the state are needed");
@@ -885,10 +900,10 @@ extern "C" int gb_embed_pairs(const void* table, const void* pairs, int dtype, c
   const int threads = d >= 256 ? 256 : 64;
   if (dtype == kF32)
     hipLaunchKernelGGL(embed_pairs_kernel<float>, dim3(n), dim3(threads), 0, stream, (const float*)table, (const float*)pairs,
-                       ids, x, n, d, vocab, buckets, mul_prev, mul_cur, tok_seq, q_start, q_len, pos0, state_slots, prev, copies);
+                       ids, x, n, d, vocab, buckets, mul_prev, mul_cur, tok_seq, q_start, q_len, pos0, state_slots, prev, copies, scale);
   else if (dtype == kBF16)
     hipLaunchKernelGGL(embed_pairs_kernel<bf16>, dim3(n), dim3(threads), 0, stream, (const bf16*)table, (const bf16*)pairs,
-                       ids, x, n, d, vocab, buckets, mul_prev, mul_cur, tok_seq, q_start, q_len, pos0, state_slots, prev, copies);
+                       ids, x, n, d, vocab, buckets, mul_prev, mul_cur, tok_seq, q_start, q_len, pos0, state_slots, prev, copies, scale);
   else
     return fail("embed_pairs: unknown dtype %d", dtype);
   return launched("embed_pairs");

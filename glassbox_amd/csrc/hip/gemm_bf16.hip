@@ -133,6 +133,7 @@ struct Groups {
   long long w_stride;
   int up_off;
   int slice_rows;   // rows of C a slice of k (the ring kernel's grouped form)
+  const float* in_scale;   // with EPI_SILU_MUL, if given: what each row of A is multiplied by (both sums are, before the unit)
 };
 
 template <int WM, int WN, int DEPTH, int EPI, bool KFULL, typename CT, bool GROUPED = false>
@@ -310,7 +311,11 @@ __global__ __launch_bounds__(256, WN == 2 ? 2 : 1) void gemm_tiled_kernel(const 
 #pragma unroll
       for (int r = 0; r < 16; ++r) {
         const int gm = m0 + wm * 32 * WM + i * 32 + 8 * (r / 4) + 4 * (lane / 32) + r % 4;
-        const float g = acc[i][0][r], u = acc[i][WN - 1][r];
+        float g = acc[i][0][r], u = acc[i][WN - 1][r];
+        if (GROUPED && grp.in_scale) {
+          const float s = grp.in_scale[min(gm, M - 1)];
+          g *= s, u *= s;
+        }
         if (gm < M) c[(size_t)gm * ldc + gn] = (CT)gated_unit(g, u, glu);
       }
     return;
@@ -624,7 +629,11 @@ __global__ __launch_bounds__(RGM * RGN * 64, 1) void gemm_ring_kernel(const bf16
 #pragma unroll
         for (int r = 0; r < 16; ++r) {
           const int gm = m0 + wm * RTM * 32 + i * 32 + 8 * (r / 4) + 4 * (lane / 32) + r % 4;
-          const float g = acc[i][2 * p][r], u = acc[i][2 * p + 1][r];
+          float g = acc[i][2 * p][r], u = acc[i][2 * p + 1][r];
+          if (GROUPED && grp.in_scale) {
+            const float s = grp.in_scale[min(gm, M - 1)];
+            g *= s, u *= s;
+          }
           if (gm < M) c[(size_t)gm * ldc + gn] = (CT)gated_unit(g, u, glu);
         }
     }
@@ -1910,11 +1919,12 @@ extern "C" int gb_gemm_bf16_glu(const void* a, int lda, const void* w, int ldw, 
 // group's W starts w_stride elements behind the one before.  Epilogue 0 stores (bfloat16 or float32), 2 forms
 // silu(gate) * up, or the clamped unit (limit, alpha, plus: see Glu), from the N / 2 gate rows of a group and the up rows
 // up_off rows behind them.  Tiles of 256 rows go through the ring kernel, which may divide k into `slices` (float32 results
-// without an epilogue): slice z's sums lie z * slice_rows rows further on in C.
+// without an epilogue): slice z's sums lie z * slice_rows rows further on in C.  in_scale (with epilogue 2, or nullptr): one
+// number a row of the product, which the row of A counts times.
 extern "C" int gb_gemm_bf16_grouped(const void* a, int lda, const int32_t* rows, const void* w, int ldw, long long w_stride,
                                     int up_off, void* c, int ldc, int c_dtype, const int32_t* map, int tiles, int tile_rows,
                                     int N, int K, int epilogue, float limit, float alpha, float plus, int slices, int slice_rows,
-                                    hipStream_t stream) {
+                                    const float* in_scale, hipStream_t stream) {
   GB_REQUIRE(limit > 0.f, "gemm_bf16_grouped: the unit's limit must be positive");
   GB_REQUIRE(tiles >= 0 && N > 0 && K > 0 && (tile_rows == 64 || tile_rows == 128 || tile_rows == 256), "gemm_bf16_grouped: bad sizes tiles=%d of %d rows, N=%d K=%d",
              tiles, tile_rows, N, K);
@@ -1930,7 +1940,7 @@ extern "C" int gb_gemm_bf16_grouped(const void* a, int lda, const int32_t* rows,
   if (tiles == 0) return 0;
   GB_REQUIRE(slices >= 1 && (slices == 1 || (tile_rows == 256 && epilogue == EPI_STORE && c_dtype == kF32 && slice_rows > 0)),
              "gemm_bf16_grouped: %d slices of k go with tiles of 256 rows and float32 results", slices);
-  const Groups grp{map, rows, w_stride, up_off, slice_rows};
+  const Groups grp{map, rows, w_stride, up_off, slice_rows, in_scale};
   const bf16* A = (const bf16*)a;
   const bf16* W = (const bf16*)w;
   if (tile_rows == 256) {

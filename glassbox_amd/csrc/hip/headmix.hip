@@ -18,7 +18,7 @@
 //   diff_combine   o = a1 - lambda a2 for every head, divided by its root mean square over vdim, times a constant.
 //   gate_heads     out = heads * sigmoid(gate), the heads' zero columns dropped.
 //   poly_norm      a N(z) + b N(z^2) + c N(z^3) + e over a row, N(v) = v / sqrt(mean(v^2) + eps).
-//   norm_add       x += g * y / sqrt(mean(y^2) + eps), g one number; optionally the new x rounded to the activations' type.
+//   norm_add       x += g * y / sqrt(mean(y^2) + eps), g one number or one a column, y optionally with a bias first; optionally the new x rounded to the activations' type.
 //
 // All arithmetic is 32-bit; a value is rounded once, when it is stored in the activations' type.
 #include "common.h"
@@ -670,16 +670,21 @@ __global__ __launch_bounds__(THREADS) void poly_norm_rows_kernel(const T* __rest
 // ------------------------------------------------------------------------------------------------ norm_add
 template <typename T>
 __global__ __launch_bounds__(256) void norm_add_kernel(float* __restrict__ x, const float* __restrict__ y,
-                                                       const float* __restrict__ g, float eps, T* __restrict__ rounded, int d) {
+                                                       const float* __restrict__ g, int g_cols, const float* __restrict__ bias,
+                                                       float eps, T* __restrict__ rounded, int d) {
   __shared__ float scratch[17];
   const float* yr = y + (size_t)blockIdx.x * d;
   float* xr = x + (size_t)blockIdx.x * d;
   float ss = 0.f;
-  for (int c = threadIdx.x; c < d; c += blockDim.x) ss = fmaf(yr[c], yr[c], ss);
-  ss = block_sum(ss, scratch);
-  const float r = g[0] / sqrtf(ss / (float)d + eps);
   for (int c = threadIdx.x; c < d; c += blockDim.x) {
-    const float v = fmaf(yr[c], r, xr[c]);
+    const float v = yr[c] + (bias ? bias[c] : 0.f);
+    ss = fmaf(v, v, ss);
+  }
+  ss = block_sum(ss, scratch);
+  const float r = (g_cols ? 1.f : g[0]) / sqrtf(ss / (float)d + eps);
+  for (int c = threadIdx.x; c < d; c += blockDim.x) {
+    const float in = yr[c] + (bias ? bias[c] : 0.f);
+    const float v = fmaf(in, g_cols ? r * g[c] : r, xr[c]);
     xr[c] = v;
     if (rounded) rounded[(size_t)blockIdx.x * d + c] = from_f<T>(v);
   }
@@ -691,7 +696,8 @@ __global__ __launch_bounds__(256) void norm_add_kernel(float* __restrict__ x, co
 // next mixer reads of it, x + conv(x), with the request's slot moved on as time_conv does.
 template <typename T, int THREADS, int WORDS>
 __global__ __launch_bounds__(THREADS) void norm_add_rows_kernel(float* __restrict__ x, const float* __restrict__ y, int slices,
-                                                                long long slice_stride, const float* __restrict__ g, float eps,
+                                                                long long slice_stride, const float* __restrict__ g, int g_cols,
+                                                                const float* __restrict__ bias, float eps,
                                                                 T* __restrict__ rounded, int d, const float* __restrict__ conv_w,
                                                                 int taps, float* __restrict__ state,
                                                                 const int32_t* __restrict__ tok_seq,
@@ -709,12 +715,13 @@ __global__ __launch_bounds__(THREADS) void norm_add_rows_kernel(float* __restric
     if (c < d) {
       f32x4 sum = *reinterpret_cast<const f32x4*>(yr + c);
       for (int z = 1; z < slices; ++z) sum += *reinterpret_cast<const f32x4*>(yr + (size_t)z * slice_stride + c);
+      if (bias) sum += *reinterpret_cast<const f32x4*>(bias + c);
       v[i] = sum;
       ss += sum[0] * sum[0] + sum[1] * sum[1] + sum[2] * sum[2] + sum[3] * sum[3];
     }
   }
   ss = block_sum(ss, scratch);
-  const float r = g[0] / sqrtf(ss / (float)d + eps);
+  const float r = (g_cols ? 1.f : g[0]) / sqrtf(ss / (float)d + eps);
   const int K = taps - 1;
   int seq = 0, pos = 0;
   if (conv_w) seq = tok_seq[t], pos = pos0[seq];
@@ -724,9 +731,10 @@ __global__ __launch_bounds__(THREADS) void norm_add_rows_kernel(float* __restric
     const int c = (threadIdx.x + i * THREADS) * 4;
     if (c < d) {
       const f32x4 old = *reinterpret_cast<const f32x4*>(xr + c);
-      f32x4 nx;
+      f32x4 nx, rg = {r, r, r, r};
+      if (g_cols) rg = *reinterpret_cast<const f32x4*>(g + c) * r;
 #pragma unroll
-      for (int e = 0; e < 4; ++e) nx[e] = fmaf(v[i][e], r, old[e]);
+      for (int e = 0; e < 4; ++e) nx[e] = fmaf(v[i][e], rg[e], old[e]);
       *reinterpret_cast<f32x4*>(xr + c) = nx;
       if (conv_w) {
         f32x4 acc = {0.f, 0.f, 0.f, 0.f};
@@ -975,12 +983,12 @@ extern "C" int gb_poly_norm(const void* z, int ldz, const float* coef, float eps
   return launched("poly_norm");
 }
 
-// x, y [n, d] float32, g one float32 on the device; rounded (or nullptr) [n, d] of `dtype` receives the new x.
+// x, y [n, d] float32, g one float32 on the device (g_cols: one a column, [d]); bias (or nullptr) float32 [d] is added to y first; rounded (or nullptr) [n, d] of `dtype` receives the new x.
 // slices > 1: y is the sum of that many [n, d] pieces, slice_stride floats apart.  conv_w (float32 [taps, d]; a step in
 // which every request brings one row): rounded receives x + conv(x) of the new x, and the requests' slots in
 // state [slots, taps - 1, d] are moved on by this row.
-extern "C" int gb_norm_add(float* x, const float* y, int slices, long long slice_stride, const float* g, float eps,
-                           void* rounded, int dtype, int n, int d, const float* conv_w, int taps, float* state,
+extern "C" int gb_norm_add(float* x, const float* y, int slices, long long slice_stride, const float* g, int g_cols,
+                           const float* bias, float eps, void* rounded, int dtype, int n, int d, const float* conv_w, int taps, float* state,
                            const int32_t* tok_seq, const int32_t* pos0, const int32_t* state_slots, hipStream_t stream) {
   GB_REQUIRE(n >= 0 && n <= 0x7fffffff && d > 0 && x && y && g, "norm_add: bad sizes n=%d d=%d", n, d);
   GB_REQUIRE(slices >= 1 && (slices == 1 || slice_stride >= (long long)n * d), "norm_add: %d slices", slices);
@@ -988,22 +996,22 @@ extern "C" int gb_norm_add(float* x, const float* y, int slices, long long slice
              "norm_add: the convolution needs a result, weights of at most %d taps, the step's tables and the state", kMaxTaps);
   if (n == 0) return 0;
   const bool words = d % 4 == 0 && d <= 8192 && words16(x) && words16(y) && words16(rounded) && words16(state) && words16(conv_w) &&
-                     slice_stride % 4 == 0;
+                     slice_stride % 4 == 0 && (!g_cols || words16(g)) && words16(bias);
   GB_REQUIRE(words || (slices == 1 && !conv_w), "norm_add: slices and the convolution take rows of at most 8192 columns, a multiple of 4");
   if (words) {
     if (n < 512) {
       GB_BY_DTYPE(dtype, "norm_add",
                   hipLaunchKernelGGL((norm_add_rows_kernel<TT, 1024, 2>), dim3((unsigned)n), dim3(1024), 0, stream, x, y, slices,
-                                     slice_stride, g, eps, (TT*)rounded, d, conv_w, taps, state, tok_seq, pos0, state_slots))
+                                     slice_stride, g, g_cols, bias, eps, (TT*)rounded, d, conv_w, taps, state, tok_seq, pos0, state_slots))
     } else {
       GB_BY_DTYPE(dtype, "norm_add",
                   hipLaunchKernelGGL((norm_add_rows_kernel<TT, 256, 8>), dim3((unsigned)n), dim3(256), 0, stream, x, y, slices,
-                                     slice_stride, g, eps, (TT*)rounded, d, conv_w, taps, state, tok_seq, pos0, state_slots))
+                                     slice_stride, g, g_cols, bias, eps, (TT*)rounded, d, conv_w, taps, state, tok_seq, pos0, state_slots))
     }
     return launched("norm_add");
   }
   GB_BY_DTYPE(dtype, "norm_add",
-              hipLaunchKernelGGL(norm_add_kernel<TT>, dim3((unsigned)n), dim3(256), 0, stream, x, y, g, eps, (TT*)rounded, d))
+              hipLaunchKernelGGL(norm_add_kernel<TT>, dim3((unsigned)n), dim3(256), 0, stream, x, y, g, g_cols, bias, eps, (TT*)rounded, d))
   return launched("norm_add");
 }
 

@@ -12,7 +12,8 @@
 // `route` leaves the result in two forms: the chosen experts and their weights a token ([n, top]), and a row of E
 // weights a token with zeros for the experts not chosen (with `shared`, one more column: sigmoid of z's column E, the
 // gate of an expert that every token uses).  `gated_units` turns the stacked gate and up projections of all experts
-// into act = silu(gate) * up * weight (or a clamped unit, see UnitOf), so that one product with the experts' down matrices side by side adds up
+// into act = silu(gate) * up * weight (or a clamped unit, see UnitOf; or with the weight on what goes into the expert: gate
+// and up sums are multiplied by it before the unit), so that one product with the experts' down matrices side by side adds up
 // sum_e a_e y_e over the token's experts (an expert not chosen contributes exact zeros).
 //
 // With many tokens a step, the experts run on the rows that chose them alone.  `sort` puts the (token, choice) entries
@@ -165,12 +166,12 @@ __global__ __launch_bounds__(4 * kWave) void route_kernel(const float* __restric
     }
 }
 
-// Logits and route in one kernel, for the router that chooses by z = W h + bias and weighs by the softmax over the chosen (up to
-// kWave experts): a workgroup a token, its waves take the experts in turn, a wave a dot product; then lane e of the first wave
+// Logits and route in one kernel, for the router that chooses by z = W h + bias and weighs by the softmax over the chosen, or
+// (sigmoid) by the sigmoids of the chosen logits as they stand (up to kWave experts): a workgroup a token, its waves take the experts in turn, a wave a dot product; then lane e of the first wave
 // holds expert e, and the number of experts that go before it (a larger logit, or the same and a lower number) is its place.
 template <typename T>
 __global__ __launch_bounds__(256) void router_kernel(const T* __restrict__ h, int ldh, const T* __restrict__ w, int ldw, int d, int words,
-                                                     int E, const float* __restrict__ bias, int top, float scale,
+                                                     int E, const float* __restrict__ bias, int top, float scale, int sigmoid,
                                                      float* __restrict__ combine, int32_t* __restrict__ ids, float* __restrict__ wts) {
   __shared__ float z[kWave];
   const int t = blockIdx.x, lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
@@ -204,8 +205,13 @@ __global__ __launch_bounds__(256) void router_kernel(const T* __restrict__ h, in
     ahead += (v > mine || (v == mine && o < lane)) ? 1 : 0;
   }
   const bool chosen = lane < E && ahead < top;
-  const float s = expf(mine - wave_max(mine));
-  const float a = s * (scale / (wave_sum(chosen ? s : 0.f) + 1e-20f));
+  float a;
+  if (sigmoid) {
+    a = scale / (1.0f + expf(-mine));
+  } else {
+    const float s = expf(mine - wave_max(mine));
+    a = s * (scale / (wave_sum(chosen ? s : 0.f) + 1e-20f));
+  }
   if (lane < E) combine[(size_t)t * E + lane] = chosen ? a : 0.f;
   if (chosen) {
     ids[(size_t)t * top + ahead] = lane;
@@ -228,7 +234,7 @@ struct UnitOf {
 // the experts' up columns, then the shared expert's gate columns and its up columns.
 template <typename I, typename O>
 __global__ void gated_units_kernel(const I* __restrict__ gu, int ld, const float* __restrict__ combine, int cols, O* __restrict__ act,
-                                   long long count, int inter, int E, int ff, UnitOf unit) {
+                                   long long count, int inter, int E, int ff, UnitOf unit, int weigh_in) {
   const long long idx = (long long)blockIdx.x * blockDim.x + threadIdx.x;
   if (idx >= count) return;
   const long long t = idx / inter;
@@ -240,14 +246,14 @@ __global__ void gated_units_kernel(const I* __restrict__ gu, int ld, const float
   if (w != 0.f) {
     const I* row = gu + (size_t)t * ld;
     const int at = j < routed ? j : 2 * routed + (j - routed), up = j < routed ? routed : inter - routed;
-    y = unit(to_f(row[at]), to_f(row[at + up])) * w;
+    y = weigh_in ? unit(to_f(row[at]) * w, to_f(row[at + up]) * w) : unit(to_f(row[at]), to_f(row[at + up])) * w;
   }
   act[idx] = from_f<O>(y);
 }
 
 // The same from 32-bit sums, four columns a thread (experts of whole groups of four columns, aligned rows).
 __global__ void gated_units_words_kernel(const float* __restrict__ gu, int ld, const float* __restrict__ combine, int cols,
-                                         bf16* __restrict__ act, long long count, int inter, int E, int ff, UnitOf unit) {
+                                         bf16* __restrict__ act, long long count, int inter, int E, int ff, UnitOf unit, int weigh_in) {
   const long long idx = (long long)blockIdx.x * blockDim.x + threadIdx.x;
   if (idx >= count) return;
   const int words = inter / 4, j = (int)(idx % words) * 4, routed = E * ff;
@@ -259,7 +265,7 @@ __global__ void gated_units_words_kernel(const float* __restrict__ gu, int ld, c
     const int at = j < routed ? j : 2 * routed + (j - routed), up = j < routed ? routed : inter - routed;
     const f32x4 g = *reinterpret_cast<const f32x4*>(row + at), u = *reinterpret_cast<const f32x4*>(row + at + up);
 #pragma unroll
-    for (int e = 0; e < 4; ++e) o[e] = (bf16)(unit(g[e], u[e]) * w);
+    for (int e = 0; e < 4; ++e) o[e] = (bf16)(weigh_in ? unit(g[e] * w, u[e] * w) : unit(g[e], u[e]) * w);
   } else {
 #pragma unroll
     for (int e = 0; e < 4; ++e) o[e] = (bf16)0.f;
@@ -333,11 +339,13 @@ __global__ __launch_bounds__(256) void count_kernel(const int32_t* __restrict__ 
 }
 
 // Workgroup e places expert e's entries behind those of the experts before it, in the order of the entries, and writes
-// its row tiles; the last workgroup also marks the tiles that are left over.
+// its row tiles; the last workgroup also marks the tiles that are left over.  row_wts (or nullptr) receives each sorted row's
+// weight out of `wts` [n, top].
 __global__ __launch_bounds__(256) void place_kernel(const int32_t* __restrict__ ids, int entries, int top, int E,
                                                     const int32_t* __restrict__ counts, int tile_rows, int tiles,
                                                     int32_t* __restrict__ rows, int32_t* __restrict__ pos,
-                                                    int32_t* __restrict__ map) {
+                                                    int32_t* __restrict__ map, const float* __restrict__ wts,
+                                                    float* __restrict__ row_wts) {
   __shared__ int part[4];
   __shared__ int first_row, first_tile, all_tiles;
   const int e = blockIdx.x, lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
@@ -371,6 +379,7 @@ __global__ __launch_bounds__(256) void place_kernel(const int32_t* __restrict__ 
       const int r = base + placed + ahead + before;
       rows[r] = i / top;
       pos[i] = r;
+      if (row_wts) row_wts[r] = wts[i];
     }
     placed += part[0] + part[1] + part[2] + part[3];
   }
@@ -390,7 +399,7 @@ __global__ __launch_bounds__(256) void place_kernel(const int32_t* __restrict__ 
     }
 }
 
-// out[t] (+)= sum over k of wts[t, k] * y[pos[t, k]]  +  gates[t * ldg] * y_shared[t]; four columns a thread.  y is the sum of
+// out[t] (+)= sum over k of wts[t, k] (1 without wts) * y[pos[t, k]]  +  gates[t * ldg] * y_shared[t]; four columns a thread.  y is the sum of
 // `slices` pieces, slice_stride floats apart (what a product that divides k leaves), added in their order.
 __global__ __launch_bounds__(256) void combine_kernel(const float* __restrict__ y, int ldy, const int32_t* __restrict__ pos,
                                                       const float* __restrict__ wts, int top, const float* __restrict__ ysh,
@@ -402,7 +411,7 @@ __global__ __launch_bounds__(256) void combine_kernel(const float* __restrict__ 
   const int t = (int)(idx / quads), c = (int)(idx % quads) * 4;
   float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
   for (int k = 0; k < top; ++k) {
-    const float w = wts[(size_t)t * top + k];
+    const float w = wts ? wts[(size_t)t * top + k] : 1.f;
     // an entry whose expert is none (a row of logits that are no numbers) was never placed: any row will do for it
     const int r = min(max(pos[(size_t)t * top + k], 0), y_rows - 1);
     float4 v = *reinterpret_cast<const float4*>(y + (size_t)r * ldy + c);
@@ -461,17 +470,17 @@ extern "C" int gb_moe_route(const float* z, int ldz, int n, int E, const float* 
 
 // h [n, ldh] and w [E, ldw] of `dtype`, d columns each; bias float32 [E] or nullptr; combine [n, E], ids and wts [n, top].
 extern "C" int gb_moe_router(const void* h, int dtype, int ldh, const void* w, int ldw, int n, int d, int E, const float* bias, int top,
-                             float scale, float* combine, int32_t* ids, float* wts, hipStream_t stream) {
+                             float scale, int sigmoid, float* combine, int32_t* ids, float* wts, hipStream_t stream) {
   GB_REQUIRE(n >= 0 && d > 0 && ldh >= d && ldw >= d && h && w && combine && ids && wts, "moe_router: bad sizes n=%d d=%d", n, d);
   GB_REQUIRE(E > 0 && E <= kWave && top > 0 && top <= E, "moe_router: %d chosen experts of %d (at most %d)", top, E, kWave);
   if (n == 0) return 0;
   const int words = dtype == kBF16 && d % 8 == 0 && ldh % 8 == 0 && ldw % 8 == 0 && (uintptr_t)h % 16 == 0 && (uintptr_t)w % 16 == 0;
   if (dtype == kF32)
     hipLaunchKernelGGL(router_kernel<float>, dim3((unsigned)n), dim3(256), 0, stream, (const float*)h, ldh, (const float*)w, ldw, d, words, E,
-                       bias, top, scale, combine, ids, wts);
+                       bias, top, scale, sigmoid, combine, ids, wts);
   else if (dtype == kBF16)
     hipLaunchKernelGGL(router_kernel<bf16>, dim3((unsigned)n), dim3(256), 0, stream, (const bf16*)h, ldh, (const bf16*)w, ldw, d, words, E,
-                       bias, top, scale, combine, ids, wts);
+                       bias, top, scale, sigmoid, combine, ids, wts);
   else
     return fail("moe_router: unknown dtype %d", dtype);
   return launched("moe_router");
@@ -505,9 +514,10 @@ extern "C" int gb_moe_relu2_units(const void* z, int in_dtype, int ld, const flo
   return launched("moe_relu2_units");
 }
 
-// The unit's numbers: limit (INFINITY: none), alpha, plus (see UnitOf; INFINITY, 1, 0 is silu(gate) * up).
+// The unit's numbers: limit (INFINITY: none), alpha, plus (see UnitOf; INFINITY, 1, 0 is silu(gate) * up).  weigh_in: a token's
+// weight for an expert multiplies the expert's gate and up sums instead of its unit.
 extern "C" int gb_moe_gated_units(const void* gu, int in_dtype, int ld, const float* combine, int cols, void* act, int out_dtype,
-                                  int n, int inter, int E, int ff, float limit, float alpha, float plus, hipStream_t stream) {
+                                  int n, int inter, int E, int ff, float limit, float alpha, float plus, int weigh_in, hipStream_t stream) {
   GB_REQUIRE(n >= 0 && inter > 0 && ld >= 2 * inter && E >= 0 && ff > 0 && E * ff <= inter && cols >= E + (E * ff < inter ? 1 : 0),
              "moe_gated_units: bad sizes n=%d inter=%d experts=%d of %d cols=%d", n, inter, E, ff, cols);
   GB_REQUIRE(limit > 0.f, "moe_gated_units: the limit must be positive");
@@ -517,16 +527,16 @@ extern "C" int gb_moe_gated_units(const void* gu, int in_dtype, int ld, const fl
   const UnitOf unit{limit, alpha, plus};
   if (in_dtype == kF32 && out_dtype == kBF16 && inter % 4 == 0 && ff % 4 == 0 && ld % 4 == 0 && (uintptr_t)gu % 16 == 0 && (uintptr_t)act % 8 == 0) {
     hipLaunchKernelGGL(gated_units_words_kernel, dim3((unsigned)((count / 4 + 255) / 256)), dim3(256), 0, stream, (const float*)gu, ld,
-                       combine, cols, (bf16*)act, count / 4, inter, E, ff, unit);
+                       combine, cols, (bf16*)act, count / 4, inter, E, ff, unit, weigh_in);
     return launched("moe_gated_units");
   }
   const dim3 grid((unsigned)((count + 255) / 256));
   if (in_dtype == kF32 && out_dtype == kF32)
-    hipLaunchKernelGGL((gated_units_kernel<float, float>), grid, dim3(256), 0, stream, (const float*)gu, ld, combine, cols, (float*)act, count, inter, E, ff, unit);
+    hipLaunchKernelGGL((gated_units_kernel<float, float>), grid, dim3(256), 0, stream, (const float*)gu, ld, combine, cols, (float*)act, count, inter, E, ff, unit, weigh_in);
   else if (in_dtype == kF32 && out_dtype == kBF16)
-    hipLaunchKernelGGL((gated_units_kernel<float, bf16>), grid, dim3(256), 0, stream, (const float*)gu, ld, combine, cols, (bf16*)act, count, inter, E, ff, unit);
+    hipLaunchKernelGGL((gated_units_kernel<float, bf16>), grid, dim3(256), 0, stream, (const float*)gu, ld, combine, cols, (bf16*)act, count, inter, E, ff, unit, weigh_in);
   else if (in_dtype == kBF16 && out_dtype == kBF16)
-    hipLaunchKernelGGL((gated_units_kernel<bf16, bf16>), grid, dim3(256), 0, stream, (const bf16*)gu, ld, combine, cols, (bf16*)act, count, inter, E, ff, unit);
+    hipLaunchKernelGGL((gated_units_kernel<bf16, bf16>), grid, dim3(256), 0, stream, (const bf16*)gu, ld, combine, cols, (bf16*)act, count, inter, E, ff, unit, weigh_in);
   else
     return fail("moe_gated_units: no kernel for operand type %d and result type %d", in_dtype, out_dtype);
   return launched("moe_gated_units");
@@ -536,13 +546,14 @@ extern "C" int gb_moe_gated_units(const void* gu, int in_dtype, int ld, const fl
 extern "C" int gb_moe_sort_tiles(int entries, int E, int tile_rows) { return entries / tile_rows + E; }
 
 extern "C" int gb_moe_sort(const int32_t* ids, int n, int top, int E, int tile_rows, int tiles, int32_t* counts, int32_t* rows,
-                           int32_t* pos, int32_t* map, hipStream_t stream) {
+                           int32_t* pos, int32_t* map, const float* wts, float* row_wts, hipStream_t stream) {
+  GB_REQUIRE(!row_wts || wts, "moe_sort: rows' weights without the entries' weights");
   GB_REQUIRE(n >= 0 && top > 0 && E > 0 && tile_rows > 0 && (long long)n * top < (1ll << 31), "moe_sort: bad sizes n=%d top=%d experts=%d", n, top, E);
   GB_REQUIRE(tiles >= gb_moe_sort_tiles(n * top, E, tile_rows), "moe_sort: %d row tiles, %d may be needed", tiles,
              gb_moe_sort_tiles(n * top, E, tile_rows));
   if (n == 0) return 0;
   hipLaunchKernelGGL(count_kernel, dim3(E), dim3(256), 0, stream, ids, n * top, counts);
-  hipLaunchKernelGGL(place_kernel, dim3(E), dim3(256), 0, stream, ids, n * top, top, E, counts, tile_rows, tiles, rows, pos, map);
+  hipLaunchKernelGGL(place_kernel, dim3(E), dim3(256), 0, stream, ids, n * top, top, E, counts, tile_rows, tiles, rows, pos, map, wts, row_wts);
   return launched("moe_sort");
 }
 

@@ -121,7 +121,7 @@ __global__ __launch_bounds__(256) void tanh_norm_add_words_kernel(float* __restr
 //      over dk, weights [dk] that all heads share;
 //   4. the first `rot` channels of every query and key head turn by the step's angles (cos, sin [n, rot / 2], times
 //      mag): neighbours = channel 2i with 2i + 1, else channel i with i + rot / 2;
-//   5. heads of hd >= max(dk, dv) columns in `out`, zeros beyond their channels; with `slots` keys and values also go
+//   5. value heads times `vscale`; heads of hd >= max(dk, dv) columns in `out`, zeros beyond their channels; with `slots` keys and values also go
 //      to their pages.
 // `single` (every request brings one row): the thread that reads a channel's slot also moves it on by one.
 template <typename T>
@@ -132,7 +132,7 @@ __global__ void qk_heads_kernel(
     const float* __restrict__ wk, float eps, int joint, const float* __restrict__ cosv, const float* __restrict__ sinv, int rot,
     float mag, int neighbours, int tied, T* __restrict__ out, int ldo, int hd, const int32_t* __restrict__ slots,
     T* __restrict__ k_pages, T* __restrict__ v_pages, int page_size, int nh, int nkv, int dk, int dv,
-    const float* __restrict__ sums) {
+    const float* __restrict__ sums, float vscale) {
   extern __shared__ float lds[];
   const int qd = nh * dk, kd = nkv * dk, channels = qd + kd, heads = nh + nkv;
   float* vals = lds;              // [dk]: the head's channels after step 1
@@ -231,7 +231,7 @@ __global__ void qk_heads_kernel(
   for (int c = tid; c < hd; c += step) {
     float r = 0.f;
     if (c < dv) r = tied ? vals[c] : to_f(row[channels + g * dv + c]) + (bias ? bias[channels + g * dv + c] : 0.f);
-    const T o = from_f<T>(r);
+    const T o = from_f<T>(r * vscale);
     vrow[c] = o;
     if (vb) vb[(size_t)c * page_size + slot % page_size] = o;
   }
@@ -255,7 +255,7 @@ __global__ __launch_bounds__(256) void qk_heads_words_kernel(
     const float* __restrict__ wk, float eps, int joint, const float* __restrict__ cosv, const float* __restrict__ sinv, int rot,
     float mag, int neighbours, int tied, bf16* __restrict__ out, int ldo, int hd, const int32_t* __restrict__ slots,
     bf16* __restrict__ k_pages, bf16* __restrict__ v_pages, int page_size, int nh, int nkv, int dk, int dv,
-    const float* __restrict__ sums, int lanes, long long units) {
+    const float* __restrict__ sums, int lanes, long long units, float vscale) {
   const int qd = nh * dk, kd = nkv * dk, channels = qd + kd, heads = nh + nkv;
   const long long gl = (long long)blockIdx.x * 256 + threadIdx.x;
   const long long unit = gl / lanes;
@@ -371,11 +371,11 @@ __global__ __launch_bounds__(256) void qk_heads_words_kernel(
   if (c0 < dv) {
     if (tied) {
 #pragma unroll
-      for (int e = 0; e < 8; ++e) val[e] = (bf16)v[e];
+      for (int e = 0; e < 8; ++e) val[e] = (bf16)(v[e] * vscale);
     } else {
       const bf16x8 x = *reinterpret_cast<const bf16x8*>(row + channels + g * dv + c0);
 #pragma unroll
-      for (int e = 0; e < 8; ++e) val[e] = (bf16)((float)x[e] + (bias ? bias[channels + g * dv + c0 + e] : 0.f));
+      for (int e = 0; e < 8; ++e) val[e] = (bf16)(((float)x[e] + (bias ? bias[channels + g * dv + c0 + e] : 0.f)) * vscale);
     }
   } else {
 #pragma unroll
@@ -558,7 +558,7 @@ extern "C" int gb_qk_heads(const void* proj, int dtype, int ld, const float* bia
                            const int32_t* tok_seq, const int32_t* q_start, const int32_t* pos0, const int32_t* state_slots,
                            int flags, const float* wq, const float* wk, float eps, const float* cosv, const float* sinv, int rot,
                            float mag, void* out, int ldo, int hd, const int32_t* slots, void* k_pages, void* v_pages,
-                           int page_size, int n, int nh, int nkv, int dk, int dv, hipStream_t stream) {
+                           int page_size, int n, int nh, int nkv, int dk, int dv, float vscale, hipStream_t stream) {
   const int single = flags & 1, joint = (flags >> 1) & 1, neighbours = (flags >> 2) & 1, tied = (flags >> 3) & 1, taps = flags >> 8;
   GB_REQUIRE(n >= 0 && nh > 0 && nkv > 0 && dk > 0 && dv > 0 && hd >= dk && hd >= dv, "qk_heads: bad sizes nh=%d nkv=%d dk=%d dv=%d hd=%d", nh, nkv, dk, dv, hd);
   GB_REQUIRE(!tied || dv == dk, "qk_heads: values that are the keys have the keys' size (dk=%d, dv=%d)", dk, dv);
@@ -593,17 +593,17 @@ extern "C" int gb_qk_heads(const void* proj, int dtype, int ld, const float* bia
     const long long units = (long long)n * (nh + nkv), threads_all = units * lanes;
     hipLaunchKernelGGL(qk_heads_words_kernel, dim3((unsigned)((threads_all + 255) / 256)), dim3(256), 0, stream, (const bf16*)proj, ld, bias,
                        wconv, taps, state, tok_seq, q_start, pos0, state_slots, single, wq, wk, eps, joint, cosv, sinv, rot, mag, neighbours,
-                       tied, (bf16*)out, ldo, hd, slots, (bf16*)k_pages, (bf16*)v_pages, page_size, nh, nkv, dk, dv, sums, lanes, units);
+                       tied, (bf16*)out, ldo, hd, slots, (bf16*)k_pages, (bf16*)v_pages, page_size, nh, nkv, dk, dv, sums, lanes, units, vscale);
     return launched("qk_heads");
   }
   if (dtype == kF32)
     hipLaunchKernelGGL(qk_heads_kernel<float>, dim3((unsigned)(n * (nh + nkv))), dim3(threads), lds, stream, (const float*)proj, ld, bias, wconv, taps,
                        state, tok_seq, q_start, pos0, state_slots, single, wq, wk, eps, joint, cosv, sinv, rot, mag, neighbours, tied,
-                       (float*)out, ldo, hd, slots, (float*)k_pages, (float*)v_pages, page_size, nh, nkv, dk, dv, sums);
+                       (float*)out, ldo, hd, slots, (float*)k_pages, (float*)v_pages, page_size, nh, nkv, dk, dv, sums, vscale);
   else if (dtype == kBF16)
     hipLaunchKernelGGL(qk_heads_kernel<bf16>, dim3((unsigned)(n * (nh + nkv))), dim3(threads), lds, stream, (const bf16*)proj, ld, bias, wconv, taps,
                        state, tok_seq, q_start, pos0, state_slots, single, wq, wk, eps, joint, cosv, sinv, rot, mag, neighbours, tied,
-                       (bf16*)out, ldo, hd, slots, (bf16*)k_pages, (bf16*)v_pages, page_size, nh, nkv, dk, dv, sums);
+                       (bf16*)out, ldo, hd, slots, (bf16*)k_pages, (bf16*)v_pages, page_size, nh, nkv, dk, dv, sums, vscale);
   else
     return fail("qk_heads: unknown dtype %d", dtype);
   return launched("qk_heads");

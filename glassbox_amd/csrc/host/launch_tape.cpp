@@ -11,7 +11,7 @@
 
 namespace {
 
-constexpr int kMaxArgs = 32;
+constexpr int kMaxArgs = 40;
 
 struct GbTapeEntry {
   uint64_t entry;     // address of the `_taped` form of the entry point

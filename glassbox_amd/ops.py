@@ -52,12 +52,13 @@ _SIGS = {
         "gb_qk_norm_store": [_vp, _i, _i, _vp, _vp, _vp, _vp, _f, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _vp],
         "gb_add_bias": [_vp, _vp, _i, _i, _vp],
         "gb_scale_rows": [_vp, _f, C.c_longlong, _vp],
+        "gb_cap_rows": [_vp, _f, _f, C.c_longlong, _vp],
         # a, lda, w, ldw, c, ldc, operand dtype, result dtype, M, N, K, accumulate, stream
         "gb_gemm_plain": [_vp, _i, _vp, _i, _vp, _i, _i, _i, _i, _i, _i, _i, _vp],
         # table, pairs, dtype, ids, x, n, d, vocab, buckets, mul_prev, mul_cur, tok_seq, q_start, q_len, pos0, state slots,
-        # prev, copies, stream
+        # prev, copies, scale, stream
         "gb_embed_pairs": [_vp, _vp, _i, _vp, _vp, _i, _i, _i, _i, C.c_longlong, C.c_longlong, _vp, _vp, _vp, _vp, _vp, _vp,
-                           _i, _vp],
+                           _i, _f, _vp],
         # gate_up, its dtype, ld, act, its dtype, n, inter, limit, alpha, stream
         "gb_glu_clamped": [_vp, _i, _i, _vp, _i, _i, _i, _f, _f, _vp],
         # x, y, alpha, bias, n, d, stream
@@ -86,8 +87,8 @@ _SIGS = {
         "gb_gate_heads": [_vp, _i, _i, _vp, _i, _i, _vp, _i, _i, _i, _i, _vp],
         # z, ldz, coef, eps, out, ldo, dtype, n, d, stream
         "gb_poly_norm": [_vp, _i, _vp, _f, _vp, _i, _i, _i, _i, _vp],
-        # x, y, slices, slice stride, g, eps, rounded, dtype, n, d, conv w, taps, state, tok_seq, pos0, state slots, stream
-        "gb_norm_add": [_vp, _vp, _i, C.c_longlong, _vp, _f, _vp, _i, _i, _i, _vp, _i, _vp, _vp, _vp, _vp, _vp],
+        # x, y, slices, slice stride, g, g a column (0/1), bias, eps, rounded, dtype, n, d, conv w, taps, state, tok_seq, pos0, state slots, stream
+        "gb_norm_add": [_vp, _vp, _i, C.c_longlong, _vp, _i, _vp, _f, _vp, _i, _i, _i, _vp, _i, _vp, _vp, _vp, _vp, _vp],
     },
     "tanhmix": {
         # x, ldx, rows, alpha, w, b, out, its dtype, ldo, n, d, stream
@@ -95,9 +96,9 @@ _SIGS = {
         # x, y, slices, slice stride, alpha, w, b, next alpha, w, b, h, its dtype, n, d, stream
         "gb_tanh_norm_add": [_vp, _vp, _i, C.c_longlong, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _vp],
         # proj, dtype, ld, bias, wconv, sums, state, tok_seq, q_start, pos0, state slots, flags and taps, wq, wk, eps, cos, sin,
-        # rot, mag, out, ldo, hd, slots, k, v, page, n, H, G, dk, dv, stream
+        # rot, mag, out, ldo, hd, slots, k, v, page, n, H, G, dk, dv, factor of the values, stream
         "gb_qk_heads": [_vp, _i, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i, _vp, _vp, _f, _vp, _vp, _i, _f, _vp, _i,
-                        _i, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _vp],
+                        _i, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _f, _vp],
         # proj, dtype, ld, bias, state, q_start, q_len, state slots, requests, channels, taps, stream
         "gb_qk_conv_state": [_vp, _i, _i, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _vp],
         # att, lda, hd, gate, ldg, one gate a head, dtype, out, ldo, n, H, dv, stream
@@ -134,6 +135,24 @@ _SIGS = {
         # kv, dtype, ld, k pages, v pages, heads, head columns, page size, total, stream
         "gb_latent_expand": [_vp, _i, _i, _vp, _vp, _i, _i, _i, _i, _vp],
     },
+    "delta": {
+        # proj, dtype, ld, column of q k v, of beta, of the decay, conv w, rate, dt, z, ldz, tok_seq, q_start, q_len, pos0, state
+        # slots, state, floats a slot, where the ring lies, first row, rows, first request, requests, H, G, dk, 16 dv + taps,
+        # q32, k32, v, beta and log decays, stream
+        "gb_delta_prep": [_vp, _i, _i, _i, _i, _i, _vp, _vp, _vp, _vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, C.c_longlong,
+                          C.c_longlong, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _vp, _vp, _vp, _vp],
+        # q32, k32, v, dtype, beta and log decays, a decay a channel (0/1), out, tok_seq, q_start, q_len, pos0, state slots, state,
+        # floats a slot, where the ring lies, first row, rows, first request, requests, longest, H, G, dk, dv, workspace, its
+        # floats, stream
+        "gb_delta_rule": [_vp, _vp, _vp, _i, _vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp, C.c_longlong, C.c_longlong, _i, _i, _i,
+                          _i, _i, _i, _i, _i, _i, _vp, C.c_longlong, _vp],
+        # o, gate, ldg, gate float32 (0/1), sigmoid (0/1), norm w, eps, out, dtype, ldo, first row, rows, H, dv, stream
+        "gb_delta_out": [_vp, _vp, _i, _i, _i, _vp, _f, _vp, _i, _i, _i, _i, _i, _i, _vp],
+        # proj, dtype, ld, column of q k v, of beta, of the decay, conv w, rate, dt, z, ldz, q_start, pos0, state slots, state, floats
+        # a slot, where the ring lies, rows, H, G, dk, 16 dv + taps, gate, ldg, gate float32 | 2 sigmoid, norm w, eps, out, ldo, stream
+        "gb_delta_step": [_vp, _i, _i, _i, _i, _i, _vp, _vp, _vp, _vp, _i, _vp, _vp, _vp, _vp, C.c_longlong, C.c_longlong, _i,
+                          _i, _i, _i, _i, _vp, _i, _i, _vp, _f, _vp, _i, _vp],
+    },
     "moe": {
         # z, ldz, n, experts, correction, top, scale, shared, combine, ids, weights, stream
         "gb_moe_route": [_vp, _i, _i, _i, _vp, _i, _f, _i, _vp, _vp, _vp, _vp],
@@ -142,15 +161,15 @@ _SIGS = {
         "gb_moe_route_by": [_vp, _i, _i, _i, _vp, _i, _f, _i, _i, _i, _i, _i, _vp, _vp, _vp, _vp],
         # z, its dtype, ld, combine, its columns, act, its dtype, lda, n, inter, experts, ff, stream
         "gb_moe_relu2_units": [_vp, _i, _i, _vp, _i, _vp, _i, _i, _i, _i, _i, _i, _vp],
-        # gate_up, its dtype, ld, combine, its columns, act, its dtype, n, inter, experts, ff, limit, alpha, plus, stream
-        "gb_moe_gated_units": [_vp, _i, _i, _vp, _i, _vp, _i, _i, _i, _i, _i, _f, _f, _f, _vp],
-        # ids, n, top, experts, rows a tile, tiles, counts, rows, pos, map, stream
-        "gb_moe_sort": [_vp, _i, _i, _i, _i, _i, _vp, _vp, _vp, _vp, _vp],
+        # gate_up, its dtype, ld, combine, its columns, act, its dtype, n, inter, experts, ff, limit, alpha, plus, weights on the way in (0/1), stream
+        "gb_moe_gated_units": [_vp, _i, _i, _vp, _i, _vp, _i, _i, _i, _i, _i, _f, _f, _f, _i, _vp],
+        # ids, n, top, experts, rows a tile, tiles, counts, rows, pos, map, weights, rows' weights, stream
+        "gb_moe_sort": [_vp, _i, _i, _i, _i, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp],
         # y, ldy, pos, weights, top, y_shared, its stride, gates, their stride, out, ldo, accumulate, n, d, rows of y, slices
         # of y, their distance, stream
         "gb_moe_combine": [_vp, _i, _vp, _vp, _i, _vp, _i, _vp, _i, _vp, _i, _i, _i, _i, _i, _i, C.c_longlong, _vp],
-        # h, dtype, ldh, w, ldw, n, d, experts, bias, top, scale, combine, ids, weights, stream
-        "gb_moe_router": [_vp, _i, _i, _vp, _i, _i, _i, _i, _vp, _i, _f, _vp, _vp, _vp, _vp],
+        # h, dtype, ldh, w, ldw, n, d, experts, bias, top, scale, sigmoid (0/1), combine, ids, weights, stream
+        "gb_moe_router": [_vp, _i, _i, _vp, _i, _i, _i, _i, _vp, _i, _f, _i, _vp, _vp, _vp, _vp],
     },
     "streams": {
         # X, stream stride, streams, w_in, gamma, gamma dtype, rows, out, out dtype, sum, m, d, eps, mix, w_out, y, stream
@@ -186,8 +205,8 @@ _SIGS = {
         "gb_gemm_bf16": [_vp, _i, _vp, _i, _vp, _i, _i, _i, _i, _i, _i, _vp, _i, _f, _vp, _i, _vp, _i, _vp, _vp, _i, _vp,
                          C.c_longlong, _vp],
         # a, lda, rows, w, ldw, distance between groups, up_off, c, ldc, c_dtype, map, tiles, rows a tile, N, K, epilogue,
-        # limit, alpha, plus, slices of k, rows of c a slice, stream
-        "gb_gemm_bf16_grouped": [_vp, _i, _vp, _vp, _i, C.c_longlong, _i, _vp, _i, _i, _vp, _i, _i, _i, _i, _i, _f, _f, _f, _i, _i, _vp],
+        # limit, alpha, plus, slices of k, rows of c a slice, factors of a's rows, stream
+        "gb_gemm_bf16_grouped": [_vp, _i, _vp, _vp, _i, C.c_longlong, _i, _vp, _i, _i, _vp, _i, _i, _i, _i, _i, _f, _f, _f, _i, _i, _vp, _vp],
         # a, lda, w, ldw, c, ldc, M, N, K, limit, alpha, plus, stream
         "gb_gemm_bf16_glu": [_vp, _i, _vp, _i, _vp, _i, _i, _i, _i, _f, _f, _f, _vp],
         "gb_gemm_bf16_split_floats": [_i, _i, _i],
@@ -205,9 +224,9 @@ _SIGS = {
         # q, q_stride, out, out_stride, dtype, positions, tok_seq, tables, table_stride, k, v, n, nh, nkv, hd, page,
         # scale, window, workspace, workspace floats, max_context, stream
         # scale, window, kept first keys, workspace, workspace floats, max_context, grouped, stream
-        # scale, window, kept first keys, run of positions, cap, sinks, workspace, workspace floats, max_context, grouped, stream
+        # scale, window, kept first keys, run of positions, cap, sinks, slopes, workspace, workspace floats, max_context, grouped, stream
         "gb_attention_plain": [_vp, _i, _vp, _i, _i, _vp, _vp, _vp, _i, _vp, _vp, _i, _i, _i, _i, _i, _f, _i, _i, _i, _f, _vp,
-                               _vp, C.c_longlong, _i, _i, _vp],
+                               _vp, _vp, C.c_longlong, _i, _i, _vp],
         "gb_attention_plain_split_floats": [_i, _i, _i, _i, _i, _i],
     },
     "attention_bf16": {
@@ -221,14 +240,14 @@ _SIGS = {
                                       _f, _i, _i, _i, _vp, C.c_longlong, _vp],
         "gb_attention_prefill_parts": [_i, _i, _i, _i, _i],
         # q, q_stride, out, out_stride, out32, ws_acc, ws_ml, positions, tables, table_stride, k, v, n_decode, nh, nkv, hd,
-        # page, scale, window, kept first keys, run of positions, cap, sinks, chunk, max_context, stream
+        # page, scale, window, kept first keys, run of positions, cap, sinks, slopes, chunk, max_context, stream
         "gb_attention_decode_bf16_by": [_vp, _i, _vp, _i, _i, _vp, _vp, _vp, _vp, _i, _vp, _vp, _i, _i, _i, _i, _i, _f, _i, _i,
-                                        _i, _f, _vp, _i, _i, _vp],
+                                        _i, _f, _vp, _vp, _i, _i, _vp],
         # q, q_stride, out, out_stride, out32, q_start, q_len, pos0, seq_base, n_seqs, max_q_len, max_context, tables,
-        # table_stride, k, v, nh, nkv, hd, page, scale, window, kept first keys, run of positions, cap, sinks, first_row,
+        # table_stride, k, v, nh, nkv, hd, page, scale, window, kept first keys, run of positions, cap, sinks, slopes, first_row,
         # n_rows, part_ws, part_floats, stream
         "gb_attention_prefill_bf16_by": [_vp, _i, _vp, _i, _i, _vp, _vp, _vp, _i, _i, _i, _i, _vp, _i, _vp, _vp, _i, _i, _i, _i,
-                                         _f, _i, _i, _i, _f, _vp, _i, _i, _vp, C.c_longlong, _vp],
+                                         _f, _i, _i, _i, _f, _vp, _vp, _i, _i, _vp, C.c_longlong, _vp],
         # the same two with the number of kept first keys after the window
         "gb_attention_decode_bf16_keep": [_vp, _i, _vp, _i, _vp, _vp, _vp, _vp, _i, _vp, _vp, _i, _i, _i, _i, _i, _f, _i, _i,
                                           _i, _i, _vp],
@@ -653,6 +672,15 @@ def scale_rows(x: torch.Tensor, s: float) -> None:
         raise KernelError("scale_rows: x must be contiguous float32")
     lib = _lib("elementwise")
     _launch(lib, lib.gb_scale_rows, _p(x), float(s), x.numel(), _stream())
+
+
+def cap_rows(x: torch.Tensor, cap: float, scale: float = 1.0) -> None:
+    """x = cap * tanh(scale * x / cap), float32."""
+    _dev(x)
+    if x.dtype != torch.float32 or not x.is_contiguous() or not cap > 0:
+        raise KernelError("cap_rows: x must be contiguous float32, the cap positive")
+    lib = _lib("elementwise")
+    _launch(lib, lib.gb_cap_rows, _p(x), float(scale), float(cap), x.numel(), _stream())
 
 
 # ------------------------------------------------------------------- residual streams
@@ -1134,11 +1162,12 @@ def norm_add_takes_rows(d: int) -> bool:
 
 
 def norm_add(x: torch.Tensor, y: torch.Tensor, g: torch.Tensor, eps: float, rounded: Optional[torch.Tensor] = None,
-             slices: int = 1, conv: Optional[tuple] = None, ctx=None) -> None:
-    """x += g * y / sqrt(mean(y^2) + eps) row by row: x float32 [n, d], ``g`` one float32 on the device.  y is float32
+             slices: int = 1, conv: Optional[tuple] = None, ctx=None, bias: Optional[torch.Tensor] = None) -> None:
+    """x += g * y / sqrt(mean(y^2) + eps) row by row: x float32 [n, d], ``g`` one float32 on the device, or one a column
+    ([d]); ``bias`` (float32 [d]) is added to y first.  y is float32
     [n, d], or with ``slices`` > 1 float32 [slices, n, d] whose sum over the slices it is (what a product that divides k
     leaves, ``gemm_slices``).  ``rounded`` ([n, d], any activations' type) receives the new x; with ``conv=(w, state)``, w [taps, d] as ``time_conv`` takes it
-    (a step in which every request brings one row; ``ctx`` the step) it receives new x + conv(new x) instead, the rows
+    (a step in which every request brings one row; ``ctx`` the step; w None: no convolution) it receives new x + conv(new x) instead, the rows
     the next mixer reads, and the requests' slots in ``state`` move on as in ``time_conv``."""
     _dev(x, y, g, rounded)
     n, d = x.shape
@@ -1149,11 +1178,17 @@ def norm_add(x: torch.Tensor, y: torch.Tensor, g: torch.Tensor, eps: float, roun
                               f"{NORM_ADD_ROWS_MAX}")
     else:
         _f32_rows(y, (n, d), "y")
-    _f32_rows(g, (1,), "g")
+    g_cols = g.numel() != 1 or d == 1
+    _f32_rows(g, (d,) if g_cols else (1,), "g")
+    if bias is not None:
+        _dev(bias)
+        _f32_rows(bias, (d,), "bias")
     if rounded is not None and (tuple(rounded.shape) != (n, d) or not rounded.is_contiguous()):
         raise KernelError("norm_add: rounded must be contiguous [n, d]")
     w = state = None
     taps = 0
+    if conv is not None and conv[0] is None:   # nothing but the new x
+        conv = None
     if conv is not None:
         w, state = conv
         _dev(w, state)
@@ -1167,7 +1202,7 @@ def norm_add(x: torch.Tensor, y: torch.Tensor, g: torch.Tensor, eps: float, roun
                          or tuple(state.shape[1:]) != (taps - 1, d)):
             raise KernelError("norm_add: state must be contiguous float32 [slots, taps - 1, d]")
     lib = _lib("headmix")
-    _launch(lib, lib.gb_norm_add, _p(x), _p(y), int(slices), n * d, _p(g), float(eps), _p(rounded),
+    _launch(lib, lib.gb_norm_add, _p(x), _p(y), int(slices), n * d, _p(g), 1 if g_cols else 0, _p(bias), float(eps), _p(rounded),
             dtype_code(rounded) if rounded is not None else F32, n, d, _p(w), taps, _p(state) if taps > 1 else None,
             _p(ctx.tok_seq) if conv is not None else None, _p(ctx.pos0) if conv is not None else None,
             _p(ctx.state_slots) if conv is not None else None, _stream())
@@ -1226,11 +1261,12 @@ def moe_relu2_units(z: torch.Tensor, combine: Optional[torch.Tensor], out: torch
 
 
 def moe_gated_units(gate_up: torch.Tensor, combine: torch.Tensor, out: torch.Tensor, n_experts: int, ff: int,
-                    unit: tuple = SILU_UNIT) -> None:
+                    unit: tuple = SILU_UNIT, weigh_in: bool = False) -> None:
     """out[t, j] = unit(gate, up) * combine[t, expert of column j], ``unit = (limit, alpha, plus)`` with g' = min(g, limit), u' =
     clamp(u, -limit, limit), g' sigmoid(alpha g') (u' + plus), by default silu(gate) * up: ``gate_up`` [n, 2 * I] holds the experts' gate columns, the
     experts' up columns, then the shared expert's gate columns and its up columns; columns e * ff .. of ``out`` are expert
-    e's, those from experts * ff on the shared expert's (weight in the last column of ``combine``)."""
+    e's, those from experts * ff on the shared expert's (weight in the last column of ``combine``).  ``weigh_in``: the weight
+    multiplies gate and up before the unit instead of the unit."""
     _dev(gate_up, combine, out)
     n, inter = out.shape
     if gate_up.shape != (n, 2 * inter) or gate_up.stride(1) != 1 or not out.is_contiguous():
@@ -1239,7 +1275,7 @@ def moe_gated_units(gate_up: torch.Tensor, combine: torch.Tensor, out: torch.Ten
         raise KernelError("moe_gated_units: combine must be contiguous float32 [n, experts (+ 1)]")
     lib = _lib("moe")
     _launch(lib, lib.gb_moe_gated_units, _p(gate_up), dtype_code(gate_up), gate_up.stride(0), _p(combine), combine.shape[1],
-            _p(out), dtype_code(out), n, inter, n_experts, ff, *map(float, unit), _stream())
+            _p(out), dtype_code(out), n, inter, n_experts, ff, *map(float, unit), 1 if weigh_in else 0, _stream())
 
 
 def moe_sort_tiles(entries: int, n_experts: int, tile_rows: int) -> int:
@@ -1248,13 +1284,17 @@ def moe_sort_tiles(entries: int, n_experts: int, tile_rows: int) -> int:
 
 
 def moe_sort(ids: torch.Tensor, n_experts: int, tile_rows: int, counts: torch.Tensor, rows: torch.Tensor, pos: torch.Tensor,
-             tile_map: torch.Tensor) -> None:
+             tile_map: torch.Tensor, weights: Optional[torch.Tensor] = None, row_weights: Optional[torch.Tensor] = None) -> None:
     """Orders the entries of ``ids`` (int32 [n, top]) by expert, entries of an expert in the order of the tokens:
     ``rows`` [n * top] receives the token behind each sorted row, ``pos`` [n, top] the sorted row of each entry, and
     ``tile_map`` [tiles, 3] cuts the sorted rows into tiles of at most ``tile_rows`` rows of one expert (expert, first row,
-    end of the expert's rows; expert -1 for the tiles left over).  ``counts`` [experts] is scratch."""
-    _dev(ids, counts, rows, pos, tile_map)
+    end of the expert's rows; expert -1 for the tiles left over).  ``counts`` [experts] is scratch.  ``row_weights`` (float32 [n * top]), if given,
+    receives each sorted row's entry of ``weights`` (float32 [n, top])."""
+    _dev(ids, counts, rows, pos, tile_map, weights, row_weights)
     n, top = ids.shape
+    if row_weights is not None:
+        _f32_rows(row_weights, (n * top,), "row_weights")
+        _f32_rows(weights, (n, top), "weights")
     _i32(ids, "ids", n * top)
     _i32(counts, "counts", n_experts)
     _i32(rows, "rows", n * top)
@@ -1262,15 +1302,16 @@ def moe_sort(ids: torch.Tensor, n_experts: int, tile_rows: int, counts: torch.Te
     tiles = tile_map.shape[0]
     _i32(tile_map, "tile_map", tiles * 3)
     lib = _lib("moe")
-    _launch(lib, lib.gb_moe_sort, _p(ids), n, top, n_experts, tile_rows, tiles, _p(counts), _p(rows), _p(pos), _p(tile_map), _stream())
+    _launch(lib, lib.gb_moe_sort, _p(ids), n, top, n_experts, tile_rows, tiles, _p(counts), _p(rows), _p(pos),
+            _p(tile_map), _p(weights) if row_weights is not None else None, _p(row_weights), _stream())
 
 
-def moe_combine(y: torch.Tensor, pos: torch.Tensor, weights: torch.Tensor, y_shared: Optional[torch.Tensor],
+def moe_combine(y: torch.Tensor, pos: torch.Tensor, weights: Optional[torch.Tensor], y_shared: Optional[torch.Tensor],
                 gates: Optional[torch.Tensor], out: torch.Tensor, accumulate: bool) -> None:
-    """out[t] (+)= sum over k of weights[t, k] * y[pos[t, k]] + gates[t] * y_shared[t], all float32; ``gates`` may be a
+    """out[t] (+)= sum over k of weights[t, k] (1 without ``weights``) * y[pos[t, k]] + gates[t] * y_shared[t], all float32; ``gates`` may be a
     column of a wider tensor; a ``y`` of [slices, rows, d] is the sum of its slices."""
     _dev(y, pos, weights, y_shared, gates, out)
-    n, top = weights.shape
+    n, top = pos.shape
     d = out.shape[1]
     slices, slice_stride = 1, 0
     if y.dim() == 3:
@@ -1281,7 +1322,8 @@ def moe_combine(y: torch.Tensor, pos: torch.Tensor, weights: torch.Tensor, y_sha
             raise KernelError(f"moe_combine: {what} must be float32 [rows, {d}] with dense rows")
     if out.shape[0] != n or y.shape[0] < n * top or (y_shared is not None and (y_shared.shape[0] != n or gates is None or gates.shape[0] != n)):
         raise KernelError("moe_combine: y holds a row for every entry, out, y_shared and gates a row for every token")
-    _f32_rows(weights, (n, top), "weights")
+    if weights is not None:
+        _f32_rows(weights, (n, top), "weights")
     _i32(pos, "pos", n * top)
     lib = _lib("moe")
     _launch(lib, lib.gb_moe_combine, _p(y), y.stride(0), _p(pos), _p(weights), top, _p(y_shared),
@@ -1293,8 +1335,9 @@ MOE_ROUTER_MAX_EXPERTS = 64   # moe.hip: a lane an expert
 
 
 def moe_router(h: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], top: int, scale: float, combine: torch.Tensor,
-               ids: torch.Tensor, weights: torch.Tensor) -> None:
-    """Logits z = h . w^T + bias and the route by them in one kernel (``moe_route`` with ``softmax="chosen"``): ``h`` [n, d] and
+               ids: torch.Tensor, weights: torch.Tensor, sigmoid: bool = False) -> None:
+    """Logits z = h . w^T + bias and the route by them in one kernel (``moe_route`` with ``softmax="chosen"``; ``sigmoid``: the
+    weights are the chosen logits' sigmoids, times scale): ``h`` [n, d] and
     ``w`` [experts, d] of one type, up to ``MOE_ROUTER_MAX_EXPERTS`` experts."""
     _dev(h, w, bias, combine, ids, weights)
     n, d = h.shape
@@ -1308,7 +1351,7 @@ def moe_router(h: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], t
         _f32_rows(bias, (E,), "bias")
     lib = _lib("moe")
     _launch(lib, lib.gb_moe_router, _p(h), dtype_code(h), _rows(h, "h"), _p(w), _rows(w, "w"), n, d, E, _p(bias), int(top), float(scale),
-            _p(combine), _p(ids), _p(weights), _stream())
+            1 if sigmoid else 0, _p(combine), _p(ids), _p(weights), _stream())
 
 
 @functools.lru_cache(maxsize=4096)
@@ -1328,15 +1371,19 @@ def gemm_grouped_takes(a: torch.Tensor, w: torch.Tensor, group_stride: int) -> b
 
 def gemm_grouped(a: torch.Tensor, rows: Optional[torch.Tensor], w: torch.Tensor, group_stride: int, n_out: int,
                  tile_map: torch.Tensor, tile_rows: int, out: torch.Tensor, silu_mul: bool = False, up_offset: int = 0,
-                 unit: tuple = SILU_UNIT) -> None:
+                 unit: tuple = SILU_UNIT, in_scale: Optional[torch.Tensor] = None) -> None:
     """Products of groups of rows with a matrix of their own each.  Sorted row r of the product reads row ``rows[r]`` of
     ``a`` (row r without ``rows``); ``tile_map`` (as ``moe_sort`` writes it) names each row tile's group and rows; group g
     uses the ``n_out`` rows of ``w`` that begin ``g * group_stride`` elements into it.  ``silu_mul``: the group's rows
     are n_out / 2 gate rows, with the up row of each ``up_offset`` rows behind it, and out = silu(gate) * up, or another
     ``unit = (limit, alpha, plus)`` as ``moe_gated_units`` takes it.  Row tiles are of 64, 128 or 256 rows; with 256 (the inner
     size a multiple of 32) a float32 ``out`` may be [slices, rows, n_out]: k is divided, and out's sum over the slices is the
-    result."""
-    _dev(a, rows, w, tile_map, out)
+    result.  ``in_scale`` (float32, one a sorted row; with ``silu_mul``): the rows of ``a`` count times these."""
+    _dev(a, rows, w, tile_map, out, in_scale)
+    if in_scale is not None:
+        if not silu_mul:
+            raise KernelError("gemm_grouped: factors of the rows go with silu_mul")
+        _f32_rows(in_scale, (out.shape[0],), "in_scale")
     K = a.shape[1]
     cols = n_out // 2 if silu_mul else n_out
     if not gemm_grouped_takes(a, w, group_stride) or a.stride(1) != 1 or w.stride(1) != 1 or w.shape[1] < K:
@@ -1353,13 +1400,13 @@ def gemm_grouped(a: torch.Tensor, rows: Optional[torch.Tensor], w: torch.Tensor,
     lib = _lib("gemm_bf16")
     _launch(lib, lib.gb_gemm_bf16_grouped, _p(a), a.stride(0), _p(rows), _p(w), w.stride(0), int(group_stride), int(up_offset),
             _p(out), out.stride(0), dtype_code(out), _p(tile_map), tiles, tile_rows, n_out, K, 2 if silu_mul else 0,
-            *map(float, unit), slices, out.shape[0], _stream())
+            *map(float, unit), slices, out.shape[0], _p(in_scale), _stream())
 
 
 # ------------------------------------------------------------------- small residual operations
 def embed_pairs(table: torch.Tensor, pairs: torch.Tensor, ctx, out: torch.Tensor, buckets: int, mul_prev: int, mul_cur: int,
-                prev: torch.Tensor) -> None:
-    """out[i] = table[id_i] + pairs[(id_(i-1) * mul_prev + id_i * mul_cur) mod buckets], row ``buckets`` of ``pairs`` for
+                prev: torch.Tensor, scale: float = 1.0) -> None:
+    """out[i] = scale * table[id_i] + pairs[(id_(i-1) * mul_prev + id_i * mul_cur) mod buckets], row ``buckets`` of ``pairs`` for
     a request's first token; float32 [n, d] or [copies, n, d].  ``prev`` int32 [slots, 1]: the last token of each
     request's earlier steps, read for the first row of a request that goes on and left for the next step."""
     _dev(table, pairs, out, prev)
@@ -1373,7 +1420,7 @@ def embed_pairs(table: torch.Tensor, pairs: torch.Tensor, ctx, out: torch.Tensor
     lib = _lib("elementwise")
     _launch(lib, lib.gb_embed_pairs, _p(table), _p(pairs), dtype_code(table), _p(ctx.token_ids), _p(out), n, d, table.shape[0],
             int(buckets), int(mul_prev), int(mul_cur), _p(ctx.tok_seq), _p(ctx.q_start), _p(ctx.q_len), _p(ctx.pos0),
-            _p(ctx.state_slots), _p(prev), int(copies), _stream())
+            _p(ctx.state_slots), _p(prev), int(copies), float(scale), _stream())
 
 
 def glu_clamped(gate_up: torch.Tensor, out: torch.Tensor, limit: float, alpha: float) -> None:
@@ -1667,11 +1714,12 @@ def attention_plain(q: torch.Tensor, out: torch.Tensor, positions: torch.Tensor,
                     tables: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, n_heads: int,
                     scale: float, window: int = 0, workspace: Optional[torch.Tensor] = None, max_context: int = 0,
                     grouped: bool = False, keep_first: int = 0, chunk: int = 0, softcap: float = 0.0,
-                    sinks: Optional[torch.Tensor] = None) -> None:
+                    sinks: Optional[torch.Tensor] = None, slopes: Optional[torch.Tensor] = None) -> None:
     """Paged attention, one block per (token, head); q may be a view into the stacked qkv rows.
     ``chunk`` > 0 (no window then): positions are cut into runs of ``chunk`` from 0 on and a token reads the keys of its
     own run up to itself; ``softcap`` > 0: scores pass softcap * tanh(score / softcap); ``sinks`` float32 [heads]:
-    exp(sinks[h]) joins the softmax's denominator of head h and has no value.
+    exp(sinks[h]) joins the softmax's denominator of head h and has no value; ``slopes`` float32 [heads]: slopes[h] times the
+    key's distance is taken off the score.
     ``window`` > 0: a token at position p reads keys p - window + 1 .. p, and with ``keep_first`` also keys
     0 .. keep_first - 1 wherever the window has moved past them.
     ``workspace`` (float32, ``attention_plain_split_floats`` elements) with ``max_context`` (at least the most keys a
@@ -1698,7 +1746,7 @@ def attention_plain(q: torch.Tensor, out: torch.Tensor, positions: torch.Tensor,
     _launch(lib, lib.gb_attention_plain, _p(q), _rows(q, "q"), _p(out), _rows(out, "out"), dtype_code(q), _p(positions),
                                        _p(tok_seq), _p(tables), tables.stride(0), _p(k_pages), _p(v_pages), n,
                                        n_heads, nkv, hd, page_size, float(scale), int(window), int(keep_first),
-                                       int(chunk), float(softcap), _p(_sinks(sinks, n_heads)),
+                                       int(chunk), float(softcap), _p(_sinks(sinks, n_heads)), _p(_sinks(slopes, n_heads)),
                                        _p(workspace), workspace.numel() if workspace is not None else 0, int(max_context),
                                        1 if grouped else 0, _stream())
 
@@ -1706,7 +1754,7 @@ def attention_plain(q: torch.Tensor, out: torch.Tensor, positions: torch.Tensor,
 def _sinks(sinks: Optional[torch.Tensor], n_heads: int) -> Optional[torch.Tensor]:
     if sinks is not None and (not sinks.is_cuda or sinks.dtype != torch.float32 or not sinks.is_contiguous()
                               or sinks.numel() != n_heads):
-        raise KernelError(f"attention: sinks must be contiguous float32 [{n_heads}] on the GPU")
+        raise KernelError(f"attention: sinks and slopes must be contiguous float32 [{n_heads}] on the GPU")
     return sinks
 
 
@@ -1736,7 +1784,8 @@ def decode_chunk(n_decode: int, n_kv_heads: int, max_context: int) -> int:
 
 
 def attention_decode(q: torch.Tensor, out: torch.Tensor, ctx, cache, n_heads: int, scale: float, window: int,
-                     keep_first: int = 0, chunk: int = 0, softcap: float = 0.0, sinks: Optional[torch.Tensor] = None) -> None:
+                     keep_first: int = 0, chunk: int = 0, softcap: float = 0.0, sinks: Optional[torch.Tensor] = None,
+                     slopes: Optional[torch.Tensor] = None) -> None:
     """Rows 0..n_decode-1 of the step (requests with a single token), split over their context."""
     n_dec = ctx.host["n_decode"]
     k_pages, v_pages = cache.k_pages, cache.v_pages
@@ -1752,11 +1801,11 @@ def attention_decode(q: torch.Tensor, out: torch.Tensor, ctx, cache, n_heads: in
     ws_acc = ctx.buffer("attn_ws_acc", (n_dec * n_heads * splits * hd,), torch.float32)
     ws_ml = ctx.buffer("attn_ws_ml", (n_dec * n_heads * splits * 2,), torch.float32)
     lib = _lib("attention_bf16")
-    if mask_chunk or softcap or sinks is not None:
+    if mask_chunk or softcap or sinks is not None or slopes is not None:
         _launch(lib, lib.gb_attention_decode_bf16_by, _p(q), _rows(q, "q"), _p(out), _rows(out, "out"),
                 1 if out.dtype == torch.float32 else 0, _p(ws_acc), _p(ws_ml), _p(ctx.positions), _p(tables), tables.stride(0),
                 _p(k_pages), _p(v_pages), n_dec, n_heads, nkv, hd, page, float(scale), int(window), int(keep_first), mask_chunk,
-                float(softcap), _p(_sinks(sinks, n_heads)), chunk, max_context, _stream())
+                float(softcap), _p(_sinks(sinks, n_heads)), _p(_sinks(slopes, n_heads)), chunk, max_context, _stream())
         return
     if keep_first or out.dtype == torch.float32:
         _launch(lib, lib.gb_attention_decode_bf16_out32 if out.dtype == torch.float32 else lib.gb_attention_decode_bf16_keep, _p(q), _rows(q, "q"), _p(out), _rows(out, "out"), _p(ws_acc), _p(ws_ml),
@@ -1776,7 +1825,7 @@ def _prefill_parts(max_q: int, max_ctx: int, n_heads: int, n_seqs: int, hd: int)
 
 def attention_prefill(q: torch.Tensor, out: torch.Tensor, ctx, cache, n_heads: int, scale: float, window: int,
                       keep_first: int = 0, chunk: int = 0, softcap: float = 0.0, sinks: Optional[torch.Tensor] = None,
-                      tables: Optional[torch.Tensor] = None) -> None:
+                      tables: Optional[torch.Tensor] = None, slopes: Optional[torch.Tensor] = None) -> None:
     """The requests of the step that bring more than one token (they follow the single-token ones).  ``tables``: block
     tables other than the cache's own (int32 [requests, pages]), for keys and values in pages of the step's making."""
     n_dec, S = ctx.host["n_decode"], ctx.num_seqs
@@ -1796,11 +1845,11 @@ def attention_prefill(q: torch.Tensor, out: torch.Tensor, ctx, cache, n_heads: i
     first_row, n_rows = n_dec, q.shape[0] - n_dec
     parts = _prefill_parts(max_q, max_ctx, n_heads, S - n_dec, hd)
     ws = ctx.buffer("attn_parts", (parts * n_rows * n_heads * (hd + 2),), torch.float32) if parts > 1 else None
-    if chunk or softcap or sinks is not None:
+    if chunk or softcap or sinks is not None or slopes is not None:
         _launch(lib, lib.gb_attention_prefill_bf16_by, _p(q), _rows(q, "q"), _p(out), _rows(out, "out"),
                 1 if out.dtype == torch.float32 else 0, _p(ctx.q_start), _p(ctx.q_len), _p(ctx.pos0), n_dec, S - n_dec, max_q,
                 max_ctx, _p(tables), tables.stride(0), _p(k_pages), _p(v_pages), n_heads, nkv, hd, page, float(scale),
-                int(window), int(keep_first), int(chunk), float(softcap), _p(_sinks(sinks, n_heads)), first_row, n_rows, _p(ws),
+                int(window), int(keep_first), int(chunk), float(softcap), _p(_sinks(sinks, n_heads)), _p(_sinks(slopes, n_heads)), first_row, n_rows, _p(ws),
                 ws.numel() if ws is not None else 0, _stream())
         return
     if keep_first or out.dtype == torch.float32:
@@ -1911,7 +1960,7 @@ def qk_heads(proj: torch.Tensor, ctx, out: torch.Tensor, head_cols: int, n_heads
              bias: Optional[torch.Tensor] = None, wconv: Optional[torch.Tensor] = None, state: Optional[torch.Tensor] = None,
              cos: Optional[torch.Tensor] = None, sin: Optional[torch.Tensor] = None, rot: int = 0, magnitude: float = 1.0,
              neighbours: bool = True, tied: bool = False, slots: Optional[torch.Tensor] = None,
-             k_pages: Optional[torch.Tensor] = None, v_pages: Optional[torch.Tensor] = None) -> None:
+             k_pages: Optional[torch.Tensor] = None, v_pages: Optional[torch.Tensor] = None, value_scale: float = 1.0) -> None:
     """The query, key and value heads of every row of the step as attention reads them, ``out`` [n, (heads + 2 kv heads) *
     head_cols], from the stacked projections ``proj`` ([n, query channels | key channels | value channels | ...]; with
     ``tied`` there are no value channels: the key channels, biased and convolved, are the values):
@@ -1920,7 +1969,7 @@ def qk_heads(proj: torch.Tensor, ctx, out: torch.Tensor, head_cols: int, n_heads
     in a step of single tokens, else by ``qk_conv_state``); an RMS norm over all query (key) channels at once with a weight a
     channel (``joint``) or over each head with ``dim`` weights that the heads share; the first ``rot`` channels of each
     head turned by the rows' angles (``cos``, ``sin`` float32 [n, rot / 2], times ``magnitude``), channel 2i with 2i + 1
-    (``neighbours``) or i with i + rot / 2.  With ``slots`` keys and values also go to their pages."""
+    (``neighbours``) or i with i + rot / 2; value heads times ``value_scale``.  With ``slots`` keys and values also go to their pages."""
     _dev(proj, out, bias, wconv, state, cos, sin, slots, k_pages, v_pages, norm_q, norm_k)
     n = proj.shape[0]
     channels = (n_heads + n_kv_heads) * dim
@@ -1954,7 +2003,7 @@ def qk_heads(proj: torch.Tensor, ctx, out: torch.Tensor, head_cols: int, n_heads
             single | (2 if joint else 0) | (4 if neighbours else 0) | (8 if tied else 0) | (int(taps) << 8), _p(norm_q), _p(norm_k),
             float(eps),
             _p(cos), _p(sin), int(rot), float(magnitude), _p(out), _rows(out, "out"), int(head_cols), _p(slots), _p(k_pages),
-            _p(v_pages), int(page), n, n_heads, n_kv_heads, dim, vdim, _stream())
+            _p(v_pages), int(page), n, n_heads, n_kv_heads, dim, vdim, float(value_scale), _stream())
     if taps > 1 and not single:
         _launch(lib, lib.gb_qk_conv_state, _p(proj), dtype_code(proj), _rows(proj, "proj"), _p(bias), _p(state), _p(ctx.q_start),
                 _p(ctx.q_len), _p(ctx.state_slots), ctx.num_seqs, channels, int(taps), _stream())
@@ -2237,3 +2286,98 @@ def latent_expand(kv: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor
     lib = _lib("latent")
     _launch(lib, lib.gb_latent_expand, _p(kv), dtype_code(kv), _act_rows(kv, kv.dtype, 2 * H * hc, "kv"), _p(k_pages), _p(v_pages), H,
             hc, P, total, _stream())
+
+
+# ------------------------------------------------------------------- gated delta rule
+DELTA_MAX_KEY_DIM = 256
+DELTA_MAX_VALUE_DIM = 4096
+DELTA_CHUNK_FROM = 32    # portions from here on go in chunks of 64 tokens
+
+
+def delta_slot(n_heads: int, n_qk_heads: int, key_dim: int, value_dim: int, taps: int) -> tuple:
+    """(floats a slot, where the convolution's ring begins): the state [heads, value_dim, key_dim] first, then ``taps`` rows of
+    the projections' channels (none for one tap), each begun at a 16-byte word."""
+    ring_at = -(-n_heads * value_dim * key_dim // 4) * 4
+    ring = taps * (2 * n_qk_heads * key_dim + n_heads * value_dim) if taps > 1 else 0
+    return ring_at + -(-ring // 4) * 4, ring_at
+
+
+def _delta_sizes(state, what: str, H: int, G: int, dk: int, dv: int, taps: int):
+    floats, ring_at = delta_slot(H, G, dk, dv, taps)
+    if state.dtype != torch.float32 or not state.is_contiguous() or state.dim() != 2 or state.shape[1] != floats:
+        raise KernelError(f"{what}: state must be contiguous float32 [slots, {floats}]")
+    return floats, ring_at
+
+
+def _delta_inputs(proj, at: int, b_at: int, a_at: int, wconv, rate, dt, z, H: int, G: int, dk: int, dv: int, what: str):
+    _dev(proj, wconv, rate, dt, z)
+    channels = 2 * G * dk + H * dv
+    _f32_rows(wconv, (wconv.shape[0], channels), f"{what}: wconv")
+    _f32_rows(rate, (H,), f"{what}: rate")
+    _f32_rows(dt, (H * dk if z is not None else H,), f"{what}: dt")
+    if z is not None and (z.dtype != torch.float32 or z.dim() != 2 or z.stride(1) != 1 or z.shape[0] != proj.shape[0] or z.shape[1] < H * dk):
+        raise KernelError(f"{what}: the decay's logits must be float32 [n, heads * key_dim] with dense rows")
+    if at + channels > proj.shape[1] or b_at + H > proj.shape[1] or (z is None and a_at + H > proj.shape[1]):
+        raise KernelError(f"{what}: the projections' rows are too short")
+
+
+def delta_rule(proj: torch.Tensor, at: int, b_at: int, a_at: int, wconv: torch.Tensor, rate: torch.Tensor, dt: torch.Tensor,
+               z: Optional[torch.Tensor], state: torch.Tensor, ctx, n_heads: int, n_qk_heads: int, key_dim: int, value_dim: int,
+               gate: torch.Tensor, sigmoid_gate: bool, norm_weight: torch.Tensor, eps: float, out: torch.Tensor) -> None:
+    """The gated delta rule over the rows of a step, from the projections to the gated heads.  ``proj`` [n, ..] holds, from column
+    ``at`` on, the query channels (``n_qk_heads`` * key_dim), the key channels and the value channels (n_heads * value_dim), at
+    ``b_at`` one logit of beta a head and, without ``z``, at ``a_at`` one of the decay a head; ``z`` float32 [n, heads * key_dim]: the
+    logits of a decay a head and key channel.  q, k and v pass a causal convolution over time (``wconv`` float32 [taps, channels], a
+    row a tap, the last the token's own) and silu; q and k then have length one and q counts times key_dim^(-1/2); log decays are
+    -``rate`` softplus(logit + ``dt``).  Per head S <- decay S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q; then
+    out = ``norm_weight`` * o / sqrt(mean(o^2) + eps) * act(``gate``), act = silu or sigmoid; ``gate`` [n, heads * value_dim] in
+    float32 or the activations' type; ``out`` may be columns of wider rows.  ``state`` float32 [slots, floats] (``delta_slot``)."""
+    what = "delta_rule"
+    H, G, dk, dv, taps = n_heads, n_qk_heads, key_dim, value_dim, wconv.shape[0]
+    _delta_inputs(proj, at, b_at, a_at, wconv, rate, dt, z, H, G, dk, dv, what)
+    _dev(state, gate, norm_weight, out)
+    n = proj.shape[0]
+    floats, ring_at = _delta_sizes(state, what, H, G, dk, dv, taps)
+    _f32_rows(norm_weight, (dv,), f"{what}: norm_weight")
+    if gate.shape != (n, H * dv) or out.shape != (n, H * dv) or out.dtype != proj.dtype or gate.dtype not in (torch.float32, out.dtype):
+        raise KernelError(f"{what}: gate and out must be [n, heads * value_dim], out of the projections' type")
+    if H % G or dk > DELTA_MAX_KEY_DIM or dv > DELTA_MAX_VALUE_DIM or not 1 <= taps <= CONV_MAX_TAPS:
+        raise KernelError(f"{what}: heads, sizes or taps that the kernels do not take")
+    lib = _lib("delta")
+    code = dtype_code(proj)
+    g32 = 1 if gate.dtype == torch.float32 else 0
+    alone, S = int(ctx.host["n_decode"]), ctx.num_seqs
+    ldz = z.stride(0) if z is not None else 0
+    if alone:   # requests with one row come first, row t being request t's
+        _launch(lib, lib.gb_delta_step, _p(proj), code, _rows(proj, "proj"), int(at), int(b_at), int(a_at), _p(wconv), _p(rate), _p(dt),
+                _p(z), ldz, _p(ctx.q_start), _p(ctx.pos0), _p(ctx.state_slots), _p(state), floats, ring_at, alone, H, G, dk,
+                16 * dv + taps, _p(gate), _rows(gate, "gate"), g32 | (2 if sigmoid_gate else 0), _p(norm_weight), float(eps), _p(out),
+                _rows(out, "out"), _stream())
+    if alone >= S:
+        return
+    q32 = ctx.buffer("delta_q", (n, G * dk), torch.float32)
+    k32 = ctx.buffer("delta_k", (n, G * dk), torch.float32)
+    v = ctx.buffer("delta_v", (n, H * dv), proj.dtype)
+    beta_lg = ctx.buffer("delta_decay", (-(-n * H // 4) * 4 + n * H * (dk if z is not None else 1),), torch.float32)
+    o = ctx.buffer("delta_o", (n, H * dv), torch.float32)
+    longest, rows = int(ctx.host["max_q_len"]), n - alone
+    _launch(lib, lib.gb_delta_prep, _p(proj), code, _rows(proj, "proj"), int(at), int(b_at), int(a_at), _p(wconv), _p(rate), _p(dt), _p(z),
+            ldz, _p(ctx.tok_seq), _p(ctx.q_start), _p(ctx.q_len), _p(ctx.pos0), _p(ctx.state_slots), _p(state), floats, ring_at,
+            alone, rows, alone, S - alone, H, G, dk, 16 * dv + taps, _p(q32), _p(k32), _p(v), _p(beta_lg), _stream())
+    ws = None
+    if ctx.tuned and longest >= DELTA_CHUNK_FROM:
+        need = delta_chunk_floats(rows, S - alone, H, dk, dv)
+        ws = ctx.buffer("delta_chunks", (need,), torch.float32) if need else None
+    _launch(lib, lib.gb_delta_rule, _p(q32), _p(k32), _p(v), code, _p(beta_lg), 1 if z is not None else 0, _p(o), _p(ctx.tok_seq),
+            _p(ctx.q_start), _p(ctx.q_len), _p(ctx.pos0), _p(ctx.state_slots), _p(state), floats, ring_at, alone, rows, alone,
+            S - alone, longest, H, G, dk, dv, _p(ws), ws.numel() if ws is not None else 0, _stream())
+    _launch(lib, lib.gb_delta_out, _p(o), _p(gate), _rows(gate, "gate"), g32, 1 if sigmoid_gate else 0, _p(norm_weight), float(eps),
+            _p(out), code, _rows(out, "out"), alone, rows, H, dv, _stream())
+
+
+@functools.lru_cache(maxsize=4096)
+def delta_chunk_floats(rows: int, n_seqs: int, n_heads: int, key_dim: int, value_dim: int) -> int:
+    """Floats of workspace with which ``delta_rule`` takes long portions in chunks, 0 where these sizes go token by token."""
+    f = _lib("delta").gb_delta_chunk_floats
+    f.restype = C.c_longlong
+    return int(f(rows, n_seqs, n_heads, key_dim, value_dim))

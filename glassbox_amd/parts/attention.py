@@ -21,17 +21,18 @@ from .base import (FULL, RUNS, WINDOW, CacheSpec, LayerCache, Mixer, PositionEnc
 
 def paged_attention(ctx, q: torch.Tensor, out: torch.Tensor, cache: LayerCache, n_heads: int, scale: float,
                     window: int, keep_first: int = 0, chunk: int = 0, softcap: float = 0.0,
-                    sinks: Optional[torch.Tensor] = None) -> None:
+                    sinks: Optional[torch.Tensor] = None, slopes: Optional[torch.Tensor] = None) -> None:
     """Attention of every row of the step over its request's pages.  ``window`` > 0: a token reads the last so many
     keys up to its own, and with ``keep_first`` the request's first so many keys as well, wherever they lie.
     ``chunk`` > 0 (instead of a window): positions are cut into runs of so many, counted from the request's first, and a
     token reads the keys of its own run up to itself.  ``softcap`` > 0: scores pass softcap * tanh(score / softcap).
     ``sinks`` (float32 [heads]): exp(sinks[h]) joins the softmax's denominator of head h and has no value.
+    ``slopes`` (float32 [heads]): slopes[h] times the key's distance is taken off the score.
 
     float32 always takes the plain kernel.  bfloat16 takes the tuned kernels where they apply: requests with
     one row go to the split-context decode kernel, longer portions to the matrix-core prefill kernel; a step
     with ``ctx.tuned`` off takes the plain kernel throughout."""
-    if (ctx.dtype == torch.float32 or not ctx.tuned
+    if (ctx.dtype == torch.float32 or not ctx.tuned or (slopes is not None and (softcap > 0 or not scale > 0))
             or not ops.tuned_attention_supports(cache.k_pages, n_heads, window, keep_first)):
         longest = int(ctx.host["max_context"])
         _, _, n_pieces, page_size, piece = cache.k_pages.shape
@@ -44,7 +45,7 @@ def paged_attention(ctx, q: torch.Tensor, out: torch.Tensor, cache: LayerCache, 
             ws = ctx.buffer("attention_plain_parts", (floats,), torch.float32) if floats else None
             ops.attention_plain(q[a:b], out[a:b], ctx.positions[a:b], ctx.tok_seq[a:b], tables, cache.k_pages, cache.v_pages,
                                 n_heads, scale, window, workspace=ws, max_context=longest, grouped=grouped,
-                                keep_first=keep_first, chunk=chunk, softcap=softcap, sinks=sinks)
+                                keep_first=keep_first, chunk=chunk, softcap=softcap, sinks=sinks, slopes=slopes)
 
         # the rows of requests with one token come first; many rows of prompt portions go eight rows a workgroup
         n, n_decode = q.shape[0], ctx.host["n_decode"]
@@ -57,9 +58,9 @@ def paged_attention(ctx, q: torch.Tensor, out: torch.Tensor, cache: LayerCache, 
         return
     n_decode = ctx.host["n_decode"]
     if n_decode > 0:
-        ops.attention_decode(q, out, ctx, cache, n_heads, scale, window, keep_first, chunk, softcap, sinks)
+        ops.attention_decode(q, out, ctx, cache, n_heads, scale, window, keep_first, chunk, softcap, sinks, slopes)
     if n_decode < ctx.num_seqs:
-        ops.attention_prefill(q, out, ctx, cache, n_heads, scale, window, keep_first, chunk, softcap, sinks)
+        ops.attention_prefill(q, out, ctx, cache, n_heads, scale, window, keep_first, chunk, softcap, sinks, slopes=slopes)
 
 
 class PagedAttention(Mixer):
@@ -544,19 +545,23 @@ class GatedAttention(Mixer):
     * ``sink``: "zero": one is added to the softmax's denominator (a sink of score 0); "learned": exp(sink_h), one number a
       head (``sink``); None: a plain softmax;
     * ``gate``: "head": head h times sigmoid(W_g h)_h (``g`` [heads, width]); "channel": every channel of the heads times
-      its own sigmoid (``g`` [heads * vdim, width]); the gate reads the mixer's input;
-    * the output projection ``o`` on the gated heads.
+      its own sigmoid (``g`` [heads * vdim, width]); the gate reads the mixer's input; None: no gate;
+    * ``slope``: slope_h * (the key's distance) is taken off head h's scores (behind a cap), slope_h = 2^(-8 (h + 1) / heads);
+    * the output projection ``o`` on the (gated) heads, with ``out_bias`` plus ``o.b``;
+    * ``result_scale``: the result counts times this number (on the value heads, where nothing is rounded for it).
 
     One product makes queries, keys, values and gates; ``ops.qk_heads`` prepares the heads (and writes the cache in steps
     of few rows); the framework's paged attention kernels do the rest."""
     replayable = True
     taped = True
     accepts_store = True
+    hands_on_bias = True
 
     def __init__(self, width: int, n_heads: int, n_kv_heads: int, dim: int, vdim: int, scale: float, eps: float,
                  bias: bool = False, taps: int = 0, tied_values: bool = False, qk_norm: str = "head", rot_dims: int = 0,
                  rot_base: float = 10000.0, rot_pairs: str = "halves", rot_scaling=None, softcap: float = 0.0, chunk: int = 0,
-                 sink: Optional[str] = None, gate: str = "channel"):
+                 sink: Optional[str] = None, gate: Optional[str] = "channel", slope: bool = False, out_bias: bool = False,
+                 result_scale: float = 1.0):
         from .rotary import Rotary
         if n_heads % n_kv_heads:
             raise ValueError(f"{n_heads} query heads are not a multiple of {n_kv_heads} key heads")
@@ -567,21 +572,24 @@ class GatedAttention(Mixer):
         if qk_norm == "joint" and taps:
             raise ValueError("one norm over all of q (and of k) behind a convolution is not served: qk_norm='head' goes with taps")
         if qk_norm not in ("joint", "head") or rot_pairs not in ("neighbours", "halves") or sink not in (None, "zero", "learned") \
-                or gate not in ("head", "channel"):
-            raise ValueError("qk_norm: joint | head; rot_pairs: neighbours | halves; sink: None | zero | learned; gate: head | channel")
+                or gate not in (None, "head", "channel"):
+            raise ValueError("qk_norm: joint | head; rot_pairs: neighbours | halves; sink: None | zero | learned; "
+                             "gate: None | head | channel")
         self.width, self.n_heads, self.n_kv_heads, self.dim, self.vdim = width, n_heads, n_kv_heads, dim, vdim
         self.scale, self.eps, self.bias, self.taps, self.tied_values = float(scale), float(eps), bool(bias), int(taps), bool(tied_values)
         self.qk_norm, self.rot_dims, self.rot_pairs, self.softcap, self.chunk = qk_norm, int(rot_dims), rot_pairs, float(softcap), int(chunk)
-        self.sink, self.gate = sink, gate
+        self.sink, self.gate, self.slope, self.out_bias, self.result_scale = sink, gate, bool(slope), bool(out_bias), float(result_scale)
         self.head_cols = cache_head_cols(dim, vdim)
         self.channels = (n_heads + n_kv_heads) * dim
         self.value_cols = 0 if tied_values else n_kv_heads * vdim
-        self.gate_cols = n_heads if gate == "head" else n_heads * vdim
+        self.gate_cols = 0 if gate is None else n_heads if gate == "head" else n_heads * vdim
+        #: columns of what the output projection reads (without a gate, the heads as attention leaves them)
+        self.mixed_cols = n_heads * (self.head_cols if gate is None else vdim)
         self.position = Rotary(rot_dims, rot_base, rot_scaling) if rot_dims else None
         # (the pages of a run that has ended are given back: no later token reads them)
         self.cache_spec = CacheSpec(n_kv_heads, self.head_cols, RUNS if self.chunk else FULL, self.chunk)
         self.state_spec = StateSpec((self.taps - 1, self.channels), torch.float32, 0.0) if self.taps > 1 else None
-        self.w_in = self.wo = self.b_in = self.wconv = self.norm_q = self.norm_k = self.sinks = None
+        self.w_in = self.wo = self.b_in = self.b_out = self.wconv = self.norm_q = self.norm_k = self.sinks = self.slopes = None
 
     def tensor_specs(self) -> Dict[str, TensorSpec]:
         H, G, D, V = self.n_heads, self.n_kv_heads, self.dim, self.vdim
@@ -601,14 +609,27 @@ class GatedAttention(Mixer):
             specs["k.conv"] = TensorSpec((G * D, self.taps), kind="f32")
         if self.sink == "learned":
             specs["sink"] = TensorSpec((H,), kind="f32")
-        specs["g"] = TensorSpec((self.gate_cols, self.width))
+        if self.gate is not None:
+            specs["g"] = TensorSpec((self.gate_cols, self.width))
         specs["o"] = TensorSpec((self.width, H * V))
+        if self.out_bias:
+            specs["o.b"] = TensorSpec((self.width,), kind="f32")
         return specs
 
     def load(self, tensors):
-        parts = [tensors["q"], tensors["k"]] + ([] if self.tied_values else [tensors["v"]]) + [tensors["g"]]
+        parts = [tensors["q"], tensors["k"]] + ([] if self.tied_values else [tensors["v"]])
+        parts += [tensors["g"]] if self.gate is not None else []
         self.w_in = _stack_rows(parts, self.width)   # one product reads the mixer's input for all of them
         self.wo = tensors["o"].contiguous()
+        if self.gate is None and self.head_cols != self.vdim:   # heads of head_cols columns, those beyond vdim being zero
+            wo = torch.zeros((self.width, self.n_heads, self.head_cols), dtype=self.wo.dtype, device=self.wo.device)
+            wo[:, :, :self.vdim] = self.wo.view(self.width, self.n_heads, self.vdim)
+            self.wo = wo.view(self.width, self.mixed_cols)
+        if self.out_bias:
+            self.b_out = (tensors["o.b"].float() * self.result_scale).contiguous()
+        if self.slope:
+            self.slopes = torch.tensor([2.0 ** (-8.0 * (h + 1) / self.n_heads) for h in range(self.n_heads)], dtype=torch.float32,
+                                       device=self.wo.device)
         if self.bias:
             self.b_in = torch.cat([tensors["q.b"], tensors["k.b"]] + ([] if self.tied_values else [tensors["v.b"]])).float().contiguous()
         self.norm_q, self.norm_k = tensors["q.norm"].float().contiguous(), tensors["k.norm"].float().contiguous()
@@ -632,15 +653,30 @@ class GatedAttention(Mixer):
             out.append(("taps", f"{self.taps} is above {ops.CONV_MAX_TAPS}, the longest convolution the kernel takes"))
         return out
 
-    def forward(self, ctx, h, residual, cache: Optional[LayerCache], store: bool = False):
+    def forward(self, ctx, h, residual, cache: Optional[LayerCache], store: bool = False, hand_on_bias: bool = False):
         """Adds the mixed rows into ``residual``; with ``store`` writes them there instead (float32 either way) or leaves
-        them in slices, and returns what ``product_in_slices`` does."""
-        if cache is None or cache.k_pages is None or (self.taps > 1 and cache.state is None):
-            raise ValueError("GatedAttention needs a layer cache with pages (and state, with a convolution)")
+        them in slices, and returns what ``product_in_slices`` does (``hand_on_bias``: the output's bias, not yet added, as a
+        third entry)."""
         n = h.shape[0]
-        H, G, V, hc = self.n_heads, self.n_kv_heads, self.vdim, self.head_cols
         proj = ctx.buffer("gated_proj", (n, self.w_in.shape[0]), ctx.dtype)   # [q | k | v | gate]
         product(ctx, h, self.w_in, proj)
+        mixed = ctx.buffer("gated_rows", (n, self.mixed_cols), ctx.dtype)
+        self.mix(ctx, proj, mixed, cache)
+        if store and (self.b_out is None or hand_on_bias):   # the caller's pass over the rows adds the slices of a product that divides k
+            made = product_in_slices(ctx, mixed, self.wo, residual)
+            return made + (self.b_out,) if hand_on_bias else made
+        product(ctx, mixed, self.wo, residual, accumulate=not store)
+        if self.b_out is not None:
+            ops.add_bias(residual, self.b_out)
+        return (residual, 1) if store else None
+
+    def mix(self, ctx, proj, mixed, cache: Optional[LayerCache]) -> None:
+        """From the stacked projections (``w_in``) to the rows that the output projection (``wo``) reads; both may be columns
+        of wider rows."""
+        if cache is None or cache.k_pages is None or (self.taps > 1 and cache.state is None):
+            raise ValueError("GatedAttention needs a layer cache with pages (and state, with a convolution)")
+        n = proj.shape[0]
+        H, G, V, hc = self.n_heads, self.n_kv_heads, self.vdim, self.head_cols
         cos, sin = self.position.table(ctx) if self.position is not None else (None, None)
         heads = ctx.buffer("gated_heads", (n, (H + 2 * G) * hc), ctx.dtype)
         slots = ctx.slots[cache.group] if cache.writable else None
@@ -649,20 +685,16 @@ class GatedAttention(Mixer):
                      bias=self.b_in, wconv=self.wconv, state=cache.state if self.taps > 1 else None, cos=cos, sin=sin,
                      rot=self.rot_dims, magnitude=self.position.magnitude if self.position is not None else 1.0,
                      neighbours=self.rot_pairs == "neighbours", tied=self.tied_values, slots=slots if direct else None,
-                     k_pages=cache.k_pages, v_pages=cache.v_pages)
+                     k_pages=cache.k_pages, v_pages=cache.v_pages, value_scale=self.result_scale)
         if slots is not None and not direct:
             # many rows: the kernel that takes a step's keys and values to their pages in whole lines
             ops.rope_store(heads, None, None, slots, cache.k_pages, cache.v_pages, H, G, hc, rotate=False,
                            portions=ctx.portions())
-        att = ctx.buffer("att", (n, H * hc), ctx.dtype)
-        paged_attention(ctx, heads[:, :H * hc], att, cache, H, self.scale, 0, 0, self.chunk, self.softcap, self.sinks)
-        gated = ctx.buffer("gated_rows", (n, H * V), ctx.dtype)
-        at = self.channels + self.value_cols
-        ops.gate_rows(att, hc, proj[:, at:at + self.gate_cols], gated, H, V, self.gate == "head")
-        if store:   # the caller's pass over the rows adds the slices of a product that divides k
-            return product_in_slices(ctx, gated, self.wo, residual)
-        product(ctx, gated, self.wo, residual, accumulate=True)
-        return None
+        att = mixed if self.gate is None else ctx.buffer("att", (n, H * hc), ctx.dtype)
+        paged_attention(ctx, heads[:, :H * hc], att, cache, H, self.scale, 0, 0, self.chunk, self.softcap, self.sinks, self.slopes)
+        if self.gate is not None:
+            at = self.channels + self.value_cols
+            ops.gate_rows(att, hc, proj[:, at:at + self.gate_cols], mixed, H, V, self.gate == "head")
 
 
 class LatentCacheAttention(Mixer):

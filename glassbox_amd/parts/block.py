@@ -135,8 +135,8 @@ class OutputNormBlock(Block):
     x += norm2(feed-forward(x)); the
     feed-forward may be absent.  The sublayers read the residual itself (the mixer through ``conv``, which may add a short
     convolution of the residual over time and keeps the state that takes); each writes its rows into a 32-bit buffer
-    (``accepts_store``), and the norm's pass over them is the pass that adds them into the residual.  The norms are
-    ``ScalarRMSNorm``s (or anything with ``add_normed``)."""
+    (``accepts_store``), and the norm's pass over them is the pass that adds them into the residual (a mixer with
+    ``hands_on_bias`` leaves its output's bias to that pass too).  The norms are ``ScalarRMSNorm``s or ``RMSNorm``s with ``adds`` (or anything with ``add_normed``)."""
     replayable = True
     taped = True
 
@@ -177,18 +177,21 @@ class OutputNormBlock(Block):
         n, width = x.shape
         h = pre if pre is not None else self.conv.forward(ctx, x, cache)
         y = ctx.buffer("sublayer_y", (n, width), torch.float32)
-        # a sublayer's rows lie in y, or in slices that the norm's pass adds up (``product_in_slices``)
-        made, slices = self.mixer.forward(ctx, h, y, cache, store=True) or (y, 1)
+        # a sublayer's rows lie in y, or in slices that the norm's pass adds up (``product_in_slices``), perhaps less a bias
+        # that pass adds as well
+        more = {"hand_on_bias": True} if getattr(self.mixer, "hands_on_bias", False) else {}
+        made, slices, *bias = self.mixer.forward(ctx, h, y, cache, store=True, **more) or (y, 1)
+        bias = bias[0] if bias else None
         handed = ctx.buffer("h", (n, width), ctx.dtype) if emit is not None else None
         if self.ffn is None:
-            self.mixer_norm.add_normed(ctx, made, x, rounded=handed, slices=slices, conv=emit)
+            self.mixer_norm.add_normed(ctx, made, x, rounded=handed, slices=slices, conv=emit, bias=bias)
             return handed
         if ctx.dtype == torch.float32:
-            self.mixer_norm.add_normed(ctx, made, x, slices=slices)
+            self.mixer_norm.add_normed(ctx, made, x, slices=slices, bias=bias)
             rows = x
         else:   # the pass that makes the residual also leaves it in the activations' type for the feed-forward
             rows = ctx.buffer("h", (n, width), ctx.dtype)
-            self.mixer_norm.add_normed(ctx, made, x, rounded=rows, slices=slices)
+            self.mixer_norm.add_normed(ctx, made, x, rounded=rows, slices=slices, bias=bias)
         made, slices = self.ffn.forward(ctx, rows, y, store=True) or (y, 1)
         self.ffn_norm.add_normed(ctx, made, x, rounded=handed, slices=slices, conv=emit)
         return handed

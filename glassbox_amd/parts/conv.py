@@ -37,7 +37,9 @@ class TimeConv(Part):
     def entry_spec(self, ctx, n: int, cache: Optional[LayerCache]):
         """``(weight, state)`` for ``ops.norm_add(conv=)`` if the pass that adds a normed sublayer into the residual may
         make this convolution's rows as well (every request of the step brings one row), else None."""
-        if (not self.taps or int(ctx.host["max_q_len"]) != 1 or not ops.norm_add_takes_rows(self.width)
+        if not self.taps:
+            return (None, None)   # the rows are the new residual, whatever the step
+        if (int(ctx.host["max_q_len"]) != 1 or not ops.norm_add_takes_rows(self.width)
                 or (self.taps > 1 and (cache is None or cache.state is None))):
             return None
         return (self.weight, cache.state if self.taps > 1 else None)

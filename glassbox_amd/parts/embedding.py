@@ -56,15 +56,15 @@ class SinusoidEmbedding(Embedding):
 
 
 class PairHashEmbedding(Embedding):
-    """The token's row plus a row of a second table chosen by the token and the one before it:
+    """The token's row (times ``scale``) plus a row of a second table chosen by the token and the one before it:
     row (previous token * mul_prev + token * mul_cur) mod buckets, and the table's last row (number ``buckets``) for a
     request's first token.  The token before a step's first row is part of the request's state: one int32 a slot
     (``state_spec``), which the model hands over as a cache layer of the embedding's own."""
     replayable = True
 
     def __init__(self, vocab: int, width: int, buckets: int, mul_prev: int, mul_cur: int,
-                 names=("weight", "pairs")):
-        super().__init__(vocab, width)
+                 names=("weight", "pairs"), scale: float = 1.0):
+        super().__init__(vocab, width, scale)
         if buckets < 1:
             raise ValueError(f"{buckets} buckets: at least one")
         self.buckets, self.mul_prev, self.mul_cur = int(buckets), int(mul_prev), int(mul_cur)
@@ -83,15 +83,17 @@ class PairHashEmbedding(Embedding):
     def forward(self, ctx, out, cache: Optional[LayerCache] = None):
         if cache is None or cache.state is None:
             raise ValueError("PairHashEmbedding needs its state (the token before each request's step)")
-        ops.embed_pairs(self.table, self.pairs, ctx, out, self.buckets, self.mul_prev, self.mul_cur, cache.state)
+        ops.embed_pairs(self.table, self.pairs, ctx, out, self.buckets, self.mul_prev, self.mul_cur, cache.state, self.scale)
 
 
 class LMHead(Part):
-    """logits = rows . W^T (times ``scale``) in float32.  ``tied_to`` names an Embedding whose table is the head."""
+    """logits = rows . W^T (times ``scale``; with ``softcap`` then softcap * tanh(logits / softcap)) in float32.  ``tied_to`` names an Embedding whose table is the head."""
     replayable = True
 
-    def __init__(self, vocab: int, width: int, tied_to: Optional[Embedding] = None, scale: float = 1.0, any_size: bool = False):
+    def __init__(self, vocab: int, width: int, tied_to: Optional[Embedding] = None, scale: float = 1.0, any_size: bool = False,
+                 softcap: float = 0.0):
         self.vocab, self.width, self.tied_to, self.scale = vocab, width, tied_to, float(scale)
+        self.softcap = float(softcap)
         self.any_size = bool(any_size)   # a width that the bfloat16 product does not take goes through the plain product
         self.weight: Optional[torch.Tensor] = None
 
@@ -120,6 +122,8 @@ class LMHead(Part):
             product(ctx, rows, self.matrix(), logits)
         else:
             ops.gemm(rows, self.matrix(), logits, rms_parts=prepared.as_gemm_arg() if prepared is not None else None)
-        if self.scale != 1.0:
+        if self.softcap > 0:
+            ops.cap_rows(logits, self.softcap, self.scale)
+        elif self.scale != 1.0:
             ops.scale_rows(logits, self.scale)
         return logits

@@ -19,7 +19,9 @@ neighbours, and only experts of the ``keep`` runs whose best s + correction is l
 ``unit="relu2"`` (an expert is W_down relu(W_up h)^2: one matrix in, no gate half); ``shared_gate=False`` (the shared
 expert's result is added as it is); ``scoring="chosen"`` (the ``top`` largest of the logits themselves, with ``bias`` z = W_router
 h + ``router.b``, and the softmax over the chosen logits alone as weights); ``unit="clamped"`` (g = min(W_gate h, limit), u =
-clamp(W_up h, -limit, limit), y = W_down (g sigmoid(alpha g) (u + 1))).
+clamp(W_up h, -limit, limit), y = W_down (g sigmoid(alpha g) (u + 1))); ``weigh_in=True`` (the weight multiplies what an expert
+reads, not what it gives: the result is sum_e expert_e(a_e h); since gate and up are linear, their sums are multiplied by a_e
+before the unit).
 """
 from __future__ import annotations
 
@@ -39,7 +41,7 @@ class RoutedExperts(FeedForward):
     def __init__(self, width: int, n_experts: int, top: int, expert_ff: int, router_scale: float = 1.0,
                  shared_ff: int = 0, correction: bool = True, scoring: str = "sigmoid", renorm: bool = True,
                  groups=None, unit: str = "swiglu", shared_gate: bool = True, bias: bool = False, limit: Optional[float] = None,
-                 alpha: float = 1.702):
+                 alpha: float = 1.702, weigh_in: bool = False):
         if not 1 <= top <= n_experts:
             raise ValueError(f"{top} experts a token out of {n_experts}")
         if scoring not in ("sigmoid", "softmax", "chosen") or unit not in ("swiglu", "relu2", "clamped"):
@@ -48,6 +50,9 @@ class RoutedExperts(FeedForward):
             raise ValueError("a choice by the logits themselves has no correction and no groups, and its weights add up to the scale")
         if bias and scoring != "chosen":
             raise ValueError("a bias on the router's logits goes with the choice by them (scoring='chosen')")
+        if weigh_in and (shared_ff or unit == "relu2"):
+            raise ValueError("weights on the experts' input go with gated units and no shared expert")
+        self.weigh_in = bool(weigh_in)
         if unit == "clamped" and not (limit is not None and limit > 0):
             raise ValueError(f"clamped units need a positive limit, got {limit}")
         self.width, self.n_experts, self.top, self.expert_ff = width, int(n_experts), int(top), int(expert_ff)
@@ -120,6 +125,10 @@ class RoutedExperts(FeedForward):
         weights = ctx.buffer("moe_weights", (n, self.top), torch.float32)
         if self.scoring == "chosen" and not self.shared_ff and E <= ops.MOE_ROUTER_MAX_EXPERTS and ctx.tuned:
             ops.moe_router(h, self.w_router, self.correction, self.top, self.router_scale, combine, ids, weights)
+        elif (self.scoring == "sigmoid" and not self.renorm and not self.has_correction and self.groups is None and not self.shared_ff
+              and E <= ops.MOE_ROUTER_MAX_EXPERTS and ctx.tuned):
+            # (the largest sigmoids are the largest logits')
+            ops.moe_router(h, self.w_router, None, self.top, self.router_scale, combine, ids, weights, sigmoid=True)
         else:
             self._route(ctx, h, combine, ids, weights)
         if self.routed(ctx, n):
@@ -128,7 +137,7 @@ class RoutedExperts(FeedForward):
         product(ctx, h, self.w_gate_up, gate_up)
         act = ctx.buffer("act", (n, self.inter), ctx.dtype)
         if self.halves == 2:
-            ops.moe_gated_units(gate_up, combine, act, E, self.expert_ff, self.gate_unit)
+            ops.moe_gated_units(gate_up, combine, act, E, self.expert_ff, self.gate_unit, weigh_in=self.weigh_in)
         else:
             ops.moe_relu2_units(gate_up, combine, act, E, self.expert_ff)
         if store:   # the caller's pass over the rows adds the slices of a product that divides k
@@ -169,11 +178,12 @@ class RoutedExperts(FeedForward):
         rows = ctx.buffer("moe_rows", (entries,), torch.int32)
         pos = ctx.buffer("moe_pos", (n, top), torch.int32)
         tile_map = ctx.buffer("moe_tiles", (tiles, 3), torch.int32)
-        ops.moe_sort(ids, E, tile_rows, counts, rows, pos, tile_map)
+        row_weights = ctx.buffer("moe_row_weights", (entries,), torch.float32) if self.weigh_in else None
+        ops.moe_sort(ids, E, tile_rows, counts, rows, pos, tile_map, weights, row_weights)
         act = ctx.buffer("act", (entries, ff), torch.bfloat16)
         if self.halves == 2:
             ops.gemm_grouped(h, rows, self.w_gate_up, ff * self.w_gate_up.stride(0), 2 * ff, tile_map, tile_rows, act,
-                             silu_mul=True, up_offset=E * ff, unit=self.gate_unit)
+                             silu_mul=True, up_offset=E * ff, unit=self.gate_unit, in_scale=row_weights)
         else:   # the unit in a pass of its own over the experts' rows, in place
             ops.gemm_grouped(h, rows, self.w_gate_up, ff * self.w_gate_up.stride(0), ff, tile_map, tile_rows, act)
             ops.moe_relu2_units(act, None, act, 0, ff)
@@ -195,5 +205,5 @@ class RoutedExperts(FeedForward):
             w = self.w_down[:, E * ff:]
             ops.gemm(act_shared, w, y_shared, workspace=split_workspace(ctx, n, d, self.shared_ff))
             gates = combine[:, E]
-        ops.moe_combine(y, pos, weights, y_shared, gates, residual, accumulate=not store)
+        ops.moe_combine(y, pos, None if self.weigh_in else weights, y_shared, gates, residual, accumulate=not store)
         return None

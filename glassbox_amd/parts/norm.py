@@ -1,6 +1,7 @@
 """RMS norm: out = g * (x / sqrt(mean(x^2) + eps)), sums in 32-bit
 (crates/glassbox-core/src/model.rs:94-100).  With ``offset`` the checkpoint holds the weight minus ``offset`` and
-g = offset + w, added in 32-bit when the weights are loaded and kept in 32-bit.  ``ScalarRMSNorm`` has one number for all
+g = offset + w, added in 32-bit when the weights are loaded and kept in 32-bit; with ``adds`` the weight is kept in 32-bit and the
+norm can also be taken of a sublayer's *output* on its way into the residual.  ``ScalarRMSNorm`` has one number for all
 coordinates and can also norm a sublayer's *output* on its way into the residual.  ``TanhNorm`` computes no statistic
 of the row at all: out = tanh(alpha x) * w + b with one number alpha.  ``GroupRMSNorm`` cuts the row into equal runs of
 channels and divides each by its own root mean square."""
@@ -18,8 +19,9 @@ class RMSNorm(Norm):
     replayable = True
     taped = True
 
-    def __init__(self, width: int, eps: float, offset: float = 0.0):
+    def __init__(self, width: int, eps: float, offset: float = 0.0, adds: bool = False):
         self.width = width
+        self.adds = bool(adds)
         self.eps = float(eps)
         self.offset = float(offset)
         self.weight: Optional[torch.Tensor] = None
@@ -28,7 +30,11 @@ class RMSNorm(Norm):
         if self.offset:
             # (offset + w rounded to bfloat16 would lose most of w: the sum stays 32-bit)
             return {"weight": TensorSpec((self.width,), kind="f32", init="zeros")}
-        return {"weight": TensorSpec((self.width,), kind="vector", init="ones")}
+        return {"weight": TensorSpec((self.width,), kind="f32" if self.adds else "vector", init="ones")}
+
+    def add_normed(self, ctx, y, x, rounded=None, slices: int = 1, conv=None, bias=None) -> None:
+        """x += g * (y + bias) / sqrt(mean((y + bias)^2) + eps), as ``ScalarRMSNorm.add_normed``."""
+        ops.norm_add(x, y, self.weight, self.eps, rounded, slices=slices, conv=conv, ctx=ctx, bias=bias)
 
     def load(self, tensors):
         w = tensors["weight"]
@@ -80,10 +86,11 @@ class ScalarRMSNorm(Norm):
         ops.rmsnorm(x, self.weight, self.eps, out, rows)
         return out
 
-    def add_normed(self, ctx, y, x, rounded=None, slices: int = 1, conv=None) -> None:
-        """x += g * y / sqrt(mean(y^2) + eps) (both float32; ``slices`` > 1: y is the sum of that many pieces);
+    def add_normed(self, ctx, y, x, rounded=None, slices: int = 1, conv=None, bias=None) -> None:
+        """x += g * y / sqrt(mean(y^2) + eps) (both float32; ``slices`` > 1: y is the sum of that many pieces; ``bias``: one
+        number a column that is added to y first);
         ``rounded`` receives the new x in its own type, or with ``conv=(weight, state)`` what a ``TimeConv`` makes of it."""
-        ops.norm_add(x, y, self.gain, self.eps, rounded, slices=slices, conv=conv, ctx=ctx)
+        ops.norm_add(x, y, self.gain, self.eps, rounded, slices=slices, conv=conv, ctx=ctx, bias=bias)
 
 
 class TanhNorm(Norm):
