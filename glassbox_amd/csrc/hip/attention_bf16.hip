@@ -58,6 +58,10 @@ struct Extra {
 };
 enum : int { kPlainScores = 0, kCapped = 1, kSloped = 2 };
 
+// Decoding over runs of positions: the chunks a request's workgroups take are counted from its run's first tile of 64 keys
+// (whose keys before the run are masked), so that a launch holds the chunks of one run and not of the whole context.
+__device__ __forceinline__ int chunks_from(int lo, int span) { return span > 0 ? lo & ~63 : 0; }
+
 __device__ __forceinline__ int first_key(int pos, int window, int span) {
   return span > 0 ? pos - pos % span : window > 0 ? max(0, pos - window + 1) : 0;
 }
@@ -213,7 +217,7 @@ __global__ __launch_bounds__(WAVES * 64) void decode_kernel(const bf16* __restri
   float* sm_acc = sm_l + WAVES * 16;      // [WAVES][HD][G]
   const int pos = positions[s];
   const int lo = first_key(pos, window, ex.span);
-  const int c0 = split * chunk;
+  const int c0 = chunks_from(lo, ex.span) + split * chunk;
   const int kept = min(keep, lo);            // keys 0 .. kept-1 are read although the window has passed them
   if (c0 > pos || (c0 + chunk <= lo && c0 >= kept)) return;  // this chunk holds no key of the request
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -298,7 +302,7 @@ __global__ __launch_bounds__(256) void decode_reduce_kernel(const float* __restr
   const int pos = positions[s];
   const int lo = first_key(pos, window, ex.span);
   // the chunks that hold keys: those of the kept first keys that lie before the window's first chunk, then the window's
-  const int first = lo / chunk, last = pos / chunk;
+  const int base = chunks_from(lo, ex.span), first = (lo - base) / chunk, last = (pos - base) / chunk;
   const int early_chunks = min((min(keep, lo) + chunk - 1) / chunk, first);
   const int count = early_chunks + last - first + 1;  // at most 256 chunks hold keys
   const size_t base0 = ((size_t)s * nh + head) * splits;
@@ -873,6 +877,7 @@ static int decode_launch(const void* q, int q_stride, OT* out, int out_stride, v
   GB_REQUIRE(q_stride % 8 == 0 && ((uintptr_t)q % 16 == 0) && out_stride % 4 == 0, "attention_decode: q rows must be 16-byte aligned");
   GB_REQUIRE(n_decode <= 65535 && nkv <= 65535, "attention_decode: too many requests or kv heads for one launch");
   if (n_decode == 0) return 0;
+  // (with runs max_context may be the most keys of a run's tiles, rather than the longest context)
   const int splits = (max_context + chunk - 1) / chunk;
   // one workgroup per request and kv head (no chunks to combine afterwards) gets 16 waves, so that as
   // many loads are in flight as with four workgroups of four

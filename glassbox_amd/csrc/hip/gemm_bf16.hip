@@ -151,6 +151,8 @@ __global__ __launch_bounds__(256, WN == 2 ? 2 : 1) void gemm_tiled_kernel(const 
   }
   __shared__ __attribute__((aligned(16))) bf16 As[2][BM][TLD];
   __shared__ __attribute__((aligned(16))) bf16 Ws[2][BN][TLD];
+  constexpr bool SCALES = GROUPED && EPI == EPI_SILU_MUL;
+  __shared__ float in_scale[SCALES ? BM : 1];   // the rows' factors (read behind the loop's barriers)
   const int tid = threadIdx.x, lane = tid % 64, wave = tid / 64;
   const int wm = wave / 2, wn = wave % 2;
   int m0 = blockIdx.y * BM;
@@ -164,6 +166,7 @@ __global__ __launch_bounds__(256, WN == 2 ? 2 : 1) void gemm_tiled_kernel(const 
     M = tile[2];
     w += (size_t)group * grp.w_stride;
     up_off = grp.up_off;
+    if (SCALES && grp.in_scale && tid < BM) in_scale[tid] = grp.in_scale[min(m0 + tid, M - 1)];
   }
   // row of W behind row r of the workgroup's W tile (r = wn*32*WN + j*32 + column)
   auto w_row = [&](int r) -> int {
@@ -306,14 +309,15 @@ __global__ __launch_bounds__(256, WN == 2 ? 2 : 1) void gemm_tiled_kernel(const 
   if (EPI == EPI_SILU_MUL) {
     const int gn = blockIdx.x * 64 + wn * 32 + lane % 32;
     if (gn >= half) return;
+    const bool scaled = SCALES && grp.in_scale;
 #pragma unroll
     for (int i = 0; i < WM; ++i)
 #pragma unroll
       for (int r = 0; r < 16; ++r) {
         const int gm = m0 + wm * 32 * WM + i * 32 + 8 * (r / 4) + 4 * (lane / 32) + r % 4;
         float g = acc[i][0][r], u = acc[i][WN - 1][r];
-        if (GROUPED && grp.in_scale) {
-          const float s = grp.in_scale[min(gm, M - 1)];
+        if (SCALES && scaled) {
+          const float s = in_scale[wm * 32 * WM + i * 32 + 8 * (r / 4) + 4 * (lane / 32) + r % 4];
           g *= s, u *= s;
         }
         if (gm < M) c[(size_t)gm * ldc + gn] = (CT)gated_unit(g, u, glu);
@@ -475,6 +479,8 @@ __global__ __launch_bounds__(RGM * RGN * 64, 1) void gemm_ring_kernel(const bf16
   }
   __shared__ __attribute__((aligned(16))) bf16 As[RING_STAGES][RBM * RBK];
   __shared__ __attribute__((aligned(16))) bf16 Ws[RING_STAGES][RBN * RBK];
+  constexpr bool SCALES = GROUPED && EPI == EPI_SILU_MUL;
+  __shared__ float in_scale[SCALES ? RBM : 1];   // the rows' factors (read behind the loop's barriers)
   const int tid = threadIdx.x, lane = tid % 64, wave = tid / 64;
   const int wm = wave / RGN, wn = wave % RGN;
   int m0 = by * RBM;
@@ -488,6 +494,7 @@ __global__ __launch_bounds__(RGM * RGN * 64, 1) void gemm_ring_kernel(const bf16
     M = tile[2];
     w += (size_t)group * grp.w_stride;
     up_off = grp.up_off;
+    if (SCALES && grp.in_scale && tid < RBM) in_scale[tid] = grp.in_scale[min(m0 + tid, M - 1)];
   }
   // row of W behind row r of the workgroup's W tile (r = wn * 64 + j * 32 + column); with EPI_SILU_MUL a wave's
   // first column tile holds gate rows and its second the up rows that belong to them
@@ -620,22 +627,24 @@ __global__ __launch_bounds__(RGM * RGN * 64, 1) void gemm_ring_kernel(const bf16
 
   // accumulator layout of a 32x32 tile: lane holds column lane%32, rows 8*(r/4) + 4*(lane/32) + r%4
   if (EPI == EPI_SILU_MUL) {
+    const bool scaled = SCALES && grp.in_scale;
 #pragma unroll
     for (int p = 0; p < RTN / 2; ++p) {
       const int gn = bx * (RBN / 2) + wn * (RTN / 2 * 32) + p * 32 + lane % 32;
       if (gn >= half) continue;
 #pragma unroll
-      for (int i = 0; i < RTM; ++i)
+      for (int i = 0; i < RTM; ++i) {
 #pragma unroll
         for (int r = 0; r < 16; ++r) {
           const int gm = m0 + wm * RTM * 32 + i * 32 + 8 * (r / 4) + 4 * (lane / 32) + r % 4;
           float g = acc[i][2 * p][r], u = acc[i][2 * p + 1][r];
-          if (GROUPED && grp.in_scale) {
-            const float s = grp.in_scale[min(gm, M - 1)];
+          if (SCALES && scaled) {
+            const float s = in_scale[wm * RTM * 32 + i * 32 + 8 * (r / 4) + 4 * (lane / 32) + r % 4];
             g *= s, u *= s;
           }
           if (gm < M) c[(size_t)gm * ldc + gn] = (CT)gated_unit(g, u, glu);
         }
+      }
     }
     return;
   }

@@ -365,9 +365,13 @@ __global__ __launch_bounds__(256) void place_kernel(const int32_t* __restrict__ 
   __syncthreads();
   const int base = first_row, mine = counts[e];
   int placed = 0;
+  int id = (int)threadIdx.x < entries ? ids[threadIdx.x] : -1;
   for (int i0 = 0; i0 < entries; i0 += 256) {
     const int i = i0 + threadIdx.x;
-    const bool hit = i < entries && ids[i] == e;
+    const bool hit = id == e;
+    const float wt = row_wts && i < entries ? wts[i] : 0.f;
+    if (i + 256 < entries) id = ids[i + 256];   // (the next round's are on their way)
+    else id = -1;
     const unsigned long long votes = __ballot(hit);
     const int before = __popcll(votes & ((1ull << lane) - 1ull));
     __syncthreads();   // the last round's sums have been read
@@ -379,7 +383,7 @@ __global__ __launch_bounds__(256) void place_kernel(const int32_t* __restrict__ 
       const int r = base + placed + ahead + before;
       rows[r] = i / top;
       pos[i] = r;
-      if (row_wts) row_wts[r] = wts[i];
+      if (row_wts) row_wts[r] = wt;
     }
     placed += part[0] + part[1] + part[2] + part[3];
   }

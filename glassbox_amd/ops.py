@@ -141,11 +141,15 @@ _SIGS = {
         # q32, k32, v, beta and log decays, stream
         "gb_delta_prep": [_vp, _i, _i, _i, _i, _i, _vp, _vp, _vp, _vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, C.c_longlong,
                           C.c_longlong, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _vp, _vp, _vp, _vp],
-        # q32, k32, v, dtype, beta and log decays, a decay a channel (0/1), out, tok_seq, q_start, q_len, pos0, state slots, state,
-        # floats a slot, where the ring lies, first row, rows, first request, requests, longest, H, G, dk, dv, workspace, its
-        # floats, stream
-        "gb_delta_rule": [_vp, _vp, _vp, _i, _vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp, C.c_longlong, C.c_longlong, _i, _i, _i,
-                          _i, _i, _i, _i, _i, _i, _vp, C.c_longlong, _vp],
+        # q32, k32, v, dtype, beta and log decays, a decay a channel (0/1), out, q_start, q_len, pos0, state slots, state, floats a
+        # slot, where the ring lies, first row, rows, first request, requests, H, G, dk, dv, stream
+        "gb_delta_scan": [_vp, _vp, _vp, _i, _vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, C.c_longlong, C.c_longlong, _i, _i, _i, _i,
+                          _i, _i, _i, _i, _vp],
+        # proj, dtype, ld, column of q k v, of beta, of the decay, conv w, rate, dt, z, ldz, q_start, q_len, pos0, state slots, state,
+        # floats a slot, where the ring lies, first row, rows, first request, requests, longest, H, G, dk, 16 dv + taps, gate, ldg,
+        # gate float32 | 2 sigmoid, norm w, eps, out, ldo, workspace, its floats, stream
+        "gb_delta_chunks": [_vp, _i, _i, _i, _i, _i, _vp, _vp, _vp, _vp, _i, _vp, _vp, _vp, _vp, _vp, C.c_longlong, C.c_longlong,
+                            _i, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _i, _i, _vp, _f, _vp, _i, _vp, C.c_longlong, _vp],
         # o, gate, ldg, gate float32 (0/1), sigmoid (0/1), norm w, eps, out, dtype, ldo, first row, rows, H, dv, stream
         "gb_delta_out": [_vp, _vp, _i, _i, _i, _vp, _f, _vp, _i, _i, _i, _i, _i, _i, _vp],
         # proj, dtype, ld, column of q k v, of beta, of the decay, conv w, rate, dt, z, ldz, q_start, pos0, state slots, state, floats
@@ -1796,6 +1800,8 @@ def attention_decode(q: torch.Tensor, out: torch.Tensor, ctx, cache, n_heads: in
     tables = ctx.tables[cache.group]
     max_context = int(ctx.host["max_context"])
     mask_chunk = int(chunk)   # the runs of positions a token sees; ``chunk`` below is the keys a workgroup takes
+    if mask_chunk:            # what is divided over workgroups is a run, from the tile of 64 keys that it begins in
+        max_context = min(max_context, mask_chunk + 63)
     chunk = decode_chunk(n_dec, nkv, max_context)
     splits = -(-max_context // chunk)
     ws_acc = ctx.buffer("attn_ws_acc", (n_dec * n_heads * splits * hd,), torch.float32)
@@ -2355,22 +2361,26 @@ def delta_rule(proj: torch.Tensor, at: int, b_at: int, a_at: int, wconv: torch.T
                 _rows(out, "out"), _stream())
     if alone >= S:
         return
+    longest, rows = int(ctx.host["max_q_len"]), n - alone
+    need = delta_chunk_floats(rows, S - alone, H, dk, dv) if ctx.tuned and longest >= DELTA_CHUNK_FROM else 0
+    if need:
+        ws = ctx.buffer("delta_chunks", (need,), torch.float32)
+        _launch(lib, lib.gb_delta_chunks, _p(proj), code, _rows(proj, "proj"), int(at), int(b_at), int(a_at), _p(wconv), _p(rate), _p(dt),
+                _p(z), ldz, _p(ctx.q_start), _p(ctx.q_len), _p(ctx.pos0), _p(ctx.state_slots), _p(state), floats, ring_at, alone, rows,
+                alone, S - alone, longest, H, G, dk, 16 * dv + taps, _p(gate), _rows(gate, "gate"), g32 | (2 if sigmoid_gate else 0),
+                _p(norm_weight), float(eps), _p(out), _rows(out, "out"), _p(ws), ws.numel(), _stream())
+        return
     q32 = ctx.buffer("delta_q", (n, G * dk), torch.float32)
     k32 = ctx.buffer("delta_k", (n, G * dk), torch.float32)
     v = ctx.buffer("delta_v", (n, H * dv), proj.dtype)
     beta_lg = ctx.buffer("delta_decay", (-(-n * H // 4) * 4 + n * H * (dk if z is not None else 1),), torch.float32)
     o = ctx.buffer("delta_o", (n, H * dv), torch.float32)
-    longest, rows = int(ctx.host["max_q_len"]), n - alone
     _launch(lib, lib.gb_delta_prep, _p(proj), code, _rows(proj, "proj"), int(at), int(b_at), int(a_at), _p(wconv), _p(rate), _p(dt), _p(z),
             ldz, _p(ctx.tok_seq), _p(ctx.q_start), _p(ctx.q_len), _p(ctx.pos0), _p(ctx.state_slots), _p(state), floats, ring_at,
             alone, rows, alone, S - alone, H, G, dk, 16 * dv + taps, _p(q32), _p(k32), _p(v), _p(beta_lg), _stream())
-    ws = None
-    if ctx.tuned and longest >= DELTA_CHUNK_FROM:
-        need = delta_chunk_floats(rows, S - alone, H, dk, dv)
-        ws = ctx.buffer("delta_chunks", (need,), torch.float32) if need else None
-    _launch(lib, lib.gb_delta_rule, _p(q32), _p(k32), _p(v), code, _p(beta_lg), 1 if z is not None else 0, _p(o), _p(ctx.tok_seq),
-            _p(ctx.q_start), _p(ctx.q_len), _p(ctx.pos0), _p(ctx.state_slots), _p(state), floats, ring_at, alone, rows, alone,
-            S - alone, longest, H, G, dk, dv, _p(ws), ws.numel() if ws is not None else 0, _stream())
+    _launch(lib, lib.gb_delta_scan, _p(q32), _p(k32), _p(v), code, _p(beta_lg), 1 if z is not None else 0, _p(o), _p(ctx.q_start),
+            _p(ctx.q_len), _p(ctx.pos0), _p(ctx.state_slots), _p(state), floats, ring_at, alone, rows, alone, S - alone, H, G, dk, dv,
+            _stream())
     _launch(lib, lib.gb_delta_out, _p(o), _p(gate), _rows(gate, "gate"), g32, 1 if sigmoid_gate else 0, _p(norm_weight), float(eps),
             _p(out), code, _rows(out, "out"), alone, rows, H, dv, _stream())
 
