@@ -975,6 +975,7 @@ GB_TAPED(gb_copy_rows)
 GB_TAPED(gb_qk_norm_store)
 GB_TAPED(gb_add_bias)
 GB_TAPED(gb_scale_rows)
+GB_TAPED(gb_cap_rows)
 GB_TAPED(gb_gemm_plain)
 GB_TAPED(gb_glu_clamped)
 GB_TAPED(gb_axpy_rows)

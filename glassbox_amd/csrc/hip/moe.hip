@@ -75,7 +75,8 @@ __global__ __launch_bounds__(4 * kWave) void route_kernel(const float* __restric
       s[j] = expf(c[j] - top_z);
     } else if (e < E) {
       s[j] = softmax ? expf(row[e] - top_z) / denom : 1.0f / (1.0f + expf(-row[e]));
-      c[j] = s[j] + (correction ? correction[e] : 0.f);
+      // (scores without a correction are chosen by their logits, whose order is the scores': sigmoids near 1 run together)
+      c[j] = correction ? s[j] + correction[e] : row[e];
     }
   }
   if (groups > 0) {

@@ -56,7 +56,8 @@ class SideBySide(Mixer):
         proj = ctx.buffer("side_proj", (n, self.w_in.shape[0]), ctx.dtype)
         product(ctx, h, self.w_in, proj)
         cols = self.left.mixed_cols
-        mixed = ctx.buffer("side_mixed", (n, self.wo.shape[1]), ctx.dtype)
+        both = self.wo.shape[1]
+        mixed = ctx.buffer("side_mixed", (n, -(-both // 8) * 8), ctx.dtype)[:, :both]   # (rows begin at 16-byte words)
         self.left.mix(ctx, proj[:, :self.left_rows], mixed[:, :cols], cache)
         self.right.mix(ctx, proj[:, self.left_rows:], mixed[:, cols:], cache)
         if store and (self.b_out is None or hand_on_bias):   # the caller's pass over the rows adds the slices

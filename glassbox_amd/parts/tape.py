@@ -39,7 +39,7 @@ import torch
 from .. import ops
 from .base import LayerCache, Part
 
-_SCALARS = (int, float, bool, str, type(None))
+_SCALARS = (int, float, bool, str, type(None), torch.dtype)
 
 
 def _constant(v):
@@ -212,14 +212,15 @@ class LayerTapes:
         rec = self.records.get(key)
         if rec is not None and rec.epoch == epoch:
             target = site.tensors(moved)
-            if target.sizes == rec.operands.sizes and rec.operands.maps_onto(target):
+            fits = lambda r: target.sizes == r.operands.sizes and r.operands.maps_onto(target)
+            if not fits(rec):
+                # a part of this layer has not made a tensor that the recorded layer's part made on its walk, or a tensor
+                # that the recorded layer held in two places is two tensors here: a kind by itself
+                key = (key, target.sizes)
+                rec = self.records.get(key)
+            if rec is not None and rec.epoch == epoch and fits(rec):
                 ops.run_tape(rec.tape, rec.operands, target)
                 return rec.result
-            # a part of this layer has not yet made a tensor that the recorded layer's part made on its walk, or a
-            # tensor that the recorded layer held in two places is two tensors here: the layer is walked
-            result = block.forward(ctx, x, cache, **kwargs)
-            site.forget()
-            return result
         # the first layer of its kind in this step (or a buffer of the step has grown since that one was recorded)
         memo = len(ctx.memo)
         tape = ops.start_tape()

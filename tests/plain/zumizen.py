@@ -7,8 +7,8 @@ Notation: T tokens at positions 0..T-1; H (query or value) heads, G key/value (o
 h // (H / G); dk key size, dv value size per head; a linear weight W is stored [out, in] and applied as x W^T.
 
 A layer:  x <- x + n1(mixer(x));  x <- x + n2(experts(x)), n1 and n2 RMS norms with a weight.
-``forward(..., coarse=True)`` rounds the activations to bfloat16 where a bfloat16 engine may: how far that moves a
-position's logits is the scale of the device tests' bfloat16 tolerance.
+``forward(..., coarse=k)`` rounds the activations to bfloat16 where a bfloat16 engine may, k = 1, 2, ... in so many ways: how far
+that moves a position's logits is the scale of the device tests' bfloat16 tolerance.
 """
 from __future__ import annotations
 
@@ -34,8 +34,10 @@ def exact(x: torch.Tensor) -> torch.Tensor:
     return x
 
 
-def bf16(x: torch.Tensor) -> torch.Tensor:
-    return x.to(torch.bfloat16).to(F64)
+def bf16(x: torch.Tensor, sample: int = 0) -> torch.Tensor:
+    """Rounded to bfloat16; with ``sample`` on a grid stretched by a few ten-thousandths, which rounds other values up."""
+    s = 1.0 + 0.00037 * sample
+    return (x * s).to(torch.bfloat16).to(F64) / s
 
 
 # ---------------------------------------------------------------------------------------------- embedding
@@ -217,10 +219,10 @@ def gated_unit(w, pre: str, x: torch.Tensor, rnd=exact) -> torch.Tensor:
 
 
 def route(z: torch.Tensor, top: int):
-    """z [T, E] -> (ids [T, top], weights [T, top]): the largest of sigmoid(z), as they stand."""
-    s = torch.sigmoid(z)
-    weights, ids = torch.topk(s, top, dim=-1)
-    return ids, weights
+    """z [T, E] -> (ids [T, top], weights [T, top]): the largest of sigmoid(z), as they stand (found by z, whose order is theirs:
+    far from zero sigmoids are one number in any precision)."""
+    z, ids = torch.topk(z, top, dim=-1)
+    return ids, torch.sigmoid(z)
 
 
 def route_margin(z: torch.Tensor, top: int) -> torch.Tensor:
@@ -253,11 +255,11 @@ def capped(z: torch.Tensor, cap: Optional[float]) -> torch.Tensor:
     return cap * torch.tanh(z / cap) if cap else z
 
 
-def forward(cfg: dict, w: Dict[str, torch.Tensor], tokens: List[int], coarse: bool = False,
+def forward(cfg: dict, w: Dict[str, torch.Tensor], tokens: List[int], coarse: int = 0,
             tap: Optional[list] = None, margins: Optional[list] = None) -> torch.Tensor:
     """Logits [T, vocab] of one whole sequence.  ``tap`` receives the residual after every layer, ``margins`` every
     router's ``route_margin``."""
-    rnd = bf16 if coarse else exact
+    rnd = (lambda t: bf16(t, coarse - 1)) if coarse else exact
     eps = cfg["norm"]["eps"]
     x = embed(cfg, w, tokens)
     for i, layer in enumerate(cfg["layers"]):
