@@ -56,7 +56,7 @@ struct Extra {
   const float* __restrict__ sinks;
   const float* __restrict__ slopes;
 };
-enum : int { kPlainScores = 0, kCapped = 1, kSloped = 2 };
+enum : int { kPlainScores = 0, kCapped = 1, kSloped = 2, kRuns = 3 };   // kRuns: plain scores over runs (decoding)
 
 // Decoding over runs of positions: the chunks a request's workgroups take are counted from its run's first tile of 64 keys
 // (whose keys before the run are masked), so that a launch holds the chunks of one run and not of the whole context.
@@ -216,8 +216,8 @@ __global__ __launch_bounds__(WAVES * 64) void decode_kernel(const bf16* __restri
   float* sm_l = sm_m + WAVES * 16;        // [WAVES][16]
   float* sm_acc = sm_l + WAVES * 16;      // [WAVES][HD][G]
   const int pos = positions[s];
-  const int lo = first_key(pos, window, ex.span);
-  const int c0 = chunks_from(lo, ex.span) + split * chunk;
+  const int lo = first_key(pos, window, MODE == kPlainScores ? 0 : ex.span);
+  const int c0 = (MODE == kPlainScores ? 0 : chunks_from(lo, ex.span)) + split * chunk;
   const int kept = min(keep, lo);            // keys 0 .. kept-1 are read although the window has passed them
   if (c0 > pos || (c0 + chunk <= lo && c0 >= kept)) return;  // this chunk holds no key of the request
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -910,10 +910,13 @@ static int decode_launch(const void* q, int q_stride, OT* out, int out_stride, v
         if (waves == 16) GB_DECODE(HD, 16, kSloped);                \
         else GB_DECODE(HD, 4, kSloped);                             \
       }                                                             \
+    } else if (ex.span > 0) {                                       \
+      if (waves == 16) GB_DECODE(HD, 16, kRuns);                    \
+      else GB_DECODE(HD, 4, kRuns);                                 \
     } else if (waves == 16) {                                       \
-      GB_DECODE(HD, 16, kPlainScores);                                   \
+      GB_DECODE(HD, 16, kPlainScores);                              \
     } else {                                                        \
-      GB_DECODE(HD, 4, kPlainScores);                                    \
+      GB_DECODE(HD, 4, kPlainScores);                               \
     }                                                               \
   }
   GB_FOR_HEAD_SIZES(GB_CASE)
