@@ -155,9 +155,10 @@ def zakusun_like(shapes: dict, layers: int, experts: int = 8, top: int = 2) -> d
                 canon={"taps": 4}, logit_scale=1.0, layers=[layer] * layers)
 
 
-def zumizen_like(shapes: dict, layers: int, run: int = 1024, experts: int = 8, top: int = 2) -> dict:
+def zumizen_like(shapes: dict, layers: int, run: int = 1536, experts: int = 8, top: int = 2) -> dict:
     """A Zumizen configuration with the widths of a Llama one: the two mixers in turn (side by side, attention and delta rule have
-    half of the heads each), routed experts in every layer with as many multiply-adds a token as the Llama's feed-forward."""
+    half of the heads each), routed experts in every layer with as many multiply-adds a token as the Llama's feed-forward.  (Behind
+    4,096 tokens a run of 1,536 positions holds 1,024.)"""
     d, H, G = shapes["hidden_size"], shapes["num_attention_heads"], shapes["num_key_value_heads"]
     hd = shapes.get("head_dim") or d // H
     half = lambda n: max(1, n // 2)
